@@ -611,6 +611,57 @@ pub struct NervaHipDeepSeekMoeForwardResult {
 
 #[repr(C)]
 #[derive(Copy, Clone)]
+pub struct NervaHipStackLayer {
+    pub mixer: u32,
+    pub heads: u32,
+    pub kv_heads: u32,
+    pub key_dim: u32,
+    pub value_dim: u32,
+    pub rotary_dims: u32,
+    pub rotary_base: f32,
+    pub score_scale: f32,
+    pub chunk_tokens: u32,
+    pub kv_layer: u32,
+    pub width: u32,
+    pub ff: u32,
+}
+
+#[repr(C)]
+#[derive(Copy, Clone)]
+pub struct NervaHipStackSessionCreateRequest {
+    pub dtype: u32,
+    pub precision: u32,
+    pub hidden: u32,
+    pub vocab_size: u32,
+    pub layer_count: u32,
+    pub max_context_tokens: u32,
+    pub norm_eps: f32,
+    pub layers: *const NervaHipStackLayer,
+    pub planned_weight_blocks: u32,
+    pub planned_gpu_resident_blocks: u32,
+    pub planned_gpu_staged_blocks: u32,
+    pub planned_weight_bytes: u64,
+    pub planned_gpu_resident_weight_bytes: u64,
+    pub planned_gpu_staged_weight_bytes: u64,
+    pub planned_weight_descriptors: *const NervaHipHfDecodeSequenceWeightBlock,
+    pub planned_weight_descriptor_count: u32,
+    pub planned_weight_descriptor_hash: u64,
+}
+
+#[repr(C)]
+#[derive(Copy, Clone)]
+pub struct NervaHipSessionExtendRequest {
+    pub session: *mut NervaHipHfDecodeSequenceSession,
+    pub tokens: *const u32,
+    pub token_count: u32,
+    pub wanted_count: u32,
+    pub wanted: *const u32,
+    pub logits: *mut f32,
+    pub residuals: *mut f32,
+}
+
+#[repr(C)]
+#[derive(Copy, Clone)]
 pub struct NervaHipGemvRequest {
     pub dtype: u32,
     pub rows: u32,
@@ -791,6 +842,10 @@ unsafe extern "C" {
     pub fn nerva_hip_deepseek_quant_fp8_f32_scale_encoded_gemm_tokens(request: *const NervaHipDeepSeekQuantFp8F32ScaleEncodedGemmTokensRequest, out: *mut NervaHipDeepSeekQuantDequantResult) -> c_int;
     pub fn nerva_hip_projection_bench(request: *const NervaHipProjectionBenchRequest, out: *mut NervaHipProjectionBenchResult) -> c_int;
     pub fn nerva_hip_deepseek_moe_forward(request: *const NervaHipDeepSeekMoeForwardRequest, out: *mut NervaHipDeepSeekMoeForwardResult) -> c_int;
+    pub fn nerva_hip_stack_session_create(request: *const NervaHipStackSessionCreateRequest, out: *mut NervaHipHfDecodeSequenceSessionCreateResult, session: *mut *mut NervaHipHfDecodeSequenceSession) -> c_int;
+    pub fn nerva_hip_bench_stack_session_create_synthetic(request: *const NervaHipStackSessionCreateRequest, seed: u64, weight_std: f32, out: *mut NervaHipHfDecodeSequenceSessionCreateResult, session: *mut *mut NervaHipHfDecodeSequenceSession) -> c_int;
+    pub fn nerva_hip_session_extend(request: *const NervaHipSessionExtendRequest, out: *mut NervaHipHfDecodeSequenceResult) -> c_int;
+    pub fn nerva_hip_session_release_sequence(session: *mut NervaHipHfDecodeSequenceSession) -> c_int;
     pub fn nerva_hip_gemv(request: *const NervaHipGemvRequest, stream: *mut c_void, hip_error: *mut i32) -> c_int;
     pub fn nerva_hip_gemv_launch_shape(prologue: u32, epilogue: u32, rows: u32, cols: u32, kernel: *mut u32, workgroups: *mut u32) -> c_int;
     pub fn nerva_hip_fp8_gemv(request: *const NervaHipFp8GemvRequest, stream: *mut c_void, hip_error: *mut i32) -> c_int;

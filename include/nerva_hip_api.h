@@ -444,6 +444,86 @@ int nerva_hip_deepseek_moe_forward(const NervaHipDeepSeekMoeForwardRequest *requ
                                    NervaHipDeepSeekMoeForwardResult *out);
 
 /* ------------------------------------------------------------------------
+ * Mixed layer stacks (no reference counterpart). A session whose layers are described one by one - kind of mixer,
+ * sizes, constants - instead of by one set of dimensions. It is created through its own call; everything after
+ * that (start / advance / run / extend / fork / batch_advance_one / destroy, the sampler, the token slots) is the
+ * session interface above.
+ *
+ * Every sublayer f sits between two layer norms (weight and bias): x <- x + N_post(f(N_pre(x))). A layer is a mixer,
+ * then - where ff != 0 - a feed-forward down(xielu(up(.))). Mixers:
+ *   ATTENTION  grouped-query attention; the heads' scores are mixed by a learned [heads][heads] matrix before the
+ *              softmax; the softmax has a learned sink per head in its denominator; the heads are gated by
+ *              sigmoid(gate(.)); rotation on the first rotary_dims of a head; with chunk_tokens != 0 a query sees its
+ *              own chunk of positions only; kv_layer names another layer whose keys and values are used
+ *              (NERVA_HIP_OWN_KEYS: its own).
+ *   MINGRU     gated recurrence of `width` channels with an f32 state (csrc/activations.cuh), gated by silu(gate(.)).
+ * The output is the final layer norm and the embedding matrix. Computed in f32 whatever the precision: norms, the
+ * residual, rotation, scores and weights, recurrence.
+ * ---------------------------------------------------------------------- */
+#define NERVA_HIP_MIXER_ATTENTION 1u
+#define NERVA_HIP_MIXER_MINGRU 2u
+#define NERVA_HIP_OWN_KEYS 4294967295u
+#define NERVA_HIP_PRECISION_16 0u /* 16-bit inputs of the matrix products, 16-bit keys and values */
+#define NERVA_HIP_PRECISION_32 1u /* f32 throughout (weights stay 16-bit values): a checking mode, not a fast one */
+
+typedef struct NervaHipStackLayer {
+  uint32_t mixer;                                  /* NERVA_HIP_MIXER_* */
+  uint32_t heads, kv_heads, key_dim, value_dim;    /* attention */
+  uint32_t rotary_dims;
+  float rotary_base, score_scale;
+  uint32_t chunk_tokens, kv_layer;
+  uint32_t width;                                  /* minGRU */
+  uint32_t ff;                                     /* feed-forward width, 0 = none */
+} NervaHipStackLayer;
+
+/* The weights come through a declared weight plan (NervaHipHfDecodeSequenceWeightBlock) over this order of 16-bit
+ * tensors: embedding; per layer norm1 w, b, norm1b w, b, [norm2 w, b, norm2b w, b], then attention: q, [k, v,] gate,
+ * mixing, sinks, o - or minGRU: z, x, gate, z bias, x bias, o - then [up, down, activation (2 numbers)]; final norm
+ * w, b. */
+typedef struct NervaHipStackSessionCreateRequest {
+  uint32_t dtype;      /* NERVA_HIP_DTYPE_BF16 */
+  uint32_t precision;  /* NERVA_HIP_PRECISION_* */
+  uint32_t hidden, vocab_size, layer_count, max_context_tokens;
+  float norm_eps;
+  const NervaHipStackLayer *layers;
+  uint32_t planned_weight_blocks, planned_gpu_resident_blocks, planned_gpu_staged_blocks;
+  uint64_t planned_weight_bytes, planned_gpu_resident_weight_bytes, planned_gpu_staged_weight_bytes;
+  const NervaHipHfDecodeSequenceWeightBlock *planned_weight_descriptors;
+  uint32_t planned_weight_descriptor_count;
+  uint64_t planned_weight_descriptor_hash;
+} NervaHipStackSessionCreateRequest;
+
+int nerva_hip_stack_session_create(const NervaHipStackSessionCreateRequest *request,
+                                   NervaHipHfDecodeSequenceSessionCreateResult *out,
+                                   NervaHipHfDecodeSequenceSession **session);
+/* The same with weights generated on the device (benchmarks): matrices N(0, weight_std), norm weights
+ * 1 + N(0, weight_std), the mixing matrix the identity plus N(0, weight_std). */
+int nerva_hip_bench_stack_session_create_synthetic(const NervaHipStackSessionCreateRequest *request, uint64_t seed,
+                                                   float weight_std,
+                                                   NervaHipHfDecodeSequenceSessionCreateResult *out,
+                                                   NervaHipHfDecodeSequenceSession **session);
+
+/* Appends given tokens to a session's sequence (or begins one, on a session without): they take the positions from
+ * the sequence's end on, and nothing before them is computed again. One token runs through the captured decode step,
+ * more through prompt blocks. Afterwards the sequence stands as if it had been started with all its tokens so far as
+ * the prompt: advance() hands out the token sampled after the last one (a sequence begun here samples greedily).
+ * Tokens that advance() has handed out count as part of the sequence, except the newest one, which has not run yet:
+ * a caller that goes on from it passes it first. logits: host [wanted_count][vocab_size] f32, the logits at the
+ * places wanted[] (ascending indices into tokens). */
+typedef struct NervaHipSessionExtendRequest {
+  NervaHipHfDecodeSequenceSession *session;
+  const uint32_t *tokens;
+  uint32_t token_count, wanted_count;
+  const uint32_t *wanted;
+  float *logits;
+  /* test hook, mixed stacks only: host [layer_count][token_count][hidden] f32, the residual rows after every layer */
+  float *residuals;
+} NervaHipSessionExtendRequest;
+int nerva_hip_session_extend(const NervaHipSessionExtendRequest *request, NervaHipHfDecodeSequenceResult *out);
+/* Ends the session's sequence: its cache and state are free for the next one. */
+int nerva_hip_session_release_sequence(NervaHipHfDecodeSequenceSession *session);
+
+/* ------------------------------------------------------------------------
  * Device-pointer operator entry points. The reference exposes these kernels
  * only inside its session (native/cuda/hf_decode_sequence/session_decode_prefill.inc.cu:74-372);
  * they are exported here so each one can be checked and timed on its own.

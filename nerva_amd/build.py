@@ -15,7 +15,8 @@ OBJ = os.path.join(CSRC, "build")
 LIB = os.path.join(HERE, "libnerva_hip.so")
 
 SOURCES = ["gemv_stream.hip", "fp8_gemv.hip", "attn_decode.hip", "attn_prompt.hip", "argmax.hip", "synth_fill.hip",
-           "sampler.hip", "gemm_rows.hip", "gemm_block.hip", "op_entry.hip", "decode_session.hip"]
+           "sampler.hip", "gemm_rows.hip", "gemm_block.hip", "gemm_any.hip", "norm_join.hip", "mingru.hip", "attn_mixed.hip",
+           "op_entry.hip", "decode_session.hip", "layer_stack.hip"]
 
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function",
          # packed fp32 VALU ops are kept off for every device function of this library
@@ -74,10 +75,12 @@ def build(verbose=False):
     for obj, log in results:
         if verbose and log.strip():
             print(log)
-    cmd = [hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB] + [o for o, _ in results]
+    part = "%s.%d.part" % (LIB, os.getpid())   # never a half-written library under the final name
+    cmd = [hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-o", part] + [o for o, _ in results]
     res = subprocess.run(cmd, capture_output=True, text=True)
     if res.returncode != 0:
         raise RuntimeError("link failed:\n" + res.stdout + res.stderr)
+    os.replace(part, LIB)
     return LIB
 
 

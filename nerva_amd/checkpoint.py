@@ -6,8 +6,8 @@ The reference's runtime does this in three steps: `config.json` -> model metadat
 manifest/names.rs:31-90), manifest x safetensors headers -> one file-backed descriptor per tensor
 (crates/nerva-model/src/weights/safetensors/{header,tensor,validation,shard}.rs,
 crates/nerva-runtime/src/engine/hf_cuda_decode/file_backed/descriptors.rs:442-521). This module is the
-same pipeline for the dense decoder families the session runs (Llama, Mistral, Qwen2, Qwen3): nothing of
-the checkpoint is read into host memory here except the headers; the session copies every tensor from
+same pipeline for the dense decoder families the session runs (Llama, Mistral, Qwen2, Qwen3) and for the mixed
+layer stacks of stacks.py (their `config.json` names an `architecture` and lists its layers): nothing of the checkpoint is read into host memory here except the headers; the session copies every tensor from
 its file range straight into the device arena.
 """
 import ctypes as C
@@ -15,7 +15,7 @@ import json
 import os
 import struct
 
-from . import abi
+from . import abi, stacks
 from .session import (WEIGHT_STRATEGY_GPU_RESIDENT, WEIGHT_STRATEGY_GPU_STAGED, DecodeSession, WeightPlan)
 
 _DTYPES = {"float16": (0, "F16"), "bfloat16": (1, "BF16")}          # request dtype code, safetensors name
@@ -23,13 +23,17 @@ _DENSE = {"llama": False, "mistral": False, "qwen2": False, "qwen3": True}  # mo
 _MAX_HEADER = 100 * 1000 * 1000                                       # the format's own bound on header bytes
 
 
-class CheckpointError(ValueError):
-    pass
+CheckpointError = stacks.CheckpointError
 
 
 def parse_config(config):
     """Model dimensions and optional-tensor flags of a dense decoder from its `config.json`
-    (hf/parser.rs:30-110; bias rule :464-479, q/k-norm rule :481-499)."""
+    (hf/parser.rs:30-110; bias rule :464-479, q/k-norm rule :481-499). A mixed stack gives
+    {"stack": stacks.StackConfig, ...} instead."""
+    if config.get("architecture") in stacks.READERS:
+        stack = stacks.READERS[config["architecture"]](config)
+        return dict(model_type=config["architecture"], dtype=_DTYPES["bfloat16"][0], st_dtype="BF16", stack=stack,
+                    vocab=stack.vocab, hidden=stack.hidden, layers=len(stack.layers))
     text = config.get("text_config", config)
     kind = (text.get("model_type") or config.get("model_type") or "").lower()
     if kind not in _DENSE:
@@ -62,6 +66,8 @@ def tensor_manifest(cfg):
     """(name, shape) of every tensor in the order of the weight arena: embeddings, per layer
     norm / q / q_norm / k / k_norm / v / o / mlp norm / gate / up / down / biases, final norm, LM head
     (layout/plan/layer_blocks.rs:9-49, weights.cu:484-591). A tied LM head is the embedding tensor again."""
+    if "stack" in cfg:
+        return cfg["stack"].manifest()
     H, A, KV, I = cfg["hidden"], cfg["heads"] * cfg["head_dim"], cfg["kv_heads"] * cfg["head_dim"], cfg["intermediate"]
     out = [("model.embed_tokens.weight", [cfg["vocab"], H])]
     for l in range(cfg["layers"]):
@@ -204,11 +210,16 @@ def marker_layers(cfg):
     return layers
 
 
-def create_session(directory, max_context, resident_bytes=None, **extra):
+def create_session(directory, max_context, resident_bytes=None, precision=stacks.PRECISION_16, **extra):
     """A decode session whose weights come from the checkpoint's files through a declared weight plan.
-    Returns (session, plan); the plan must outlive the create call only."""
+    Returns (session, plan); the plan must outlive the create call only. `precision`: of a mixed stack's
+    session (the dense families have the 16-bit one only)."""
     plan = plan_checkpoint(directory, resident_bytes)
     cfg = plan.cfg
+    if "stack" in cfg:
+        return DecodeSession.create_stack(cfg["stack"], plan, max_context, precision, **extra), plan
+    if precision != stacks.PRECISION_16:
+        raise CheckpointError("%s sessions compute in 16-bit precision only" % cfg["model_type"])
     lib = abi.load()
     req = abi.NervaHipHfDecodeSequenceSessionCreateRequest()
     req.dtype, req.hidden, req.heads, req.kv_heads = cfg["dtype"], cfg["hidden"], cfg["heads"], cfg["kv_heads"]

@@ -26,44 +26,14 @@
 #include <atomic>
 #include <vector>
 
-#include "argmax.cuh"
-#include "attn_decode.cuh"
-#include "gemm_rows.cuh"
-#include "sampler.cuh"
-#include "gemv_stream.cuh"
-#include "runtime_state.hpp"
+#include "layer_stack.hpp"
+#include "session.hpp"
 #include "synth_fill.cuh"
+#include "weight_plan.hpp"
 
 using namespace nv;
 
 namespace {
-
-using Slot = NervaHipSyntheticTokenSlot;
-
-struct LayerDev {
-  const uint16_t *rms_attn, *rms_mlp, *wqkv, *q_norm, *k_norm, *q_bias, *k_bias, *v_bias, *wo, *o_bias,
-      *wgu, *wdown;
-};
-
-enum StepMode { kDecodeStep = 0, kPromptStep = 1, kPromptHeadStep = 2 };
-enum LaunchKind { kLEmbed = 0, kLQkv, kLAttn, kLO, kLGateUp, kLDown, kLHead, kLAdvance, kLKinds };
-
-// The weight arena of a session and of every session forked from it (one stream of the weights can
-// then serve a token row of each of them); freed by the last of them to go.
-struct SharedWeights {
-  char *origin = nullptr;  // what the allocator returned (and takes back)
-  char *base = nullptr;    // the first kMatrixAlign boundary in it: offsets of the weight layout count from here
-  uint64_t bytes = 0;
-  std::atomic<uint32_t> refs{1};
-};
-
-// What a batch step needs to know of each of its sequences, in device memory: the cache and position
-// for the attention launches, the token slots for the embedding.
-struct BatchTable {
-  AttnSeq seq[kGemmMaxTokens];
-  const Slot *slots[kGemmMaxTokens];
-  SamplerParams sample[kGemmMaxTokens];
-};
 
 struct StepProfiler {
   hipStream_t stream;
@@ -93,80 +63,6 @@ struct StepProfiler {
 };
 
 }  // namespace
-
-struct NervaHipHfDecodeSequenceSession {
-  uint32_t dtype = 0, hidden = 0, heads = 0, kv_heads = 0, head_dim = 0, intermediate = 0, vocab = 0,
-           layers = 0, max_ctx = 0;
-  float eps = 0.0f, theta = 0.0f;
-  hipStream_t stream = nullptr;
-  SharedWeights *weights = nullptr;  // shared with forks
-  char *arena = nullptr;             // everything but the weights: KV cache, sequence state, activations, workspaces
-  uint32_t pair_gap = 0;             // elements between a layer's gate rows and its up rows (see kPairGapElems)
-  bool arena_in_weights = false;     // `arena` lies behind the weights in their allocation (the creating session)
-  uint64_t state_bytes = 0;          // size of `arena`
-  uint64_t arena_bytes = 0;          // weights + state, as reported to the caller
-  char *pinned = nullptr;
-  uint64_t pinned_bytes = 0;
-  std::vector<LayerDev> layer;
-  const uint16_t *emb = nullptr, *final_norm = nullptr, *lm_head = nullptr;
-  uint16_t *kc = nullptr, *vc = nullptr;
-  uint32_t block_count = 0;
-  uint32_t *table = nullptr, *prompt = nullptr;
-  uint32_t *state = nullptr;  // state[0] cursor, state[1] prompt count, state[2] steps executed so far,
-                              // state[3] fault word (set by a kernel whose bounded wait gave up; cleared by start)
-  Slot *slots = nullptr;
-  float *x = nullptr, *r = nullptr, *qkv = nullptr, *logits = nullptr, *rope_freq = nullptr, *rope_cs = nullptr;
-  uint16_t *attn16 = nullptr, *ff16 = nullptr;
-  void *attn_ws = nullptr, *sample_ws = nullptr;
-  uint32_t attn_splits = 1;
-  uint32_t attn_single_blocks = 0;   // contexts of up to this many blocks go to one split (0 with a forced split factor)
-  uint64_t *attn_tagged = nullptr;   // tagged split partials of the decode step kernel
-  uint32_t *attn_plan = nullptr;     // this step's split plan of the decode attention (attn_plan_fill), or null
-  uint64_t *attn_trace = nullptr;  // NERVA_HIP_ATTN_TRACE=1: per-layer stage timestamps of selected attention workgroups
-  Slot *host_slots = nullptr;
-  uint32_t *host_prompt = nullptr;
-  uint32_t *host_state = nullptr;
-  // captured steps: 0 decode step with the greedy finish, 1 prompt step, 2 decode step with the
-  // temperature / top-k / top-p sampler (its parameters live in device memory, so one capture
-  // serves every such configuration)
-  hipGraph_t graph[3] = {nullptr, nullptr, nullptr};
-  hipGraphExec_t exec[3] = {nullptr, nullptr, nullptr};
-  uint64_t graph_nodes[3] = {0, 0, 0};
-  // prompt blocks: up to prefill_block_tokens prompt tokens per pass through the layers (weights streamed
-  // once per block on the matrix cores); false = one prompt step per token
-  bool block_prefill = false;
-  // the multi-row kernels take this model's shapes (prompt blocks and batch steps need it)
-  bool rows_ready = false;
-  float *blogits = nullptr;          // [NERVA_HIP_BATCH_MAX_BLOCK_TOKENS][vocab] logits of a batch step
-  BatchTable *btable = nullptr, *host_btable = nullptr;
-  Slot *bslots = nullptr, *host_bslots = nullptr;   // a batch step's published slots, gathered for one copy
-  float *px = nullptr, *pr = nullptr, *pqkv = nullptr, *prope = nullptr;
-  uint16_t *pxn16 = nullptr, *pattn16 = nullptr, *pff16 = nullptr;
-  char *pattn_ws = nullptr;
-  uint64_t pattn_ws_stride = 0;
-  char *pgemm_ws = nullptr;        // partial sums of the K-sliced projections of a prompt block
-  uint64_t pgemm_ws_bytes = 0;
-  uint32_t prefill_block_tokens = kGemmMaxTokens;   // tokens per prompt block: 512 or 256 where every projection has the kernel for it
-  SamplerDev sampler{};            // normalised configuration of the active sequence
-  SamplerDev *sampler_dev = nullptr;
-  uint64_t *sampler_keys = nullptr;
-  hipEvent_t ev0 = nullptr, ev1 = nullptr;
-  // test hook: the next decode step is launched kernel by kernel and every intermediate vector is
-  // copied behind the previous one into this caller-owned device buffer (step_trace_bytes)
-  char *trace_buf = nullptr;
-  uint64_t trace_used = 0;
-  // echo of the caller's weight plan
-  uint32_t planned_weight_blocks = 0, planned_gpu_resident_blocks = 0, planned_gpu_staged_blocks = 0,
-           planned_weight_descriptor_count = 0;
-  uint64_t planned_weight_bytes = 0, planned_gpu_resident_weight_bytes = 0,
-           planned_gpu_staged_weight_bytes = 0, planned_weight_descriptor_hash = 0;
-  uint64_t resident_weight_bytes = 0, kv_bytes = 0;
-  // active sequence
-  bool started = false, finished = false;
-  uint32_t prompt_count = 0, observed = 0, cursor = 0, seed_token = 0, has_eos = 0, eos = 0;
-};
-
-using Session = NervaHipHfDecodeSequenceSession;
 
 namespace {
 
@@ -278,20 +174,6 @@ __global__ void advance_cursor_kernel(uint32_t *state, uint32_t max_steps) {
   if (threadIdx.x == 0 && blockIdx.x == 0 && state[0] < max_steps) state[0] = state[0] + 1u;
 }
 
-struct Carver {
-  uint64_t offset = 0;
-  uint64_t take(uint64_t bytes, uint64_t align = 256) {
-    const uint64_t at = (offset + align - 1) & ~(align - 1);
-    offset = at + ((bytes + 255u) & ~uint64_t{255});
-    return at;
-  }
-};
-// Weight matrices start on 8 MiB boundaries of device memory (the arena's first such boundary is its origin for
-// the weight layout). What the gate/up launch costs depends on its matrix's address modulo 8 MiB - the up rows lie
-// a fixed 96 MiB behind the gate rows, and the memory channels are chosen by a hash that reaches up to those bits:
-// with the rotated walk 31.0 us at 0 modulo 8 MiB, 31.4 at 2 and 6 MiB, 31.8 at 4 MiB, 32.1 at an odd KiB (the
-// plain walk: 33.0 / 31.7 / 31.3 / 31.8 / 31.7). At most 8 MiB a matrix is left unused: under 1.2 GB for 36 layers.
-constexpr uint64_t kMatrixAlign = 8u << 20;
 // The up rows of a layer start 4 KiB behind the end of its gate rows (large matrices only), so that gate row i
 // and up row i - which one wave of the decode step's gate/up launch streams side by side - lie half a row apart
 // in the memory channels' interleave instead of exactly on top of each other. With the rotated walk the launch
@@ -323,7 +205,9 @@ bool layer_has_weights(const NervaHipHfDecodeChainLayer &l) {
          l.w_up && l.w_down;
 }
 
-void destroy_session(Session *s) {
+}  // namespace
+
+void nv::destroy_session(Session *s) {
   if (s == nullptr) return;
   if (s->stream) (void)hipStreamSynchronize(s->stream);
   for (int i = 0; i < 3; ++i) {
@@ -342,9 +226,12 @@ void destroy_session(Session *s) {
   delete s;
 }
 
+namespace {
+
 // Enqueue one step on the session stream (eagerly or under stream capture). With
 // `only` >= 0 just the per-layer launches of that kind are enqueued (profiling).
 hipError_t enqueue_step(Session *s, StepMode mode, StepProfiler *prof, int only = -1) {
+  if (s->stack != nullptr) return stack_enqueue_step(s);   // (profiling and tracing are refused before they get here)
   hipStream_t st = s->stream;
   const uint32_t A = s->heads * s->head_dim, KV = s->kv_heads * s->head_dim;
   hipError_t err = hipSuccess;
@@ -564,6 +451,7 @@ bool eager_steps() {
 
 // Kernel launches of one step (which = 0: decode step, 1: prompt step).
 uint64_t step_launches(const Session *s, int which) {
+  if (s->stack != nullptr) return stack_step_launches(s);
   // embed + (lm head + greedy finish | lm head + two sampler launches | cursor advance)
   const uint64_t fixed = which == 1 ? 2 : (s->sampler.mode == kSamplerGreedy ? 3 : 4);
   return fixed + 5ull * s->layers;
@@ -713,6 +601,8 @@ hipError_t reset_sequence(Session *s, const uint32_t *prompt_tokens, uint32_t pr
   // the words cleared here none of an earlier sequence's can ever match
   if (err == hipSuccess && s->attn_tagged != nullptr)
     err = hipMemsetAsync(s->attn_tagged, 0, attn_step_workspace_bytes(s->heads), s->stream);
+  if (err == hipSuccess && s->stack_state_bytes != 0)   // a new sequence's recurrent state
+    err = hipMemsetAsync(s->stack_state, 0, s->stack_state_bytes, s->stream);
   if (err == hipSuccess) {
     hipLaunchKernelGGL(set_state_kernel, dim3(1), dim3(64), 0, s->stream, s->state, 0u, prompt_count, 1u);
     err = hipGetLastError();
@@ -734,13 +624,13 @@ uint32_t block_operand_tiles(uint32_t tokens) {
   return operand ? gemm_packed_tiles(tokens) : 0u;
 }
 
-// Prompt tokens 0 .. count-1 through every layer in blocks of up to prefill_block_tokens tokens, with the
+// Prompt tokens begin .. count-1 through every layer in blocks of up to prefill_block_tokens tokens, with the
 // prompt staging (16-bit hidden state between layers, prefill_kernels.cu:494-508): per block and
 // layer one RMSNorm launch, the qkv projection as a multi-row GEMM, the K/V rows of the block into the
 // cache, the attention of all its tokens in one launch (token z attends to keys 0 .. first + z), and
 // the o / gate-up / down projections as multi-row GEMMs. Leaves the cursor at `count`. The reference
 // prefills in chunks too (session_decode_prefill.inc.cu:1879-2243).
-hipError_t prefill_blocks(Session *s, uint32_t count, uint32_t prompt_count, NervaHipHfDecodeSequenceResult *out) {
+hipError_t prefill_blocks(Session *s, uint32_t begin, uint32_t count, uint32_t prompt_count, NervaHipHfDecodeSequenceResult *out) {
   hipStream_t st = s->stream;
   const uint32_t H = s->hidden, A = s->heads * s->head_dim, KV = s->kv_heads * s->head_dim, I = s->intermediate;
   const float *rope_freq = s->theta > 0.0f ? s->rope_freq : nullptr;
@@ -752,7 +642,7 @@ hipError_t prefill_blocks(Session *s, uint32_t count, uint32_t prompt_count, Ner
   const uint32_t prompt_splits = want_prompt_splits >= 1 && want_prompt_splits <= static_cast<int>(kAttnMaxSplits)
                                      ? static_cast<uint32_t>(want_prompt_splits)
                                      : 0u;
-  for (uint32_t first = 0; err == hipSuccess && first < count; first += s->prefill_block_tokens) {
+  for (uint32_t first = begin; err == hipSuccess && first < count; first += s->prefill_block_tokens) {
     const uint32_t T = std::min<uint32_t>(s->prefill_block_tokens, count - first);
     const uint32_t tiles = block_operand_tiles(T);
     if (s->dtype == kBF16)
@@ -887,127 +777,63 @@ hipError_t prefill_blocks(Session *s, uint32_t count, uint32_t prompt_count, Ner
   return err;
 }
 
-// ---- weights from the caller's plan -----------------------------------------------------------
-// A declared weight plan (weights.cu:157-160) comes with descriptors that tile the weight bytes
-// [0, resident_weight_bytes) in the reference's arena order - embeddings, then per layer rms_attn,
-// w_q, [q_norm], w_k, [k_norm], w_v, w_o, rms_mlp, w_gate, w_up, w_down, [q/k/v/o bias], then the
-// final norm and the LM head (weights.cu:484-591, session_api_lifecycle.inc.cu:124-148) - each with a
-// host-memory or a file source. The descriptors are then THE source of the weights; the tensor
-// pointers of the request only say which optional tensors exist (weights.cu:18-23) and may be null
-// otherwise (weights.cu:237-243). This library keeps [q;k;v] and [gate;up] as row-concatenated
-// matrices elsewhere in its own arena, so a descriptor's byte range is cut along the tensor
-// boundaries of that order and every piece goes to its tensor's place.
-constexpr uint32_t kWeightStrategyGpuResident = 1, kWeightStrategyGpuStaged = 2;  // weight_plan.rs:3-4
+}  // namespace
 
-struct WeightSegment {
-  uint64_t logical, bytes;  // position in the reference's arena order
-  char *device;
-};
+namespace nv {
 
-template <typename Request>
-bool weight_plan_declared(const Request *rq) {
-  return rq->planned_weight_blocks != 0 || rq->planned_weight_bytes != 0;
-}
-
-void hash_le(uint64_t &hash, uint64_t value, int bytes) {
-  for (int i = 0; i < bytes; ++i) {
-    hash ^= (value >> (8 * i)) & 0xffu;
-    hash *= 0x00000100000001b3ull;
-  }
-}
-
-bool descriptor_has_file(const NervaHipHfDecodeSequenceWeightBlock &d) {
-  return d.source_file != nullptr && d.source_file_len != 0;
-}
-
-// weights.cu:411-467: contiguous from 0, even offsets and sizes, a source each, a known strategy, and
-// totals, counts and the FNV-1a hash over (block_id, block_version, offset_bytes, bytes, strategy)
-// equal to what the plan declares.
-bool validate_weight_descriptors(const NervaHipHfDecodeSequenceSessionCreateRequest *rq, uint64_t resident_weight_bytes) {
-  uint64_t cursor = 0, hash = 0xcbf29ce484222325ull, resident_bytes = 0, staged_bytes = 0;
-  uint32_t resident_blocks = 0, staged_blocks = 0;
-  for (uint32_t i = 0; i < rq->planned_weight_descriptor_count; ++i) {
-    const NervaHipHfDecodeSequenceWeightBlock &d = rq->planned_weight_descriptors[i];
-    if (d.bytes == 0 || d.reserved != 0 || (d.host_source == nullptr && !descriptor_has_file(d)) ||
-        d.offset_bytes != cursor || d.offset_bytes % 2 != 0 || d.bytes % 2 != 0)
-      return false;
-    if (cursor + d.bytes < cursor) return false;
-    cursor += d.bytes;
-    hash_le(hash, d.block_id, 8);
-    hash_le(hash, d.block_version, 8);
-    hash_le(hash, d.offset_bytes, 8);
-    hash_le(hash, d.bytes, 8);
-    hash_le(hash, d.strategy, 4);
-    if (d.strategy == kWeightStrategyGpuResident) {
-      resident_blocks += 1;
-      resident_bytes += d.bytes;
-    } else if (d.strategy == kWeightStrategyGpuStaged) {
-      staged_blocks += 1;
-      staged_bytes += d.bytes;
-    } else {
-      return false;
+hipError_t allocate_session(Session *s, int32_t *failure_stage, bool with_weights) {
+  s->arena_bytes = s->weights->bytes + s->state_bytes;
+  *failure_stage = 2;
+  hipError_t err = hipStreamCreateWithFlags(&s->stream, hipStreamNonBlocking);
+  if (err == hipSuccess && with_weights) {
+    err = counted_malloc(reinterpret_cast<void **>(&s->weights->origin), kMatrixAlign + s->weights->bytes + s->state_bytes);
+    if (err == hipSuccess) {
+      const uint64_t lead = (kMatrixAlign - (reinterpret_cast<uintptr_t>(s->weights->origin) & (kMatrixAlign - 1))) & (kMatrixAlign - 1);
+      s->weights->base = s->weights->origin + lead;
+      s->arena = s->weights->base + s->weights->bytes;
+      s->arena_in_weights = true;
     }
+  } else if (err == hipSuccess) {
+    err = counted_malloc(reinterpret_cast<void **>(&s->arena), s->state_bytes);
   }
-  return cursor == resident_weight_bytes && cursor == rq->planned_weight_bytes &&
-         hash == rq->planned_weight_descriptor_hash && resident_blocks == rq->planned_gpu_resident_blocks &&
-         staged_blocks == rq->planned_gpu_staged_blocks && resident_bytes == rq->planned_gpu_resident_weight_bytes &&
-         staged_bytes == rq->planned_gpu_staged_weight_bytes;
+  if (err != hipSuccess) return err;
+  *failure_stage = 3;
+  const uint64_t pinned_seq = (static_cast<uint64_t>(s->max_ctx) * (sizeof(Slot) + 4) + 256 + 255u) & ~uint64_t{255};
+  const uint64_t pinned_table = (sizeof(BatchTable) + 255u) & ~uint64_t{255};
+  s->pinned_bytes = pinned_seq + pinned_table + static_cast<uint64_t>(NERVA_HIP_BATCH_MAX_BLOCK_TOKENS) * sizeof(Slot);
+  err = counted_host_malloc(reinterpret_cast<void **>(&s->pinned), s->pinned_bytes);
+  if (err == hipSuccess) err = hipEventCreate(&s->ev0);
+  if (err == hipSuccess) err = hipEventCreate(&s->ev1);
+  if (err != hipSuccess) return err;
+  s->host_slots = reinterpret_cast<Slot *>(s->pinned);
+  s->host_prompt = reinterpret_cast<uint32_t *>(s->pinned + static_cast<uint64_t>(s->max_ctx) * sizeof(Slot));
+  s->host_state = s->host_prompt + s->max_ctx;
+  s->host_btable = reinterpret_cast<BatchTable *>(s->pinned + pinned_seq);
+  s->host_bslots = reinterpret_cast<Slot *>(s->pinned + pinned_seq + pinned_table);
+  return hipSuccess;
 }
 
-// weights.cu:797-908: every descriptor to the device, from memory directly or from its file through a
-// pinned staging buffer. `segments` is sorted and gapless in the reference's order.
-hipError_t copy_weight_descriptors(const NervaHipHfDecodeSequenceSessionCreateRequest *rq,
-                                   const std::vector<WeightSegment> &segments, hipStream_t stream, uint64_t *h2d_bytes,
-                                   uint64_t *sync_calls) {
-  constexpr uint64_t kStagingBytes = 64ull << 20;
-  char *staging = nullptr;
+hipError_t set_device_position(Session *s, uint32_t cursor, uint32_t prompt_count, uint32_t clear_fault) {
+  hipLaunchKernelGGL(set_state_kernel, dim3(1), dim3(64), 0, s->stream, s->state, cursor, prompt_count, clear_fault);
+  return hipGetLastError();
+}
+
+}  // namespace nv
+
+namespace {
+
+// Prompt tokens begin .. end-1 (already in s->prompt, the cursor at `begin`), the last one with the head and the
+// sampler: blocks where the model has them, else one captured prompt step per token.
+hipError_t prompt_tokens(Session *s, uint32_t begin, uint32_t end, NervaHipHfDecodeSequenceResult *out) {
+  if (s->stack != nullptr) return stack_prompt(s, begin, end, nullptr, 0, nullptr, nullptr, out);
   hipError_t err = hipSuccess;
-  size_t at = 0;  // descriptors ascend, so the segment cursor only moves forward
-  for (uint32_t i = 0; err == hipSuccess && i < rq->planned_weight_descriptor_count; ++i) {
-    const NervaHipHfDecodeSequenceWeightBlock &d = rq->planned_weight_descriptors[i];
-    FILE *file = nullptr;
-    if (d.host_source == nullptr) {
-      if (staging == nullptr) err = counted_host_malloc(reinterpret_cast<void **>(&staging), kStagingBytes);
-      if (err != hipSuccess) break;
-      const std::string path(d.source_file, d.source_file_len);
-      file = fopen(path.c_str(), "rb");
-      if (file == nullptr) {
-        err = hipErrorInvalidValue;
-        break;
-      }
-    }
-    uint64_t done = 0;
-    while (err == hipSuccess && done < d.bytes) {
-      const uint64_t logical = d.offset_bytes + done;
-      while (at < segments.size() && segments[at].logical + segments[at].bytes <= logical) ++at;
-      if (at == segments.size()) {
-        err = hipErrorInvalidValue;
-        break;
-      }
-      const WeightSegment &seg = segments[at];
-      const uint64_t inside = logical - seg.logical;
-      uint64_t piece = std::min(d.bytes - done, seg.bytes - inside);
-      if (file == nullptr) {
-        err = hipMemcpyAsync(seg.device + inside, reinterpret_cast<const char *>(d.host_source) + done, piece,
-                             hipMemcpyHostToDevice, stream);
-      } else {
-        piece = std::min(piece, kStagingBytes);
-        if (fseeko(file, static_cast<off_t>(d.file_offset_begin + done), SEEK_SET) != 0 ||
-            fread(staging, 1, piece, file) != piece) {
-          err = hipErrorInvalidValue;
-          break;
-        }
-        err = hipMemcpyAsync(seg.device + inside, staging, piece, hipMemcpyHostToDevice, stream);
-        if (err == hipSuccess) err = hipStreamSynchronize(stream);  // the one staging buffer is reused
-        *sync_calls += 1;
-      }
-      done += piece;
-    }
-    if (file != nullptr) fclose(file);
-    *h2d_bytes += done;
+  if (s->block_prefill) {
+    if (end - begin > 1) err = prefill_blocks(s, begin, end - 1, end, out);
+  } else {
+    for (uint32_t i = begin; err == hipSuccess && i + 1 < end; ++i) err = launch_step(s, 1, out);
   }
-  if (err == hipSuccess) err = hipStreamSynchronize(stream);
-  if (staging != nullptr) (void)hipHostFree(staging);
+  if (err == hipSuccess) err = enqueue_step(s, kPromptHeadStep, nullptr);
+  if (err == hipSuccess) out->kernel_launches += step_launches(s, 0);
   return err;
 }
 
@@ -1082,35 +908,9 @@ hipError_t setup_state(Session *s, int32_t *failure_stage, bool with_weights) {
   const uint64_t off_btable = c.take(sizeof(BatchTable));
   const uint64_t off_bslots = c.take(static_cast<uint64_t>(NERVA_HIP_BATCH_MAX_BLOCK_TOKENS) * sizeof(Slot));
   s->state_bytes = c.offset;
-  s->arena_bytes = s->weights->bytes + s->state_bytes;
 
-  *failure_stage = 2;
-  hipError_t err = hipStreamCreateWithFlags(&s->stream, hipStreamNonBlocking);
-  if (err == hipSuccess && with_weights) {
-    err = counted_malloc(reinterpret_cast<void **>(&s->weights->origin), kMatrixAlign + s->weights->bytes + s->state_bytes);
-    if (err == hipSuccess) {
-      const uint64_t lead = (kMatrixAlign - (reinterpret_cast<uintptr_t>(s->weights->origin) & (kMatrixAlign - 1))) & (kMatrixAlign - 1);
-      s->weights->base = s->weights->origin + lead;
-      s->arena = s->weights->base + s->weights->bytes;
-      s->arena_in_weights = true;
-    }
-  } else if (err == hipSuccess) {
-    err = counted_malloc(reinterpret_cast<void **>(&s->arena), s->state_bytes);
-  }
+  hipError_t err = allocate_session(s, failure_stage, with_weights);
   if (err != hipSuccess) return err;
-  *failure_stage = 3;
-  const uint64_t pinned_seq = (static_cast<uint64_t>(s->max_ctx) * (sizeof(Slot) + 4) + 256 + 255u) & ~uint64_t{255};
-  const uint64_t pinned_table = (sizeof(BatchTable) + 255u) & ~uint64_t{255};
-  s->pinned_bytes = pinned_seq + pinned_table + static_cast<uint64_t>(NERVA_HIP_BATCH_MAX_BLOCK_TOKENS) * sizeof(Slot);
-  err = counted_host_malloc(reinterpret_cast<void **>(&s->pinned), s->pinned_bytes);
-  if (err == hipSuccess) err = hipEventCreate(&s->ev0);
-  if (err == hipSuccess) err = hipEventCreate(&s->ev1);
-  if (err != hipSuccess) return err;
-  s->host_slots = reinterpret_cast<Slot *>(s->pinned);
-  s->host_prompt = reinterpret_cast<uint32_t *>(s->pinned + static_cast<uint64_t>(s->max_ctx) * sizeof(Slot));
-  s->host_state = s->host_prompt + s->max_ctx;
-  s->host_btable = reinterpret_cast<BatchTable *>(s->pinned + pinned_seq);
-  s->host_bslots = reinterpret_cast<Slot *>(s->pinned + pinned_seq + pinned_table);
 
   auto dev16 = [&](uint64_t off) { return reinterpret_cast<uint16_t *>(s->arena + off); };
   s->kc = dev16(off_kc);
@@ -1204,7 +1004,9 @@ hipError_t setup_state(Session *s, int32_t *failure_stage, bool with_weights) {
   return err;
 }
 
-void fill_create_result(const Session *s, NervaHipHfDecodeSequenceSessionCreateResult *out) {
+}  // namespace
+
+void nv::fill_create_result(const Session *s, NervaHipHfDecodeSequenceSessionCreateResult *out) {
   out->device_count = 1;
   out->dtype = s->dtype;
   out->hidden = s->hidden;
@@ -1240,6 +1042,8 @@ void fill_create_result(const Session *s, NervaHipHfDecodeSequenceSessionCreateR
       out->device_memory_bandwidth_bps = static_cast<uint64_t>(clock_khz) * 1000ull * 2ull * (static_cast<uint64_t>(bus_bits) / 8ull);
   }
 }
+
+namespace {
 
 int create_impl(const NervaHipHfDecodeSequenceSessionCreateRequest *rq, bool synthetic, uint64_t seed,
                 float weight_std, uint32_t with_qk_norm, NervaHipHfDecodeSequenceSessionCreateResult *out,
@@ -1738,7 +1542,8 @@ int nerva_hip_hf_decode_sequence_session_fork_shared_weights(
   s->lm_head = parent->lm_head;
   s->layer = parent->layer;
 
-  hipError_t err = setup_state(s, &out->failure_stage, false);
+  s->stack = parent->stack;
+  hipError_t err = s->stack != nullptr ? stack_setup_state(s, &out->failure_stage, false) : setup_state(s, &out->failure_stage, false);
   uint64_t syncs = 1;
   if (err == hipSuccess && clone) {
     err = hipStreamSynchronize(parent->stream);
@@ -1751,8 +1556,13 @@ int nerva_hip_hf_decode_sequence_session_fork_shared_weights(
     copy(s->prompt, parent->prompt, static_cast<uint64_t>(s->max_ctx) * 4);
     copy(s->slots, parent->slots, static_cast<uint64_t>(s->max_ctx) * sizeof(Slot));
     copy(s->state, parent->state, 64);
-    copy(s->kc, parent->kc, kv_half);
-    copy(s->vc, parent->vc, kv_half);
+    if (s->stack != nullptr) {
+      copy(s->stack_cache, parent->stack_cache, s->kv_bytes);
+      if (s->stack_state_bytes != 0) copy(s->stack_state, parent->stack_state, s->stack_state_bytes);
+    } else {
+      copy(s->kc, parent->kc, kv_half);
+      copy(s->vc, parent->vc, kv_half);
+    }
     copy(s->sampler_dev, parent->sampler_dev, sizeof(SamplerDev));
     s->sampler = parent->sampler;
     s->prompt_count = parent->prompt_count;
@@ -1804,7 +1614,7 @@ int nerva_hip_hf_decode_sequence_batch_advance_one(const NervaHipHfDecodeSequenc
   };
   // :46-61: same weights by descriptor hash, same dimensions
   auto same_model = [](const Session *a, const Session *b) {
-    return a->planned_weight_descriptor_hash != 0 && a->planned_weight_descriptor_hash == b->planned_weight_descriptor_hash &&
+    return a->stack == b->stack && a->planned_weight_descriptor_hash != 0 && a->planned_weight_descriptor_hash == b->planned_weight_descriptor_hash &&
            a->dtype == b->dtype && a->hidden == b->hidden && a->heads == b->heads && a->kv_heads == b->kv_heads &&
            a->head_dim == b->head_dim && a->intermediate == b->intermediate && a->vocab == b->vocab &&
            a->layers == b->layers && a->resident_weight_bytes == b->resident_weight_bytes;
@@ -2018,15 +1828,9 @@ int nerva_hip_hf_decode_sequence_session_start(const NervaHipHfDecodeSequenceSes
   if (err == hipSuccess) err = reset_sequence(s, request->prompt_tokens, P, out);
   // prefill: the first P-1 prompt tokens (in blocks on the matrix cores where the shapes allow,
   // else one captured prompt step per token), then one prompt step with the LM head and sampler
-  if (err == hipSuccess && P > 1 && !s->block_prefill) err = ensure_graph(s, 1, out);
+  if (err == hipSuccess && P > 1 && s->stack == nullptr && !s->block_prefill) err = ensure_graph(s, 1, out);
   if (err == hipSuccess) err = hipEventRecord(s->ev0, s->stream);
-  if (s->block_prefill) {
-    if (err == hipSuccess && P > 1) err = prefill_blocks(s, P - 1, P, out);
-  } else {
-    for (uint32_t i = 0; err == hipSuccess && i + 1 < P; ++i) err = launch_step(s, 1, out);
-  }
-  if (err == hipSuccess) err = enqueue_step(s, kPromptHeadStep, nullptr);
-  if (err == hipSuccess) out->kernel_launches += step_launches(s, 0);
+  if (err == hipSuccess) err = prompt_tokens(s, 0, P, out);
   if (err == hipSuccess) err = hipEventRecord(s->ev1, s->stream);
   if (err != hipSuccess) {
     out->hip_error = static_cast<int32_t>(err);
@@ -2046,6 +1850,95 @@ int nerva_hip_hf_decode_sequence_session_start(const NervaHipHfDecodeSequenceSes
   out->pinned_host_bytes = static_cast<uint64_t>(s->max_ctx) * sizeof(Slot);
   out->status = 0;
   return 0;
+}
+
+int nerva_hip_session_extend(const NervaHipSessionExtendRequest *request, NervaHipHfDecodeSequenceResult *out) {
+  if (!begin_result(out)) return -1;
+  if (request == nullptr || request->session == nullptr || request->tokens == nullptr || request->token_count == 0 ||
+      (request->wanted_count != 0 && (request->wanted == nullptr || request->logits == nullptr)))
+    return -1;
+  Session *s = request->session;
+  const uint32_t n = request->token_count;
+  if (request->residuals != nullptr && s->stack == nullptr) {
+    out->hip_error = NERVA_HIP_ERROR_NOT_SUPPORTED;
+    return -1;
+  }
+  const bool going_on = s->started && !s->finished;
+  const uint32_t begin = going_on ? s->cursor : 0u;
+  if (static_cast<uint64_t>(begin) + n > s->max_ctx) return -1;
+  for (uint32_t i = 0; i < n; ++i)
+    if (request->tokens[i] >= s->vocab) return -1;
+  for (uint32_t i = 0; i < request->wanted_count; ++i)
+    if (request->wanted[i] >= n || (i != 0 && request->wanted[i] <= request->wanted[i - 1])) return -1;
+  const uint32_t end = begin + n;
+  fill_header(s, out, 0, request->tokens[n - 1]);
+  hipError_t err = hipSuccess;
+  if (!going_on) {
+    s->started = false;
+    NervaHipHfDecodeSamplerConfig greedy{};
+    err = set_sampler(s, greedy);
+    if (err == hipSuccess) err = reset_sequence(s, request->tokens, n, out);
+    s->has_eos = 0;
+  } else {
+    err = hipStreamSynchronize(s->stream);
+    if (err == hipSuccess)
+      err = hipMemcpy(s->prompt + begin, request->tokens, static_cast<uint64_t>(n) * sizeof(uint32_t), hipMemcpyHostToDevice);
+    if (err == hipSuccess) err = set_device_position(s, begin, end, 0);
+    out->h2d_bytes = static_cast<uint64_t>(n) * sizeof(uint32_t);
+  }
+  const auto logits_out = [&](uint32_t i) {   // the last step's logits are wanted row i
+    err = hipMemcpyAsync(request->logits + static_cast<uint64_t>(i) * s->vocab, s->logits, s->vocab * sizeof(float), hipMemcpyDeviceToHost,
+                         s->stream);
+    if (err == hipSuccess) err = hipStreamSynchronize(s->stream);
+    out->d2h_bytes += s->vocab * sizeof(float);
+    out->sync_calls += 1;
+  };
+  if (n == 1 && request->residuals == nullptr) {
+    if (err == hipSuccess) err = ensure_graph(s, decode_graph(s), out);
+    if (err == hipSuccess) err = launch_step(s, decode_graph(s), out);
+    if (err == hipSuccess && request->wanted_count != 0) logits_out(0);
+  } else if (s->stack != nullptr) {
+    if (err == hipSuccess)
+      err = stack_prompt(s, begin, end, request->wanted, request->wanted_count, request->logits, request->residuals, out);
+  } else {
+    if (err == hipSuccess && !s->block_prefill) err = ensure_graph(s, 1, out);
+    // runs of tokens that end at a wanted place (or at the end), each with the head on its last token
+    uint32_t at = 0;
+    for (uint32_t i = 0; err == hipSuccess && at < n; ++i) {
+      const uint32_t stop = i < request->wanted_count ? request->wanted[i] + 1 : n;
+      if (stop > at) err = prompt_tokens(s, begin + at, begin + stop, out);
+      if (err == hipSuccess && stop < end - begin) err = set_device_position(s, begin + stop, end, 0);
+      if (err == hipSuccess && i < request->wanted_count) logits_out(i);
+      at = stop;
+    }
+  }
+  if (err == hipSuccess) err = hipStreamSynchronize(s->stream);
+  out->sync_calls += 1;
+  if (err != hipSuccess) {
+    out->hip_error = static_cast<int32_t>(err);
+    s->finished = true;
+    return -1;
+  }
+  s->prompt_count = end;
+  s->seed_token = request->tokens[n - 1];
+  s->observed = 0;
+  s->cursor = end;
+  s->started = true;
+  s->finished = false;
+  out->resident_kv_bytes = s->kv_bytes;
+  out->kv_tokens = end;
+  out->device_arena_bytes = s->arena_bytes;
+  out->status = 0;
+  return 0;
+}
+
+int nerva_hip_session_release_sequence(NervaHipHfDecodeSequenceSession *session) {
+  if (session == nullptr) return -1;
+  const bool idle = hipStreamSynchronize(session->stream) == hipSuccess;
+  session->started = false;
+  session->finished = false;
+  session->prompt_count = session->observed = session->cursor = 0;
+  return idle ? 0 : -1;
 }
 
 int nerva_hip_hf_decode_sequence_session_advance(const NervaHipHfDecodeSequenceSessionAdvanceRequest *request,
@@ -2257,6 +2150,10 @@ int nerva_hip_hf_decode_sequence_u16(const NervaHipHfDecodeSequenceRequest *rq, 
 int nerva_hip_session_profile_step(NervaHipHfDecodeSequenceSession *s, uint32_t repeats, NervaHipStepProfile *out) {
   if (!begin_result(out)) return -1;
   if (s == nullptr || repeats == 0 || !s->started) return -1;
+  if (s->stack != nullptr) {   // a step advances the recurrent state: it cannot be repeated in place
+    out->hip_error = NERVA_HIP_ERROR_NOT_SUPPORTED;
+    return -1;
+  }
   hipError_t err = hipStreamSynchronize(s->stream);
   uint32_t pos = 0;
   if (err == hipSuccess) err = hipMemcpy(&pos, s->state, 4, hipMemcpyDeviceToHost);
@@ -2380,7 +2277,7 @@ int nerva_hip_session_shares_weight_stream(NervaHipHfDecodeSequenceSession *s) {
 int nerva_hip_steps_are_eager(void) { return eager_steps() ? 1 : 0; }
 
 uint64_t nerva_hip_session_step_trace_bytes(NervaHipHfDecodeSequenceSession *s) {
-  if (s == nullptr) return 0;
+  if (s == nullptr || s->stack != nullptr) return 0;
   auto slot = [](uint64_t bytes) { return (bytes + 255u) & ~uint64_t{255}; };
   const uint64_t A = static_cast<uint64_t>(s->heads) * s->head_dim, KV = static_cast<uint64_t>(s->kv_heads) * s->head_dim;
   const uint64_t per_layer = slot(s->hidden * 2ull) + slot((A + 2 * KV) * 4) + slot(A * 2) + slot(s->hidden * 4ull) +
@@ -2394,7 +2291,7 @@ int nerva_hip_session_trace_next_step(NervaHipHfDecodeSequenceSession *s, void *
     s->trace_buf = nullptr;
     return 0;
   }
-  if (bytes < nerva_hip_session_step_trace_bytes(s)) return -1;
+  if (s->stack != nullptr || bytes < nerva_hip_session_step_trace_bytes(s)) return -1;
   if (s->sampler.mode != kSamplerGreedy) return -1;  // the greedy step only
   s->trace_buf = static_cast<char *>(device_buffer);
   s->trace_used = 0;
@@ -2417,7 +2314,7 @@ int nerva_hip_session_read_slots(NervaHipHfDecodeSequenceSession *s, uint32_t fi
 
 int nerva_hip_session_read_kv_range(NervaHipHfDecodeSequenceSession *s, uint32_t layer, uint32_t first_token,
                                     uint32_t token_count, uint16_t *host_k, uint16_t *host_v) {
-  if (s == nullptr || host_k == nullptr || host_v == nullptr || layer >= s->layers ||
+  if (s == nullptr || s->stack != nullptr || host_k == nullptr || host_v == nullptr || layer >= s->layers ||
       static_cast<uint64_t>(first_token) + token_count > s->max_ctx)
     return -1;
   if (token_count == 0) return 0;

@@ -14,6 +14,8 @@
 // (deterministic) and applies the epilogue.
 #include "gemm_rows.cuh"
 
+#include "activations.cuh"
+
 #include <stdlib.h>
 
 #include <algorithm>
@@ -66,6 +68,14 @@ __device__ __forceinline__ void block_epilogue(const GemmRowsParams &p, uint32_t
     uint16_t h[4];
 #pragma unroll
     for (int r = 0; r < 4; ++r) h[r] = enc16<DT>(silu(y[r]) * up[r]);
+    const uint64_t at16 = p.out_packed_tiles != 0 ? gemm_x_packed_index(p.out_packed_tiles, t, row) : at;
+    *reinterpret_cast<uint2 *>(p.out16 + at16) =
+        make_uint2(h[0] | (static_cast<uint32_t>(h[1]) << 16), h[2] | (static_cast<uint32_t>(h[3]) << 16));
+  } else if constexpr (EPI == kGemmXielu) {
+    const XieluParams act = xielu_params<DT>(p.act);
+    uint16_t h[4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) h[r] = enc16<DT>(xielu(y[r], act));
     const uint64_t at16 = p.out_packed_tiles != 0 ? gemm_x_packed_index(p.out_packed_tiles, t, row) : at;
     *reinterpret_cast<uint2 *>(p.out16 + at16) =
         make_uint2(h[0] | (static_cast<uint32_t>(h[1]) << 16), h[2] | (static_cast<uint32_t>(h[3]) << 16));
@@ -1034,6 +1044,7 @@ hipError_t launch_deep_dt(int epilogue, const GemmRowsParams &p, const DeepPlan 
   switch (epilogue) {
     case kGemmF32: return launch_deep<DT, kGemmF32>(p, partials, plan, stream);
     case kGemmResidual: return launch_deep<DT, kGemmResidual>(p, partials, plan, stream);
+    case kGemmXielu: return launch_deep<DT, kGemmXielu>(p, partials, plan, stream);
     case kGemmSwiglu: return launch_deep<DT, kGemmSwiglu>(p, partials, plan, stream);
     default: return hipErrorInvalidValue;
   }
@@ -1065,6 +1076,7 @@ hipError_t launch_wide_dt(int epilogue, const GemmRowsParams &p, uint32_t kslice
   switch (epilogue) {
     case kGemmF32: return launch_wide<DT, kGemmF32>(p, partials, kslices, stream);
     case kGemmResidual: return launch_wide<DT, kGemmResidual>(p, partials, kslices, stream);
+    case kGemmXielu: return launch_wide<DT, kGemmXielu>(p, partials, kslices, stream);
     case kGemmSwiglu: return launch_wide<DT, kGemmSwiglu>(p, partials, kslices, stream);
     default: return hipErrorInvalidValue;
   }
@@ -1080,6 +1092,9 @@ hipError_t launch_block_dt(int epilogue, const GemmRowsParams &p, const GemmBloc
     case kGemmResidual:
       return plan.row_tiles == 2 ? launch_block_nr<DT, kGemmResidual, 2>(p, partials, plan.kslices, plan.waves, stream)
                                  : launch_block_nr<DT, kGemmResidual, 1>(p, partials, plan.kslices, plan.waves, stream);
+    case kGemmXielu:
+      return plan.row_tiles == 2 ? launch_block_nr<DT, kGemmXielu, 2>(p, partials, plan.kslices, plan.waves, stream)
+                                 : launch_block_nr<DT, kGemmXielu, 1>(p, partials, plan.kslices, plan.waves, stream);
     case kGemmSwiglu: return launch_block_nr<DT, kGemmSwiglu, 2>(p, partials, plan.kslices, plan.waves, stream);
     default: return hipErrorInvalidValue;
   }

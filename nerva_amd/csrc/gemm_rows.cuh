@@ -37,7 +37,8 @@ __host__ __device__ __forceinline__ uint64_t gemm_x_packed_index(uint32_t tiles,
 __host__ __device__ __forceinline__ uint32_t gemm_packed_tiles(uint32_t tokens) {
   return tokens > 256u ? 32u : tokens > 128u ? 16u : tokens > 64u ? 8u : tokens > 32u ? 4u : 2u;
 }
-enum : int { kGemmF32 = 0, kGemmResidual = 1, kGemmSwiglu = 2 };
+// kGemmXielu: a plain projection whose outputs leave as round16(xielu(y)) (activations.cuh).
+enum : int { kGemmF32 = 0, kGemmResidual = 1, kGemmSwiglu = 2, kGemmXielu = 3 };
 
 struct GemmRowsParams {
   const uint16_t *w;         // [rows][cols] row-major 16-bit (SwiGLU: [2*rows][cols], gate rows first)
@@ -45,13 +46,14 @@ struct GemmRowsParams {
   const uint16_t *bias;      // optional [rows] (SwiGLU: [2*rows])
   const float *residual;     // kGemmResidual: [tokens][rows]
   float *out_f32;            // kGemmF32 / kGemmResidual: [tokens][rows]
-  uint16_t *out16;           // kGemmSwiglu: [tokens][rows] = round16(silu(gate) * up)
+  uint16_t *out16;           // kGemmSwiglu: [tokens][rows] = round16(silu(gate) * up); kGemmXielu: round16(xielu(y))
+  const uint16_t *act;       // kGemmXielu: the activation's two numbers
   uint32_t rows, cols, tokens;
   uint32_t pair_gap;         // kGemmSwiglu: elements left unused between the last gate row and the first up row
   uint32_t round_out;        // kGemmResidual: round the sum to 16 bit
   uint32_t x_packed;         // != 0: x16 is in matrix-operand order (gemm_x_packed_index) instead of [tokens][cols];
                              // the value is its token-tile count and must be gemm_packed_tiles(tokens)
-  uint32_t out_packed_tiles; // kGemmSwiglu: != 0 writes out16 in operand order with this many token tiles
+  uint32_t out_packed_tiles; // kGemmSwiglu, kGemmXielu: != 0 writes out16 in operand order with this many token tiles
   uint32_t keep_partials;    // kGemmF32, only where gemm_rows_partial_slices() says so: the K slices' partial sums stay in
                              // the workspace ([slice][128 tokens][rows] f32) for a reader that adds them; out_f32 is not written
   void *workspace;           // optional: room for the f32 partial sums of the shared-X kernel's K slices

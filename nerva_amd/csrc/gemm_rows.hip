@@ -1,6 +1,8 @@
 // Multi-row projection on the matrix cores (see gemm_rows.cuh).
 #include "gemm_rows.cuh"
 
+#include "activations.cuh"
+
 #include <stdlib.h>
 
 #include <mutex>
@@ -170,6 +172,14 @@ __global__ __launch_bounds__(kGThreads) void gemm_rows_kernel(GemmRowsParams p) 
     if constexpr (EPI == kGemmSwiglu) {
       const uint64_t at16 = p.out_packed_tiles != 0 ? gemm_x_packed_index(p.out_packed_tiles, t, grow0 + r) : at;
       p.out16[at16] = enc16<DT>(silu(y[0]) * y[NR - 1]);
+    } else if constexpr (EPI == kGemmXielu) {
+      const XieluParams act = xielu_params<DT>(p.act);
+#pragma unroll
+      for (int j = 0; j < NR; ++j) {
+        const uint32_t row = grow0 + r + j * 16u;
+        p.out16[p.out_packed_tiles != 0 ? gemm_x_packed_index(p.out_packed_tiles, t, row) : static_cast<uint64_t>(t) * p.rows + row] =
+            enc16<DT>(xielu(y[j], act));
+      }
     } else {
 #pragma unroll
       for (int j = 0; j < NR; ++j) {
@@ -281,6 +291,9 @@ hipError_t launch_dt(int epilogue, const GemmRowsParams &p, hipStream_t stream) 
     case kGemmF32:
       if (kw4) return two && can_two ? launch_one<DT, kGemmF32, 2, 4>(p, stream) : launch_one<DT, kGemmF32, 1, 4>(p, stream);
       return two && can_two ? launch_one<DT, kGemmF32, 2, 8>(p, stream) : launch_one<DT, kGemmF32, 1, 8>(p, stream);
+    case kGemmXielu:
+      if (kw4) return launch_one<DT, kGemmXielu, 1, 4>(p, stream);
+      return two && can_two ? launch_one<DT, kGemmXielu, 2, 8>(p, stream) : launch_one<DT, kGemmXielu, 1, 8>(p, stream);
     case kGemmResidual:
       if (kw4) return launch_one<DT, kGemmResidual, 1, 4>(p, stream);
       return two && can_two ? launch_one<DT, kGemmResidual, 2, 8>(p, stream) : launch_one<DT, kGemmResidual, 1, 8>(p, stream);
@@ -312,9 +325,10 @@ hipError_t launch_gemm_rows(uint32_t dtype, int epilogue, const GemmRowsParams &
   if (epilogue == kGemmResidual && p.residual == nullptr) return hipErrorInvalidValue;
   // rows shared by the last two workgroups are written twice: an in-place residual would be added twice
   if (epilogue == kGemmResidual && p.rows % 16 != 0 && p.residual == p.out_f32) return hipErrorInvalidValue;
-  if (epilogue == kGemmSwiglu && p.out16 == nullptr) return hipErrorInvalidValue;
+  if ((epilogue == kGemmSwiglu || epilogue == kGemmXielu) && p.out16 == nullptr) return hipErrorInvalidValue;
+  if (epilogue == kGemmXielu && p.act == nullptr) return hipErrorInvalidValue;
   // (operand order is defined in runs of 32 columns: an output of another width has no such layout)
-  if (p.out_packed_tiles != 0 && (epilogue != kGemmSwiglu || p.out_packed_tiles * 16u < p.tokens || p.rows % 32 != 0))
+  if (p.out_packed_tiles != 0 && ((epilogue != kGemmSwiglu && epilogue != kGemmXielu) || p.out_packed_tiles * 16u < p.tokens || p.rows % 32 != 0))
     return hipErrorInvalidValue;
   if (p.x_packed != 0 && p.x_packed != gemm_packed_tiles(p.tokens)) return hipErrorInvalidValue;   // tiles the kernel will assume
   if (dtype != kBF16 && dtype != kF16) return hipErrorInvalidValue;

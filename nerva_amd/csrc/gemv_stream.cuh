@@ -23,13 +23,21 @@
 // (kernels.cu:577-612,651-687), greedy sampler (sampler.cu:89-119,394-407).
 #pragma once
 
+#include "activations.cuh"
 #include "nerva_hip_api.h"
+#include "norm_join.cuh"
 #include "nv_common.cuh"
 
 namespace nv {
 
-enum : int { kProX16 = 0, kProRmsNorm = 1 };
-enum : int { kEpiF32 = 0, kEpiResidual = 1, kEpiSwiglu = 2, kEpiOut16 = 3, kEpiArgmax = 4 };
+// kProJoin: the residual row takes in a sublayer's normalised output and is normalised itself (norm_join.cuh) - what a
+// stack with a norm before and after every sublayer has between two projections.
+enum : int { kProX16 = 0, kProRmsNorm = 1, kProJoin = 2 };
+// kEpiXielu: out16 = round16(xielu(y)). kEpiMinGru: three rows of W per output (gate, candidate, output gate: rows i,
+// i + rows, i + 2 rows), which advance element i of a recurrent state and leave its gated value in out16.
+enum : int { kEpiF32 = 0, kEpiResidual = 1, kEpiSwiglu = 2, kEpiOut16 = 3, kEpiArgmax = 4, kEpiXielu = 5, kEpiMinGru = 6 };
+// Rows of W that meet in one output element.
+constexpr int gemv_rows_per_output(int epilogue) { return epilogue == kEpiSwiglu ? 2 : epilogue == kEpiMinGru ? 3 : 1; }
 
 // Device sampler state. The LM-head GEMV (or the stand-alone argmax kernel) stores
 // one candidate per workgroup; sample_finish_kernel (one workgroup) reduces them
@@ -82,6 +90,10 @@ struct GemvParams {
   const uint32_t *cursor;  // optional step guard: skip when *cursor >= max_steps
   uint32_t max_steps;
   SampleParams sample;
+  JoinNorm join;               // kProJoin (xf is not used)
+  const uint16_t *act;         // kEpiXielu: the activation's two numbers
+  const uint16_t *bias2;       // kEpiMinGru: bias of the candidate rows (`bias` is the gate's)
+  float *state;                // kEpiMinGru: [rows] f32, advanced in place
   // test hook of the RMSNorm prologue: when set, workgroup 0 also writes the 16-bit vector the rows
   // are multiplied with (the prologue's output, which otherwise exists in LDS only) to [cols]
   uint16_t *x16_dump;
@@ -153,7 +165,7 @@ enum : int { kScalar = 0, kVecGuarded = 1, kVecFull = 2 };
 template <uint32_t DT, int PRO, int EPI, int NR, int U, int MODE, bool DOT2>
 __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
   extern __shared__ __align__(16) uint16_t xs[];  // cols (rounded up to 8) 16-bit values
-  __shared__ float red[kWavesPerBlock];
+  __shared__ float red[PRO == kProJoin ? kWavesPerBlock * 3 : kWavesPerBlock];
   __shared__ uint32_t red_i[kWavesPerBlock];
   __shared__ uint32_t red_h[kWavesPerBlock];
 
@@ -162,7 +174,8 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
   const int lane = threadIdx.x & (kWave - 1);
   const int wave = threadIdx.x / kWave;
   const uint32_t cols = p.cols;
-  const uint32_t units = (EPI == kEpiSwiglu) ? p.rows : (p.rows + NR - 1) / NR;
+  constexpr bool kJoint = gemv_rows_per_output(EPI) > 1;   // a unit's rows lie p.rows apart and make one output
+  const uint32_t units = kJoint ? p.rows : (p.rows + NR - 1) / NR;
   const uint32_t wave_global = blockIdx.x * kWavesPerBlock + wave;
   const uint32_t wave_stride = gridDim.x * kWavesPerBlock;
   const uint32_t nchunks = cols / (kWave * 8);
@@ -170,8 +183,8 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
   auto unit_rows = [&](uint32_t unit, uint32_t (&row)[NR], const uint16_t *(&wrow)[NR], bool (&live)[NR]) {
 #pragma unroll
     for (int k = 0; k < NR; ++k) {
-      if constexpr (EPI == kEpiSwiglu) {
-        row[k] = unit + k * p.rows;  // k = 0 gate row, k = 1 up row
+      if constexpr (kJoint) {
+        row[k] = unit + k * p.rows;  // SwiGLU: k = 0 gate row, k = 1 up row
         live[k] = true;
       } else {
         row[k] = unit * NR + k;
@@ -212,6 +225,8 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
     } else {
       for (uint32_t c = threadIdx.x; c < cols; c += kBlock) xs[c] = p.x16[c];
     }
+  } else if constexpr (PRO == kProJoin) {
+    join_norm_row<DT, kWavesPerBlock>(p.join, cols, blockIdx.x == 0, red, [&](uint32_t c, float v) { xs[c] = enc16<DT>(v); });
   } else {
     // x = round16(v * rsqrt(mean(v^2) + eps) * gamma)
     float ss = 0.0f;
@@ -256,6 +271,8 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
 
   // ---- main loop: each wave owns NR rows per iteration -------------------
   Best best{0.0f, 0u, 0u};
+  XieluParams act{};
+  if constexpr (EPI == kEpiXielu) act = xielu_params<DT>(p.act);
 
   // One unit of NR rows per phase. buf[ph] holds the unit's head (requested earlier); the
   // head of the unit after it goes into buf[ph ^ 1] before buf[ph] is consumed, so the
@@ -338,6 +355,10 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
           u += dec16<DT>(p.bias[row[1]]);
         }
         p.out16[unit] = enc16<DT>(silu(g) * u);
+      } else if constexpr (EPI == kEpiMinGru) {
+        const float next = mingru_step(acc[0] + dec16<DT>(p.bias[unit]), acc[1] + dec16<DT>(p.bias2[unit]), p.state[unit]);
+        p.state[unit] = next;
+        p.out16[unit] = enc16<DT>(next * silu(acc[2]));
       } else {
 #pragma unroll
         for (int k = 0; k < NR; ++k) {
@@ -352,6 +373,8 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
             p.out_f32[row[k]] = y;
           } else if constexpr (EPI == kEpiOut16) {
             p.out16[row[k]] = enc16<DT>(y);
+          } else if constexpr (EPI == kEpiXielu) {
+            p.out16[row[k]] = enc16<DT>(xielu(y, act));
           } else if constexpr (EPI == kEpiArgmax) {
             p.out_f32[row[k]] = y;
             Best cand{y, row[k], isfinite(y) ? 1u : 0u};
@@ -402,8 +425,9 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
 // ---------------------------------------------------------------------------
 // Register budget as resident waves per SIMD (= workgroups per CU): 6 with a 16-bit input,
 // 5 with the RMSNorm prologue, which holds the f32 activations and the norm weights in
-// registers across the first weight requests (a budget of 6 makes it spill).
-constexpr int fast_waves_per_simd(int prologue) { return prologue == kProRmsNorm ? 5 : 6; }
+// registers across the first weight requests (a budget of 6 makes it spill), 4 with the join
+// prologue, which holds two f32 rows and the weights and biases of two norms.
+constexpr int fast_waves_per_simd(int prologue) { return prologue == kProJoin ? 4 : prologue == kProRmsNorm ? 5 : 6; }
 constexpr int kFastMaxCols = 12288;  // x staged through at most 6 x 16 B per lane in registers ...
 constexpr int kFastMaxColsLoop = 30720;  // ... or, with a 16-bit input, copied into LDS behind the first weight requests
 
@@ -436,14 +460,14 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   constexpr int TB = WG * kWave;
   constexpr uint32_t kXregBpr = 8 / B;   // batches per 4096-column row
   extern __shared__ __align__(16) uint16_t xs[];
-  __shared__ float red[WG];
+  __shared__ float red[PRO == kProJoin ? WG * 3 : WG];
   __shared__ uint32_t red_i[WG];
   __shared__ uint32_t red_h[WG];
 
   const int lane = threadIdx.x & (kWave - 1);
   const int wave = threadIdx.x / kWave;
   const uint32_t cols = p.cols;
-  const uint32_t units = p.rows;  // NR == 1: rows; kEpiSwiglu (NR == 2): gate/up pairs
+  const uint32_t units = p.rows;  // NR == 1: rows; kEpiSwiglu (NR == 2): gate/up pairs; kEpiMinGru (NR == 3): triples
   const uint32_t wave_global = blockIdx.x * WG + wave;
   const uint32_t wave_stride = gridDim.x * WG;
   const uint32_t bpr = cols / (kWave * 8 * B);  // request batches per row
@@ -456,6 +480,7 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   float4 xa[PRO == kProRmsNorm ? 2 : 1], xb[PRO == kProRmsNorm ? 2 : 1];
   uint4 gw[PRO == kProRmsNorm ? 2 : 1];
   const bool norm_in_regs = cols <= TB * 16;
+  JoinRegs join[PRO == kProJoin ? 2 : 1];   // (the launcher keeps cols <= TB * 16 here)
   // (the same for every wave of the launch; a constant in the variant with exact start-up waits, which only
   // runs at 4096 columns, so its request counts stay countable)
   const bool x_in_regs = EXACT || cols <= static_cast<uint32_t>(kFastMaxCols);
@@ -468,6 +493,9 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
         if (c < cols) xraw[i] = *reinterpret_cast<const uint4 *>(p.x16 + c);
       }
     }
+  } else if constexpr (PRO == kProJoin) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) join_load8(p.join, (i * TB + threadIdx.x) * 8, cols, join[i]);
   } else {
     if (norm_in_regs) {
 #pragma unroll
@@ -488,8 +516,9 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   constexpr uint32_t kBatchElems = B * kWave * 8;
   const uint16_t *wp[NR];
   uint4 buf0[NR][B], buf1[NR][B];
-  float res0 = 0.0f, res1 = 0.0f;     // residual element requested with a row's first batch
-#define NV_FAST_ISSUE(DST, RES)                                                                   \
+  float res0 = 0.0f, res1 = 0.0f;     // residual element (recurrent state) requested with a row's first batch
+  float zb0 = 0.0f, zb1 = 0.0f, ub0 = 0.0f, ub1 = 0.0f;   // kEpiMinGru: the row's two biases, likewise
+#define NV_FAST_ISSUE(DST, RES, ZB, UB)                                                                 \
   do {                                                                                            \
     if (ib == 0) {                                                                                \
       if constexpr (ROT) ic = iu % bpr;                                                           \
@@ -497,6 +526,11 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
         wp[k] = p.w + static_cast<uint64_t>(iu + k * p.rows) * cols + k * p.pair_gap + ic * kBatchElems + lane * 8; \
       if constexpr (EPI == kEpiResidual) {                                                        \
         if (EXACT || lane == 0) RES = p.residual[iu];                                             \
+      }                                                                                           \
+      if constexpr (EPI == kEpiMinGru) {                                                          \
+        RES = p.state[iu];                                                                        \
+        ZB = dec16<DT>(p.bias[iu]);                                                               \
+        UB = dec16<DT>(p.bias2[iu]);                                                              \
       }                                                                                           \
     }                                                                                             \
     _Pragma("unroll") for (int u = 0; u < B; ++u)                                                 \
@@ -514,11 +548,11 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
     }                                                                                             \
   } while (0)
   if constexpr (EXACT) {  // the launcher guarantees two batches per row at least
-    NV_FAST_ISSUE(buf0, res0);
-    NV_FAST_ISSUE(buf1, res1);
+    NV_FAST_ISSUE(buf0, res0, zb0, ub0);
+    NV_FAST_ISSUE(buf1, res1, zb1, ub1);
   } else {
-    if (total > 0) NV_FAST_ISSUE(buf0, res0);
-    if (total > 1) NV_FAST_ISSUE(buf1, res1);
+    if (total > 0) NV_FAST_ISSUE(buf0, res0, zb0, ub0);
+    if (total > 1) NV_FAST_ISSUE(buf1, res1, zb1, ub1);
   }
 
   // ---- 3. step guard (after the requests: they do not depend on it and are always in bounds)
@@ -538,6 +572,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
       for (uint32_t c = threadIdx.x * 8; c < cols; c += TB * 8)
         *reinterpret_cast<uint4 *>(xs + c) = *reinterpret_cast<const uint4 *>(p.x16 + c);
     }
+  } else if constexpr (PRO == kProJoin) {
+    join_norm_regs<DT, WG>(p.join, cols, blockIdx.x == 0, join, red, xs);
   } else {
     float ss = 0.0f;
     if (norm_in_regs) {
@@ -597,12 +633,16 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   Best best{0.0f, 0u, 0u};
   uint32_t cu = wave_global, cb = 0;  // batch being consumed: unit, batch within the row
   float acc[NR];
-  float res_cur = 0.0f;
-#define NV_FAST_CONSUME(SRC, RES)                                                                 \
+  float res_cur = 0.0f, zb_cur = 0.0f, ub_cur = 0.0f;
+  XieluParams act{};
+  if constexpr (EPI == kEpiXielu) act = xielu_params<DT>(p.act);
+#define NV_FAST_CONSUME(SRC, RES, ZB, UB)                                                               \
   do {                                                                                            \
     if (cb == 0) {                                                                                \
       _Pragma("unroll") for (int k = 0; k < NR; ++k) acc[k] = 0.0f;                               \
       res_cur = RES;                                                                              \
+      zb_cur = ZB;                                                                                \
+      ub_cur = UB;                                                                                \
       if constexpr (ROT) cc = cu % bpr;                                                           \
     }                                                                                             \
     const uint32_t c0 = (ROT ? cc : cb) * (B * kWave * 8) + lane * 8;                             \
@@ -626,6 +666,10 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
             u += dec16<DT>(p.bias[cu + p.rows]);                                                  \
           }                                                                                       \
           p.out16[cu] = enc16<DT>(silu(g) * u);                                                   \
+        } else if constexpr (EPI == kEpiMinGru) {                                                 \
+          const float next = mingru_step(acc[0] + zb_cur, acc[NR > 1 ? 1 : 0] + ub_cur, res_cur); \
+          p.state[cu] = next;                                                                     \
+          p.out16[cu] = enc16<DT>(next * silu(acc[NR - 1]));                                      \
         } else {                                                                                  \
           float y = acc[0];                                                                       \
           if (p.bias != nullptr) y += dec16<DT>(p.bias[cu]);                                      \
@@ -637,6 +681,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
             p.out_f32[cu] = y;                                                                    \
           } else if constexpr (EPI == kEpiOut16) {                                                \
             p.out16[cu] = enc16<DT>(y);                                                           \
+          } else if constexpr (EPI == kEpiXielu) {                                                \
+            p.out16[cu] = enc16<DT>(xielu(y, act));                                               \
           } else if constexpr (EPI == kEpiArgmax) {                                               \
             p.out_f32[cu] = y;                                                                    \
             Best cand{y, cu, isfinite(y) ? 1u : 0u};                                              \
@@ -652,27 +698,27 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
     // one unit per turn: its batches alternate between the two buffers, the batch index is a constant
     for (uint32_t t = 0; t < total; t += kXregBpr) {
       cb = 0;
-      NV_FAST_CONSUME(buf0, res0);
-      if (t + 2 < total) NV_FAST_ISSUE(buf0, res0);
+      NV_FAST_CONSUME(buf0, res0, zb0, ub0);
+      if (t + 2 < total) NV_FAST_ISSUE(buf0, res0, zb0, ub0);
       cb = 1;
-      NV_FAST_CONSUME(buf1, res1);
-      if (t + 3 < total) NV_FAST_ISSUE(buf1, res1);
+      NV_FAST_CONSUME(buf1, res1, zb1, ub1);
+      if (t + 3 < total) NV_FAST_ISSUE(buf1, res1, zb1, ub1);
       if constexpr (kXregBpr == 4) {
         cb = 2;
-        NV_FAST_CONSUME(buf0, res0);
-        if (t + 4 < total) NV_FAST_ISSUE(buf0, res0);
+        NV_FAST_CONSUME(buf0, res0, zb0, ub0);
+        if (t + 4 < total) NV_FAST_ISSUE(buf0, res0, zb0, ub0);
         cb = 3;
-        NV_FAST_CONSUME(buf1, res1);
-        if (t + 5 < total) NV_FAST_ISSUE(buf1, res1);
+        NV_FAST_CONSUME(buf1, res1, zb1, ub1);
+        if (t + 5 < total) NV_FAST_ISSUE(buf1, res1, zb1, ub1);
       }
     }
   } else {
     for (uint32_t t = 0; t < total; t += 2) {
-      NV_FAST_CONSUME(buf0, res0);
-      if (t + 2 < total) NV_FAST_ISSUE(buf0, res0);
+      NV_FAST_CONSUME(buf0, res0, zb0, ub0);
+      if (t + 2 < total) NV_FAST_ISSUE(buf0, res0, zb0, ub0);
       if (t + 1 < total) {
-        NV_FAST_CONSUME(buf1, res1);
-        if (t + 3 < total) NV_FAST_ISSUE(buf1, res1);
+        NV_FAST_CONSUME(buf1, res1, zb1, ub1);
+        if (t + 3 < total) NV_FAST_ISSUE(buf1, res1, zb1, ub1);
       }
     }
   }

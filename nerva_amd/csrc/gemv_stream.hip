@@ -52,7 +52,7 @@ __global__ __launch_bounds__(1024) void sample_finish_kernel(SampleParams s, uin
 
 template <uint32_t DT, int PRO, int EPI, int MODE>
 hipError_t launch_one(const GemvParams &p, const GemvPlan &plan, size_t lds, hipStream_t stream) {
-  constexpr int NR = EPI == kEpiSwiglu ? 2 : kDefaultNR;  // swiglu: the gate row and the up row
+  constexpr int NR = gemv_rows_per_output(EPI) > 1 ? gemv_rows_per_output(EPI) : kDefaultNR;  // (swiglu: gate and up row)
   const uint32_t blocks = plan.blocks;
   const int wg = plan.wg_waves;
   if constexpr (MODE == kFast) {
@@ -81,13 +81,17 @@ hipError_t launch_one(const GemvParams &p, const GemvPlan &plan, size_t lds, hip
       if constexpr (EPI == kEpiSwiglu) {
         if (wg == 16) NV_GEMV_LAUNCH(2, false, 16, false, true);
         else NV_GEMV_LAUNCH(2, false, 4, false, true);
-      } else if constexpr (PRO == kProRmsNorm && EPI == kEpiArgmax) {
+      } else if constexpr (PRO != kProX16 && EPI == kEpiArgmax) {
         NV_GEMV_LAUNCH(1, false, 16, false, true);
       } else if constexpr (PRO == kProRmsNorm && EPI == kEpiF32) {
         NV_GEMV_LAUNCH(2, false, 4, false, true);
       } else {
         return hipErrorInvalidValue;
       }
+    } else if constexpr (EPI == kEpiMinGru) {
+      // three rows an output, two chunks of each a batch
+      if (wg == 16) NV_GEMV_LAUNCH(2, false, 16, false, false);
+      else NV_GEMV_LAUNCH(2, false, 4, false, false);
     } else if (plan.chunks == 2 && NR == 1) {
       // rows that are whole batches of 1024 columns but not of 2048 (hidden 5120, MLP width 25600): two chunks a batch
       if (wg == 16) NV_GEMV_LAUNCH(2, false, 16, false, false);
@@ -120,6 +124,15 @@ hipError_t launch_one(const GemvParams &p, const GemvPlan &plan, size_t lds, hip
 
 template <uint32_t DT, int PRO, int MODE>
 hipError_t launch_epi(int epilogue, const GemvParams &p, const GemvPlan &plan, size_t lds, hipStream_t stream) {
+  if constexpr (PRO == kProJoin) {   // what a stack with the join seam has between its projections
+    switch (epilogue) {
+      case kEpiF32: return launch_one<DT, PRO, kEpiF32, MODE>(p, plan, lds, stream);
+      case kEpiArgmax: return launch_one<DT, PRO, kEpiArgmax, MODE>(p, plan, lds, stream);
+      case kEpiXielu: return launch_one<DT, PRO, kEpiXielu, MODE>(p, plan, lds, stream);
+      case kEpiMinGru: return launch_one<DT, PRO, kEpiMinGru, MODE>(p, plan, lds, stream);
+      default: return hipErrorInvalidValue;
+    }
+  } else {
   switch (epilogue) {
     case kEpiF32: return launch_one<DT, PRO, kEpiF32, MODE>(p, plan, lds, stream);
     case kEpiResidual: return launch_one<DT, PRO, kEpiResidual, MODE>(p, plan, lds, stream);
@@ -128,6 +141,7 @@ hipError_t launch_epi(int epilogue, const GemvParams &p, const GemvPlan &plan, s
     case kEpiArgmax: return launch_one<DT, PRO, kEpiArgmax, MODE>(p, plan, lds, stream);
     default: return hipErrorInvalidValue;
   }
+  }
 }
 
 template <uint32_t DT, int MODE>
@@ -135,6 +149,7 @@ hipError_t launch_pro(int prologue, int epilogue, const GemvParams &p, const Gem
                       hipStream_t stream) {
   if (prologue == kProX16) return launch_epi<DT, kProX16, MODE>(epilogue, p, plan, lds, stream);
   if (prologue == kProRmsNorm) return launch_epi<DT, kProRmsNorm, MODE>(epilogue, p, plan, lds, stream);
+  if (prologue == kProJoin) return launch_epi<DT, kProJoin, MODE>(epilogue, p, plan, lds, stream);
   return hipErrorInvalidValue;
 }
 
@@ -146,8 +161,8 @@ bool aligned16(const void *ptr) { return (reinterpret_cast<uintptr_t>(ptr) & 15u
 // launches measured the same (qkv, o, down: within 0.1 us) or worse (gate_up 32.8 -> 34.6 us: one workgroup of
 // 16 waves per CU instead of five of 4) with 16.
 int fast_workgroup_waves(int prologue, int epilogue, uint32_t rows, uint32_t cols) {
-  (void)cols;
-  return prologue == kProRmsNorm && epilogue == kEpiArgmax && rows >= 65536u ? 16 : kWavesPerBlock;
+  if (prologue == kProJoin && cols > kWavesPerBlock * kWave * 16u) return 16;   // the seam's row in the lanes' registers
+  return prologue != kProX16 && epilogue == kEpiArgmax && rows >= 65536u ? 16 : kWavesPerBlock;
 }
 
 }  // namespace
@@ -196,7 +211,7 @@ GemvPlan gemv_plan(int prologue, int epilogue, uint32_t rows, uint32_t cols, boo
     if (nv::tuning(kTuneGemvRotatedWalk) != 2) {
       if (epilogue == kEpiSwiglu) {
         plan.rotated = true;                                  // gate/up pair: 2 KiB of each row a batch
-      } else if (prologue == kProRmsNorm && epilogue == kEpiArgmax && plan.wg_waves == 16 && plan.chunks == 4) {
+      } else if (prologue != kProX16 && epilogue == kEpiArgmax && plan.wg_waves == 16 && plan.chunks == 4) {
         plan.rotated = true;                                  // LM head: 1 KiB a batch
         plan.chunks = 1;
       } else if (prologue == kProRmsNorm && epilogue == kEpiF32 && plan.wg_waves == 4 && cols == 4096u && auto_grid &&
@@ -220,9 +235,14 @@ hipError_t launch_gemv(uint32_t dtype, int prologue, int epilogue, const GemvPar
   if (p.w == nullptr || p.rows == 0 || p.cols == 0) return hipErrorInvalidValue;
   if (prologue == kProX16 && p.x16 == nullptr) return hipErrorInvalidValue;
   if (prologue == kProRmsNorm && (p.xf == nullptr || p.gamma == nullptr)) return hipErrorInvalidValue;
+  if (prologue == kProJoin && (p.join.x == nullptr || p.join.pre_w == nullptr || p.join.pre_b == nullptr || p.join.x_out == p.join.x ||
+                               (p.join.y != nullptr && (p.join.post_w == nullptr || p.join.post_b == nullptr))))
+    return hipErrorInvalidValue;
+  if (epilogue == kEpiXielu && p.act == nullptr) return hipErrorInvalidValue;
+  if (epilogue == kEpiMinGru && (p.bias == nullptr || p.bias2 == nullptr || p.state == nullptr)) return hipErrorInvalidValue;
   if ((epilogue == kEpiF32 || epilogue == kEpiResidual || epilogue == kEpiArgmax) && p.out_f32 == nullptr)
     return hipErrorInvalidValue;
-  if ((epilogue == kEpiSwiglu || epilogue == kEpiOut16) && p.out16 == nullptr) return hipErrorInvalidValue;
+  if ((epilogue == kEpiSwiglu || epilogue == kEpiOut16 || epilogue == kEpiXielu || epilogue == kEpiMinGru) && p.out16 == nullptr) return hipErrorInvalidValue;
   if (epilogue == kEpiResidual && p.residual == nullptr) return hipErrorInvalidValue;
   if (epilogue == kEpiArgmax && (p.sample.part_value == nullptr || p.sample.part_index == nullptr ||
                                  p.sample.part_has == nullptr))
@@ -230,7 +250,10 @@ hipError_t launch_gemv(uint32_t dtype, int prologue, int epilogue, const GemvPar
   if (dtype != kF16 && dtype != kBF16) return hipErrorInvalidValue;
 
   const bool vec16 = aligned16(p.w) && (prologue == kProX16 ? aligned16(p.x16)
-                                                             : (aligned16(p.xf) && aligned16(p.gamma)));
+                                         : prologue == kProJoin
+                                             ? aligned16(p.join.x) && aligned16(p.join.y) && aligned16(p.join.x_out) && aligned16(p.join.post_w) &&
+                                                   aligned16(p.join.post_b) && aligned16(p.join.pre_w) && aligned16(p.join.pre_b)
+                                             : (aligned16(p.xf) && aligned16(p.gamma)));
   const size_t lds = static_cast<size_t>((p.cols + 7) / 8 * 8) * sizeof(uint16_t);
   if (lds > 60 * 1024) return hipErrorInvalidValue;  // K up to 30720 fits one workgroup's LDS
   const GemvPlan plan = gemv_plan(prologue, epilogue, p.rows, p.cols, vec16, tuning);

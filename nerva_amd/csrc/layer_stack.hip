@@ -1,0 +1,867 @@
+// Sessions over a mixed layer stack (see layer_stack.hpp).
+#include "layer_stack.hpp"
+
+#include <math.h>
+
+#include <algorithm>
+#include <new>
+
+#include "attn_mixed.cuh"
+#include "gemm_any.cuh"
+#include "mingru.cuh"
+#include "norm_join.cuh"
+#include "synth_fill.cuh"
+#include "weight_plan.hpp"
+
+using namespace nv;
+
+namespace {
+
+struct Angles {
+  const float *step;
+  const uint32_t *cos_col, *sin_col;
+  uint32_t count, columns;
+};
+
+// Embedding rows and rotation tables of the tokens at positions first .. first + gridDim.x - 1, or of the one at the
+// device cursor (a prompt token, or the token the position before it published).
+template <uint32_t DT>
+__global__ __launch_bounds__(kBlock) void stack_embed_kernel(const uint16_t *emb, const uint32_t *prompt, const Slot *slots,
+                                                             const uint32_t *state, bool at_cursor, uint32_t first,
+                                                             uint32_t max_steps, uint32_t hidden, uint32_t vocab, float *x,
+                                                             Angles angles, float *rope) {
+  const uint32_t t = blockIdx.x, pos = at_cursor ? state[0] : first + t;
+  if (pos >= max_steps) return;
+  for (uint32_t i = threadIdx.x; i < angles.count; i += kBlock) {
+    float sn, cs;
+    sincosf(static_cast<float>(pos) * angles.step[i], &sn, &cs);
+    float *row = rope + static_cast<uint64_t>(t) * angles.columns;
+    row[angles.cos_col[i]] = cs;
+    row[angles.sin_col[i]] = sn;
+  }
+  uint32_t token = !at_cursor || pos < state[1] ? prompt[pos] : slots[pos - 1].token;
+  if (token >= vocab) token = 0;   // prompts are validated on the host; sampled ids are < vocab
+  const uint16_t *row = emb + static_cast<uint64_t>(token) * hidden;
+  for (uint32_t i = threadIdx.x; i < hidden; i += kBlock) x[static_cast<uint64_t>(t) * hidden + i] = dec16<DT>(row[i]);
+}
+
+// Identity plus noise for a synthetic mixing matrix (the noise is there already).
+__global__ void add_identity_kernel(uint16_t *m, uint32_t n) {
+  const uint32_t i = blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) m[static_cast<uint64_t>(i) * n + i] = f32_to_bf16(bf16_to_f32(m[static_cast<uint64_t>(i) * n + i]) + 1.0f);
+}
+
+bool wide(const Session *s) { return s->stack->precision == NERVA_HIP_PRECISION_32; }
+
+// The seam that is due before the next projection: the norm of the sublayer output in s->y / s->py, if there is one.
+struct Seam {
+  const uint16_t *post_w = nullptr, *post_b = nullptr;
+};
+
+// ---- decode step, 16-bit precision -----------------------------------------------------------
+
+struct DecodeRow {
+  float *x, *next;   // the residual row, and where the next seam leaves it
+  Seam due;
+};
+
+JoinNorm decode_seam(Session *s, DecodeRow &row, const uint16_t *pre_w, const uint16_t *pre_b) {
+  JoinNorm j{};
+  j.x = row.x;
+  j.pre_w = pre_w;
+  j.pre_b = pre_b;
+  j.eps = s->eps;
+  if (row.due.post_w != nullptr) {
+    j.y = s->y;
+    j.post_w = row.due.post_w;
+    j.post_b = row.due.post_b;
+    j.x_out = row.next;
+    std::swap(row.x, row.next);
+    row.due = Seam{};
+  }
+  return j;
+}
+
+GemvParams decode_gemv(Session *s, const uint16_t *w, uint32_t rows, uint32_t cols) {
+  GemvParams p{};
+  p.w = w;
+  p.rows = rows;
+  p.cols = cols;
+  p.cursor = s->state;
+  p.max_steps = s->max_ctx;
+  return p;
+}
+
+MixedAttnParams attention_params(Session *s, const StackLayer &layer, const float *proj, const float *rope) {
+  const StackModel &m = *s->stack;
+  const StackLayer &owner = m.layers[layer.cache_layer];
+  MixedAttnParams a{};
+  a.proj = proj;
+  a.proj_stride = layer.in_rows;
+  a.q_col = layer.q_col;
+  a.k_col = layer.k_col;
+  a.v_col = layer.v_col;
+  a.gate_col = layer.gate_col;
+  a.talk = layer.talk;
+  a.sink = layer.sink;
+  a.k_cache = s->stack_cache + owner.k_offset;
+  a.v_cache = s->stack_cache + owner.v_offset;
+  a.table = s->stack_tables + owner.table_offset;
+  a.rope_cs = rope + layer.rotation;
+  a.rot_dims = layer.spec.rotary_dims;
+  a.rope_stride = m.rotation_columns;
+  a.heads = layer.spec.heads;
+  a.kv_heads = layer.spec.kv_heads;
+  a.key_dim = layer.spec.key_dim;
+  a.value_dim = layer.spec.value_dim;
+  a.chunk = layer.spec.chunk_tokens;
+  a.scale = layer.spec.score_scale;
+  a.cache32 = wide(s) ? 1u : 0u;
+  a.max_steps = s->max_ctx;
+  a.workspace = s->attn_ws;
+  a.last_block = m.logical_blocks - 1;
+  return a;
+}
+
+// Final norm, head, sampler of the row in (row.x, s->y): logits, slot[cursor], cursor + 1.
+hipError_t decode_head(Session *s, DecodeRow &row) {
+  const StackModel &m = *s->stack;
+  GemvParams p = decode_gemv(s, s->lm_head, s->vocab, s->hidden);
+  p.join = decode_seam(s, row, m.final_w, m.final_b);
+  p.out_f32 = s->logits;
+  sample_bind_workspace(p.sample, s->sample_ws);
+  p.sample.slots = s->slots;
+  p.sample.cursor_rw = s->state;
+  uint32_t candidates = 0;
+  hipError_t err = launch_gemv(s->dtype, kProJoin, kEpiArgmax, p, s->stream, nullptr, &candidates);
+  if (err != hipSuccess) return err;
+  if (s->sampler.mode == kSamplerGreedy) return launch_sample_finish(p.sample, candidates, s->state, s->max_ctx, s->stream);
+  SamplerParams sp{};
+  sp.logits = s->logits;
+  sp.vocab = s->vocab;
+  sp.config = s->sampler_dev;
+  sp.keys = s->sampler_keys;
+  sp.out = p.sample;
+  sp.cursor = s->state;
+  sp.max_steps = s->max_ctx;
+  return launch_sampler(sp, s->stream);
+}
+
+hipError_t embed_rows(Session *s, bool at_cursor, uint32_t first, uint32_t tokens, float *x) {
+  const StackModel &m = *s->stack;
+  const uint32_t *cols = reinterpret_cast<const uint32_t *>(s->rope_freq + m.angle_step.size());
+  const uint32_t n = static_cast<uint32_t>(m.angle_step.size());
+  const Angles angles{s->rope_freq, cols, cols + n, n, m.rotation_columns};
+  hipLaunchKernelGGL(stack_embed_kernel<kBF16>, dim3(tokens), dim3(kBlock), 0, s->stream, s->emb, s->prompt, s->slots, s->state,
+                     at_cursor, first, s->max_ctx, s->hidden, s->vocab, x, angles, s->prope);
+  return hipGetLastError();
+}
+
+hipError_t decode_step_16(Session *s) {
+  const StackModel &m = *s->stack;
+  hipStream_t st = s->stream;
+  hipError_t err = embed_rows(s, true, 0, 1, s->x);
+  DecodeRow row{s->x, s->r, Seam{}};
+  for (size_t l = 0; err == hipSuccess && l < m.layers.size(); ++l) {
+    const StackLayer &w = m.layers[l];
+    GemvParams p = decode_gemv(s, w.w_in, w.in_rows, s->hidden);
+    p.join = decode_seam(s, row, w.norm[0], w.norm[1]);
+    if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION) {
+      p.out_f32 = s->qkv;
+      err = launch_gemv(s->dtype, kProJoin, kEpiF32, p, st);
+      MixedAttnParams a = attention_params(s, w, s->qkv, s->prope);
+      a.cursor = s->state;
+      a.tokens = 1;
+      a.out16 = s->attn16;
+      if (err == hipSuccess && w.own_cache()) err = launch_mixed_publish(s->dtype, a, st);
+      if (err == hipSuccess) err = launch_mixed_attention(s->dtype, a, st);
+    } else {
+      p.rows = w.spec.width;
+      p.out16 = s->attn16;
+      p.bias = w.z_bias;
+      p.bias2 = w.x_bias;
+      p.state = s->stack_state + w.state_offset;
+      err = launch_gemv(s->dtype, kProJoin, kEpiMinGru, p, st);
+    }
+    if (err == hipSuccess) {
+      p = decode_gemv(s, w.w_out, s->hidden, w.out_cols);
+      p.x16 = s->attn16;
+      p.out_f32 = s->y;
+      err = launch_gemv(s->dtype, kProX16, kEpiF32, p, st);
+      row.due = Seam{w.norm[2], w.norm[3]};
+    }
+    if (err != hipSuccess || w.spec.ff == 0) continue;
+    p = decode_gemv(s, w.w_up, w.spec.ff, s->hidden);
+    p.join = decode_seam(s, row, w.norm[4], w.norm[5]);
+    p.act = w.act;
+    p.out16 = s->ff16;
+    err = launch_gemv(s->dtype, kProJoin, kEpiXielu, p, st);
+    if (err == hipSuccess) {
+      p = decode_gemv(s, w.w_down, s->hidden, w.spec.ff);
+      p.x16 = s->ff16;
+      p.out_f32 = s->y;
+      err = launch_gemv(s->dtype, kProX16, kEpiF32, p, st);
+      row.due = Seam{w.norm[6], w.norm[7]};
+    }
+  }
+  return err == hipSuccess ? decode_head(s, row) : err;
+}
+
+// ---- blocks of token rows --------------------------------------------------------------------
+
+// Token tiles of the matrix-operand order a projection's input takes, 0 where its shape goes through gemm_any.
+uint32_t operand_tiles(const Session *s, int epilogue, uint32_t rows, uint32_t cols, uint32_t tokens) {
+  if (wide(s) || cols % 32 != 0) return 0;
+  const bool taken = tokens <= kGemmMaxTokens       ? gemm_rows_supported(rows, cols, tokens)
+                     : tokens <= kGemmWideMaxTokens ? gemm_wide_slices(epilogue, rows, cols, tokens, s->pgemm_ws_bytes) != 0
+                                                    : gemm_deep_slices(epilogue, rows, cols, tokens, s->pgemm_ws_bytes) != 0;
+  return taken ? gemm_packed_tiles(tokens) : 0u;
+}
+
+struct Block {
+  Session *s;
+  uint32_t tokens, first;
+  bool at_cursor;      // the one token at the device cursor (a step of a 32-bit session)
+  Seam due;
+  uint64_t launches;
+
+  hipError_t join(const uint16_t *pre_w, const uint16_t *pre_b, uint32_t tiles) {
+    JoinRows j{};
+    j.x = s->px;
+    if (due.post_w != nullptr) {
+      j.y = s->py;
+      j.post_w = due.post_w;
+      j.post_b = due.post_b;
+      due = Seam{};
+    }
+    j.pre_w = pre_w;
+    j.pre_b = pre_b;
+    if (pre_w != nullptr) {
+      if (wide(s)) j.out32 = static_cast<float *>(s->pxn);
+      else j.out16 = static_cast<uint16_t *>(s->pxn);
+    }
+    j.packed_tiles = tiles;
+    j.tokens = tokens;
+    j.cols = s->hidden;
+    j.eps = s->eps;
+    launches += 1;
+    return launch_join_rows(s->dtype, j, s->stream);
+  }
+
+  // x: the 16-bit or f32 rows of `tiles` layout; out: f32 rows, or for the activation 16-bit rows of out_tiles layout
+  hipError_t project(int epilogue, const uint16_t *w, uint32_t rows, uint32_t cols, const void *x, uint32_t tiles, void *out,
+                     uint32_t out_tiles, const uint16_t *act) {
+    launches += 1;
+    const bool narrow = epilogue == kGemmXielu && !wide(s);
+    if (tiles != 0) {
+      GemmRowsParams g{};
+      g.w = w;
+      g.x16 = static_cast<const uint16_t *>(x);
+      g.x_packed = tiles;
+      g.rows = rows;
+      g.cols = cols;
+      g.tokens = tokens;
+      g.workspace = s->pgemm_ws;
+      g.workspace_bytes = s->pgemm_ws_bytes;
+      g.act = act;
+      if (narrow) {
+        g.out16 = static_cast<uint16_t *>(out);
+        g.out_packed_tiles = out_tiles;
+      } else {
+        g.out_f32 = static_cast<float *>(out);
+      }
+      return launch_gemm_rows(s->dtype, epilogue, g, s->stream);
+    }
+    GemmAnyParams g{};
+    g.w = w;
+    if (wide(s)) g.x32 = static_cast<const float *>(x);
+    else g.x16 = static_cast<const uint16_t *>(x);
+    g.rows = rows;
+    g.cols = cols;
+    g.tokens = tokens;
+    g.act = act;
+    if (narrow) {
+      g.out16 = static_cast<uint16_t *>(out);
+      g.out_packed_tiles = out_tiles;
+    } else {
+      g.out_f32 = static_cast<float *>(out);
+    }
+    return launch_gemm_any(s->dtype, epilogue, g, s->stream);
+  }
+
+  hipError_t mixer(const StackLayer &w) {
+    const uint32_t in_tiles = operand_tiles(s, kGemmF32, w.in_rows, s->hidden, tokens);
+    const uint32_t out_tiles = operand_tiles(s, kGemmF32, s->hidden, w.out_cols, tokens);
+    hipError_t err = join(w.norm[0], w.norm[1], in_tiles);
+    if (err == hipSuccess) err = project(kGemmF32, w.w_in, w.in_rows, s->hidden, s->pxn, in_tiles, s->pqkv, 0, nullptr);
+    if (err != hipSuccess) return err;
+    if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION) {
+      MixedAttnParams a = attention_params(s, w, s->pqkv, s->prope);
+      a.position = first;
+      a.tokens = tokens;
+      if (at_cursor) a.cursor = s->state;
+      if (wide(s)) a.out32 = static_cast<float *>(s->pmix);
+      else a.out16 = static_cast<uint16_t *>(s->pmix);
+      a.packed_tiles = out_tiles;
+      if (w.own_cache()) {
+        err = launch_mixed_publish(s->dtype, a, s->stream);
+        launches += 1;
+      }
+      if (err == hipSuccess) err = launch_mixed_attention(s->dtype, a, s->stream);
+    } else {
+      MinGruRows g{};
+      g.zxg = s->pqkv;
+      g.z_bias = w.z_bias;
+      g.x_bias = w.x_bias;
+      g.state = s->stack_state + w.state_offset;
+      if (wide(s)) g.out32 = static_cast<float *>(s->pmix);
+      else g.out16 = static_cast<uint16_t *>(s->pmix);
+      g.packed_tiles = out_tiles;
+      g.tokens = tokens;
+      g.width = w.spec.width;
+      if (at_cursor) {
+        g.cursor = s->state;
+        g.max_steps = s->max_ctx;
+      }
+      err = launch_mingru_rows(s->dtype, g, s->stream);
+    }
+    launches += 1;
+    if (err == hipSuccess) err = project(kGemmF32, w.w_out, s->hidden, w.out_cols, s->pmix, out_tiles, s->py, 0, nullptr);
+    due = Seam{w.norm[2], w.norm[3]};
+    return err;
+  }
+
+  hipError_t feed_forward(const StackLayer &w) {
+    const uint32_t up_tiles = operand_tiles(s, kGemmXielu, w.spec.ff, s->hidden, tokens);
+    const uint32_t down_tiles = operand_tiles(s, kGemmF32, s->hidden, w.spec.ff, tokens);
+    hipError_t err = join(w.norm[4], w.norm[5], up_tiles);
+    if (err == hipSuccess) err = project(kGemmXielu, w.w_up, w.spec.ff, s->hidden, s->pxn, up_tiles, s->pff, down_tiles, w.act);
+    if (err == hipSuccess) err = project(kGemmF32, w.w_down, s->hidden, w.spec.ff, s->pff, down_tiles, s->py, 0, nullptr);
+    due = Seam{w.norm[6], w.norm[7]};
+    return err;
+  }
+
+  // residuals: host [layers][row_stride] f32, the block's rows of every layer, or null
+  hipError_t layers(float *residuals, uint64_t row_stride) {
+    hipError_t err = embed_rows(s, at_cursor, first, tokens, s->px);
+    launches += 1;
+    const StackModel &m = *s->stack;
+    for (size_t l = 0; err == hipSuccess && l < m.layers.size(); ++l) {
+      err = mixer(m.layers[l]);
+      if (err == hipSuccess && m.layers[l].spec.ff != 0) err = feed_forward(m.layers[l]);
+      if (err == hipSuccess && residuals != nullptr) {
+        err = join(nullptr, nullptr, 0);
+        if (err == hipSuccess)
+          err = hipMemcpyAsync(residuals + l * row_stride, s->px, static_cast<uint64_t>(tokens) * s->hidden * sizeof(float),
+                               hipMemcpyDeviceToHost, s->stream);
+      }
+    }
+    return err;
+  }
+
+  // Logits of the block's rows pick[0 .. count) into s->pwant_logits (count <= kStackWantedRows) or, for the one row of
+  // a block of one token, into `logits`. Leaves the residual rows as they are where rows are picked.
+  hipError_t logits_of(const uint32_t *pick, uint32_t count, float *logits) {
+    const StackModel &m = *s->stack;
+    const uint32_t tiles = !wide(s) && s->hidden % 32 == 0 && gemm_rows_supported(s->vocab, s->hidden, count) ? gemm_packed_tiles(count) : 0u;
+    JoinRows j{};
+    j.x = s->px;
+    if (due.post_w != nullptr) {
+      j.y = s->py;
+      j.post_w = due.post_w;
+      j.post_b = due.post_b;
+    }
+    j.pre_w = m.final_w;
+    j.pre_b = m.final_b;
+    j.pick = pick;
+    if (wide(s)) j.out32 = static_cast<float *>(s->pwant);
+    else j.out16 = static_cast<uint16_t *>(s->pwant);
+    j.packed_tiles = tiles;
+    j.tokens = count;
+    j.cols = s->hidden;
+    j.eps = s->eps;
+    hipError_t err = launch_join_rows(s->dtype, j, s->stream);
+    const uint32_t rows = tokens;
+    tokens = count;
+    if (err == hipSuccess) err = project(kGemmF32, s->lm_head, s->vocab, s->hidden, s->pwant, tiles, logits, 0, nullptr);
+    tokens = rows;
+    launches += 1;
+    return err;
+  }
+};
+
+// The sampler from s->logits (sessions whose head is not the decode step's).
+hipError_t sample_logits(Session *s) {
+  SamplerParams sp{};
+  sp.logits = s->logits;
+  sp.vocab = s->vocab;
+  sp.config = s->sampler_dev;
+  sp.keys = s->sampler_keys;
+  sample_bind_workspace(sp.out, s->sample_ws);
+  sp.out.slots = s->slots;
+  sp.out.cursor_rw = s->state;
+  sp.cursor = s->state;
+  sp.max_steps = s->max_ctx;
+  return launch_sampler(sp, s->stream);
+}
+
+}  // namespace
+
+hipError_t nv::stack_enqueue_step(Session *s) {
+  if (!wide(s)) return decode_step_16(s);
+  Block b{s, 1, 0, true, Seam{}, 0};
+  hipError_t err = b.layers(nullptr, 0);
+  if (err == hipSuccess) err = b.logits_of(nullptr, 1, s->logits);
+  if (err == hipSuccess) err = sample_logits(s);
+  return err;
+}
+
+uint64_t nv::stack_step_launches(const Session *s) {
+  // (the seam is a launch of its own in a 32-bit session only)
+  uint64_t n = 1 + (wide(s) ? 4 : s->sampler.mode == kSamplerGreedy ? 2 : 3);
+  for (const StackLayer &w : s->stack->layers) {
+    const uint64_t seam = wide(s) ? 1 : 0;
+    n += seam + (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION ? (w.own_cache() ? 4 : 3) : (wide(s) ? 3 : 2));
+    if (w.spec.ff != 0) n += seam + 2;
+  }
+  return n;
+}
+
+hipError_t nv::stack_prompt(Session *s, uint32_t begin, uint32_t end, const uint32_t *wanted, uint32_t wanted_count, float *logits,
+                            float *residuals, NervaHipHfDecodeSequenceResult *out) {
+  hipError_t err = hipSuccess;
+  uint32_t next_wanted = 0;
+  const uint64_t H = s->hidden;
+  for (uint32_t first = begin; err == hipSuccess && first < end; first += kStackBlockTokens) {
+    Block b{s, std::min(kStackBlockTokens, end - first), first, false, Seam{}, 0};
+    err = b.layers(residuals != nullptr ? residuals + static_cast<uint64_t>(first - begin) * H : nullptr,
+                   static_cast<uint64_t>(end - begin) * H);
+    while (err == hipSuccess && next_wanted < wanted_count && wanted[next_wanted] < first + b.tokens - begin) {
+      uint32_t *rows = s->host_state, count = 0;   // (pinned; the copies below are waited for before it is written again)
+      while (count < kStackWantedRows && next_wanted + count < wanted_count && wanted[next_wanted + count] < first + b.tokens - begin) {
+        rows[count] = wanted[next_wanted + count] - (first - begin);
+        count += 1;
+      }
+      err = hipMemcpyAsync(s->pwant_rows, rows, count * sizeof(uint32_t), hipMemcpyHostToDevice, s->stream);
+      if (err == hipSuccess) err = b.logits_of(s->pwant_rows, count, s->pwant_logits);
+      if (err == hipSuccess)
+        err = hipMemcpyAsync(logits + static_cast<uint64_t>(next_wanted) * s->vocab, s->pwant_logits,
+                             static_cast<uint64_t>(count) * s->vocab * sizeof(float), hipMemcpyDeviceToHost, s->stream);
+      if (err == hipSuccess) err = hipStreamSynchronize(s->stream);
+      out->d2h_bytes += static_cast<uint64_t>(count) * s->vocab * sizeof(float);
+      out->sync_calls += 1;
+      next_wanted += count;
+    }
+    if (err == hipSuccess && first + b.tokens == end) {
+      // the sequence's last token so far: head and sampler at its position
+      err = set_device_position(s, end - 1, end, 0);
+      const uint64_t last = b.tokens - 1;
+      if (err == hipSuccess && !wide(s)) {
+        // (with residuals read back the last seam is done already)
+        err = hipMemcpyAsync(s->x, s->px + last * H, H * sizeof(float), hipMemcpyDeviceToDevice, s->stream);
+        if (err == hipSuccess) err = hipMemcpyAsync(s->y, s->py + last * H, H * sizeof(float), hipMemcpyDeviceToDevice, s->stream);
+        DecodeRow row{s->x, s->r, b.due};
+        if (err == hipSuccess) err = decode_head(s, row);
+      } else if (err == hipSuccess) {
+        s->host_state[kStackWantedRows] = static_cast<uint32_t>(last);
+        err = hipMemcpyAsync(s->pwant_rows, s->host_state + kStackWantedRows, sizeof(uint32_t), hipMemcpyHostToDevice, s->stream);
+        if (err == hipSuccess) err = b.logits_of(s->pwant_rows, 1, s->logits);
+        if (err == hipSuccess) err = sample_logits(s);
+      }
+      b.launches += 3;
+    }
+    out->kernel_launches += b.launches;
+  }
+  return err;
+}
+
+// ---- layout ----------------------------------------------------------------------------------
+
+namespace {
+
+struct LayerOffsets {
+  uint64_t norm[8], w_in, w_out, talk, sink, z_bias, x_bias, w_up, w_down, act;
+};
+
+// Largest chunk any reader of layer l's cache looks at (0: one of them looks at everything).
+uint32_t widest_chunk(const std::vector<StackLayer> &layers, size_t l) {
+  uint32_t widest = 0;
+  for (const StackLayer &r : layers) {
+    if (r.spec.mixer != NERVA_HIP_MIXER_ATTENTION || r.cache_layer != l) continue;
+    if (r.spec.chunk_tokens == 0) return 0;
+    widest = std::max(widest, r.spec.chunk_tokens);
+  }
+  return widest;
+}
+
+bool layer_valid(const NervaHipStackLayer *layers, uint32_t count, uint32_t l, uint32_t hidden) {
+  const NervaHipStackLayer &d = layers[l];
+  if (static_cast<uint64_t>(d.ff) * 2 > 60 * 1024) return false;
+  (void)hidden;
+  if (d.mixer == NERVA_HIP_MIXER_MINGRU) return d.width != 0 && static_cast<uint64_t>(d.width) * 2 <= 60 * 1024;
+  if (d.mixer != NERVA_HIP_MIXER_ATTENTION) return false;
+  if (d.heads == 0 || d.kv_heads == 0 || d.heads % d.kv_heads != 0 || d.key_dim == 0 || d.value_dim == 0 || d.rotary_dims % 2 != 0 ||
+      d.rotary_dims > d.key_dim || d.value_dim > kMixedMaxValueDim || static_cast<uint64_t>(d.kv_heads) * d.key_dim > kMixedMaxFolded ||
+      static_cast<uint64_t>(d.heads) * d.value_dim * 2 > 60 * 1024 || !isfinite(d.score_scale) ||
+      (d.rotary_dims != 0 && !(d.rotary_base > 0.0f && isfinite(d.rotary_base))))
+    return false;
+  if (d.kv_layer == NERVA_HIP_OWN_KEYS) return true;
+  // the layer it borrows from comes before it, has keys of its own, and they have this layer's shape
+  if (d.kv_layer >= count || d.kv_layer >= l) return false;
+  const NervaHipStackLayer &o = layers[d.kv_layer];
+  return o.mixer == NERVA_HIP_MIXER_ATTENTION && o.kv_layer == NERVA_HIP_OWN_KEYS && o.kv_heads == d.kv_heads && o.key_dim == d.key_dim &&
+         o.value_dim == d.value_dim;
+}
+
+template <typename F>
+bool create_checks(const NervaHipStackSessionCreateRequest *rq, bool synthetic, F &&unsupported) {
+  if (rq == nullptr || rq->hidden == 0 || rq->vocab_size == 0 || rq->layer_count == 0 || rq->max_context_tokens == 0 ||
+      rq->layers == nullptr || rq->precision > NERVA_HIP_PRECISION_32 || !(rq->norm_eps >= 0.0f) || !isfinite(rq->norm_eps))
+    return false;
+  if (rq->dtype != NERVA_HIP_DTYPE_BF16 || static_cast<uint64_t>(rq->hidden) * 2 > 60 * 1024) {
+    unsupported();
+    return false;
+  }
+  for (uint32_t l = 0; l < rq->layer_count; ++l)
+    if (!layer_valid(rq->layers, rq->layer_count, l, rq->hidden)) return false;
+  // the weights come through a complete plan
+  return synthetic || (rq->planned_weight_blocks != 0 && rq->planned_weight_bytes != 0 && rq->planned_weight_descriptors != nullptr &&
+                       rq->planned_weight_descriptor_count == rq->planned_weight_blocks && rq->planned_weight_descriptor_hash != 0);
+}
+
+int create_stack(const NervaHipStackSessionCreateRequest *rq, bool synthetic, uint64_t seed, float weight_std,
+                 NervaHipHfDecodeSequenceSessionCreateResult *out, Session **session_out) {
+  if (!begin_result(out)) return -1;
+  if (session_out == nullptr) return -1;
+  *session_out = nullptr;
+  out->failure_stage = 1;
+  if (!create_checks(rq, synthetic, [&] { out->hip_error = NERVA_HIP_ERROR_NOT_SUPPORTED; })) return -1;
+  if (!device_ready(&out->hip_error)) return -1;
+
+  std::shared_ptr<StackModel> model(new (std::nothrow) StackModel());
+  Session *s = new (std::nothrow) Session();
+  if (s == nullptr || model == nullptr) {
+    delete s;
+    return -1;
+  }
+  s->weights = new (std::nothrow) SharedWeights();
+  if (s->weights == nullptr) {
+    delete s;
+    return -1;
+  }
+  const uint64_t H = rq->hidden, V = rq->vocab_size;
+  const uint32_t L = rq->layer_count;
+  s->dtype = rq->dtype;
+  s->hidden = rq->hidden;
+  s->vocab = rq->vocab_size;
+  s->layers = L;
+  s->max_ctx = rq->max_context_tokens;
+  s->eps = rq->norm_eps;
+  s->planned_weight_blocks = rq->planned_weight_blocks;
+  s->planned_gpu_resident_blocks = rq->planned_gpu_resident_blocks;
+  s->planned_gpu_staged_blocks = rq->planned_gpu_staged_blocks;
+  s->planned_weight_bytes = rq->planned_weight_bytes;
+  s->planned_gpu_resident_weight_bytes = rq->planned_gpu_resident_weight_bytes;
+  s->planned_gpu_staged_weight_bytes = rq->planned_gpu_staged_weight_bytes;
+  s->planned_weight_descriptor_count = rq->planned_weight_descriptor_count;
+  s->planned_weight_descriptor_hash = rq->planned_weight_descriptor_hash;
+
+  // ---- layers: columns of the projections, rotations, caches, states
+  StackModel &m = *model;
+  m.precision = rq->precision;
+  m.layers.resize(L);
+  m.logical_blocks = (s->max_ctx + kKvBlockTokens - 1) / kKvBlockTokens;
+  const uint64_t cache_elem = rq->precision == NERVA_HIP_PRECISION_32 ? 4 : 2;
+  std::vector<std::pair<uint32_t, float>> rotations;   // (dims, base) met so far, in the order of their columns
+  std::vector<uint32_t> rotation_at;
+  for (uint32_t l = 0; l < L; ++l) {
+    StackLayer &w = m.layers[l];
+    w.spec = rq->layers[l];
+    const NervaHipStackLayer &d = w.spec;
+    if (d.mixer == NERVA_HIP_MIXER_ATTENTION) {
+      const bool own = d.kv_layer == NERVA_HIP_OWN_KEYS;
+      w.cache_layer = own ? l : d.kv_layer;
+      w.out_cols = d.heads * d.value_dim;
+      w.k_col = w.q_col + d.heads * d.key_dim;
+      w.v_col = w.k_col + (own ? d.kv_heads * d.key_dim : 0u);
+      w.gate_col = w.v_col + (own ? d.kv_heads * d.value_dim : 0u);
+      w.in_rows = w.gate_col + w.out_cols;
+      size_t r = 0;
+      while (r < rotations.size() && rotations[r] != std::make_pair(d.rotary_dims, d.rotary_base)) ++r;
+      if (r == rotations.size()) {
+        rotations.emplace_back(d.rotary_dims, d.rotary_base);
+        rotation_at.push_back(m.rotation_columns);
+        const uint32_t half = d.rotary_dims / 2;
+        for (uint32_t i = 0; i < half; ++i) {
+          m.angle_step.push_back(static_cast<float>(pow(static_cast<double>(d.rotary_base), -2.0 * i / d.rotary_dims)));
+          m.angle_cos.push_back(m.rotation_columns + i);
+          m.angle_sin.push_back(m.rotation_columns + half + i);
+        }
+        m.rotation_columns += d.rotary_dims;
+      }
+      w.rotation = rotation_at[r];
+      s->heads = std::max(s->heads, d.heads);
+      s->kv_heads = std::max(s->kv_heads, d.kv_heads);
+      s->head_dim = std::max(s->head_dim, d.key_dim);
+    } else {
+      w.out_cols = d.width;
+      w.in_rows = 3 * d.width;
+      w.state_offset = m.state_floats;
+      m.state_floats += (d.width + 63u) & ~63u;
+    }
+    m.max_in = std::max(m.max_in, w.in_rows);
+    m.max_mix = std::max(m.max_mix, w.out_cols);
+    m.max_ff = std::max(m.max_ff, d.ff);
+  }
+  s->intermediate = m.max_ff;
+  for (uint32_t l = 0; l < L; ++l) {
+    StackLayer &w = m.layers[l];
+    if (!w.own_cache()) continue;
+    // A block of token rows writes all its keys before its first query looks back: the oldest key that query may see
+    // and the newest key written lie less than chunk + kStackBlockTokens positions apart, one block more for the edges.
+    const uint32_t chunk = widest_chunk(m.layers, l);
+    const uint64_t reach = (static_cast<uint64_t>(chunk) + kStackBlockTokens + kKvBlockTokens - 1) / kKvBlockTokens + 1;
+    w.ring_blocks = chunk == 0 || reach > m.logical_blocks ? m.logical_blocks : static_cast<uint32_t>(reach);
+    const auto area = [&](uint32_t dim) {
+      const uint64_t at = m.cache_bytes;
+      m.cache_bytes += (static_cast<uint64_t>(w.ring_blocks) * w.spec.kv_heads * kKvBlockTokens * dim * cache_elem + 255u) & ~uint64_t{255};
+      return at;
+    };
+    w.k_offset = area(w.spec.key_dim);
+    w.v_offset = area(w.spec.value_dim);
+    w.table_offset = m.table_entries;
+    m.table_entries += m.logical_blocks;
+  }
+
+  // ---- weight arena layout
+  Carver c;
+  const auto matrix = [&](uint64_t rows, uint64_t cols) {
+    const uint64_t bytes = rows * cols * 2;
+    return c.take(bytes, bytes >= kMatrixAlign ? kMatrixAlign : 8192u);
+  };
+  const uint64_t off_emb = matrix(V, H);
+  std::vector<LayerOffsets> lo(L);
+  for (uint32_t l = 0; l < L; ++l) {
+    const StackLayer &w = m.layers[l];
+    const NervaHipStackLayer &d = w.spec;
+    for (uint64_t &at : lo[l].norm) at = c.take(H * 2);
+    lo[l].w_in = matrix(w.in_rows, H);
+    lo[l].w_out = matrix(H, w.out_cols);
+    if (d.mixer == NERVA_HIP_MIXER_ATTENTION) {
+      lo[l].talk = c.take(static_cast<uint64_t>(d.heads) * d.heads * 2);
+      lo[l].sink = c.take(d.heads * 2ull);
+    } else {
+      lo[l].z_bias = c.take(d.width * 2ull);
+      lo[l].x_bias = c.take(d.width * 2ull);
+    }
+    if (d.ff != 0) {
+      lo[l].w_up = matrix(d.ff, H);
+      lo[l].w_down = matrix(H, d.ff);
+      lo[l].act = c.take(4);
+    }
+  }
+  const uint64_t off_final_w = c.take(H * 2), off_final_b = c.take(H * 2);
+  s->weights->bytes = c.offset;
+
+  // ---- the plan's order of tensors: (offset in the arena, elements, kind of synthetic value)
+  enum Kind { kMatrix, kUnit, kZero, kTalk };
+  struct Piece {
+    uint64_t off, elems;
+    Kind kind;
+    uint32_t n;
+  };
+  std::vector<Piece> pieces;
+  const auto piece = [&](uint64_t off, uint64_t elems, Kind kind, uint32_t n = 0) { pieces.push_back(Piece{off, elems, kind, n}); };
+  piece(off_emb, V * H, kMatrix);
+  for (uint32_t l = 0; l < L; ++l) {
+    const StackLayer &w = m.layers[l];
+    const NervaHipStackLayer &d = w.spec;
+    for (uint32_t i = 0; i < (d.ff != 0 ? 8u : 4u); ++i) piece(lo[l].norm[i], H, i % 2 == 0 ? kUnit : kZero);
+    const auto rows_of = [&](uint32_t first, uint32_t rows) { piece(lo[l].w_in + static_cast<uint64_t>(first) * H * 2, rows * H, kMatrix); };
+    if (d.mixer == NERVA_HIP_MIXER_ATTENTION) {
+      rows_of(w.q_col, d.heads * d.key_dim);
+      if (w.own_cache()) {
+        rows_of(w.k_col, d.kv_heads * d.key_dim);
+        rows_of(w.v_col, d.kv_heads * d.value_dim);
+      }
+      rows_of(w.gate_col, w.out_cols);
+      piece(lo[l].talk, static_cast<uint64_t>(d.heads) * d.heads, kTalk, d.heads);
+      piece(lo[l].sink, d.heads, kZero);
+    } else {
+      for (uint32_t i = 0; i < 3; ++i) rows_of(i * d.width, d.width);
+      piece(lo[l].z_bias, d.width, kZero);
+      piece(lo[l].x_bias, d.width, kZero);
+    }
+    piece(lo[l].w_out, H * w.out_cols, kMatrix);
+    if (d.ff != 0) {
+      piece(lo[l].w_up, d.ff * H, kMatrix);
+      piece(lo[l].w_down, H * d.ff, kMatrix);
+      piece(lo[l].act, 2, kZero);
+    }
+  }
+  piece(off_final_w, H, kUnit);
+  piece(off_final_b, H, kZero);
+  uint64_t elems = 0;
+  for (const Piece &p : pieces) elems += p.elems;
+  s->resident_weight_bytes = elems * 2;
+  if (!synthetic && !validate_weight_descriptors(rq, s->resident_weight_bytes)) {
+    destroy_session(s);
+    return -1;
+  }
+
+  s->stack = model;
+  hipError_t err = stack_setup_state(s, &out->failure_stage, true);
+  uint64_t h2d = 0, syncs = 1;
+  if (err == hipSuccess) {
+    char *base = s->weights->base;
+    const auto w16 = [&](uint64_t off) { return reinterpret_cast<const uint16_t *>(base + off); };
+    s->emb = s->lm_head = w16(off_emb);
+    m.final_w = w16(off_final_w);
+    m.final_b = w16(off_final_b);
+    for (uint32_t l = 0; l < L; ++l) {
+      StackLayer &w = m.layers[l];
+      for (int i = 0; i < 8; ++i) w.norm[i] = w16(lo[l].norm[i]);
+      w.w_in = w16(lo[l].w_in);
+      w.w_out = w16(lo[l].w_out);
+      if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION) {
+        w.talk = w16(lo[l].talk);
+        w.sink = w16(lo[l].sink);
+      } else {
+        w.z_bias = w16(lo[l].z_bias);
+        w.x_bias = w16(lo[l].x_bias);
+      }
+      if (w.spec.ff != 0) {
+        w.w_up = w16(lo[l].w_up);
+        w.w_down = w16(lo[l].w_down);
+        w.act = w16(lo[l].act);
+      }
+    }
+    out->failure_stage = 4;
+    if (synthetic) {
+      for (size_t i = 0; err == hipSuccess && i < pieces.size(); ++i) {
+        const Piece &p = pieces[i];
+        err = launch_synth_16(base + p.off, s->dtype, seed, i + 1, p.elems, p.kind == kUnit ? 1.0f : 0.0f, weight_std, s->stream);
+        if (err == hipSuccess && p.kind == kTalk) {
+          hipLaunchKernelGGL(add_identity_kernel, dim3((p.n + 255u) / 256u), dim3(256), 0, s->stream,
+                             reinterpret_cast<uint16_t *>(base + p.off), p.n);
+          err = hipGetLastError();
+        }
+      }
+      if (err == hipSuccess) err = hipStreamSynchronize(s->stream);
+    } else {
+      std::vector<WeightSegment> segments;
+      uint64_t logical = 0;
+      for (const Piece &p : pieces) {
+        segments.push_back(WeightSegment{logical, p.elems * 2, base + p.off});
+        logical += p.elems * 2;
+      }
+      err = copy_weight_descriptors(rq, segments, s->stream, &h2d, &syncs);
+    }
+  }
+  if (err != hipSuccess) {
+    out->hip_error = static_cast<int32_t>(err);
+    destroy_session(s);
+    return -1;
+  }
+  out->failure_stage = 0;
+  fill_create_result(s, out);
+  out->prefill_chunk_tokens = kStackBlockTokens;
+  out->h2d_bytes = h2d;
+  out->sync_calls = syncs;
+  out->status = 0;
+  *session_out = s;
+  return 0;
+}
+
+}  // namespace
+
+hipError_t nv::stack_setup_state(Session *s, int32_t *failure_stage, bool with_weights) {
+  const StackModel &m = *s->stack;
+  const uint64_t H = s->hidden, V = s->vocab, T = kStackBlockTokens, es = wide(s) ? 4 : 2;
+  s->block_count = m.logical_blocks;
+  s->kv_bytes = m.cache_bytes;
+  s->stack_state_bytes = m.state_floats * sizeof(float);
+  s->pgemm_ws_bytes = wide(s) ? 0 : gemm_block_workspace_bytes(static_cast<uint32_t>(std::max<uint64_t>({H, m.max_in, m.max_ff})));
+  Carver c;
+  const uint64_t off_cache = c.take(m.cache_bytes), off_tables = c.take(m.table_entries * 4ull), off_rec = c.take(s->stack_state_bytes);
+  const uint64_t off_prompt = c.take(s->max_ctx * 4ull), off_slots = c.take(static_cast<uint64_t>(s->max_ctx) * sizeof(Slot)),
+                 off_state = c.take(64);
+  const uint64_t off_x = c.take(H * 4), off_r = c.take(H * 4), off_y = c.take(H * 4), off_in = c.take(m.max_in * 4ull),
+                 off_logits = c.take(V * 4), off_mix16 = c.take(m.max_mix * 2ull), off_ff16 = c.take(m.max_ff * 2ull);
+  const uint64_t angles = m.angle_step.size();
+  const uint64_t off_angles = c.take(angles * 12 + 4);
+  const uint64_t off_sample_ws = c.take(sample_workspace_bytes()), off_sampler_dev = c.take(sizeof(SamplerDev)),
+                 off_sampler_keys = c.take(sampler_workspace_bytes(s->vocab));
+  const uint64_t off_px = c.take(T * H * 4), off_py = c.take(T * H * 4), off_pin = c.take(T * m.max_in * 4),
+                 off_pxn = c.take(T * H * es), off_pmix = c.take(T * m.max_mix * es), off_pff = c.take(T * m.max_ff * es),
+                 off_prope = c.take(T * m.rotation_columns * 4ull + 4), off_pgemm = c.take(s->pgemm_ws_bytes);
+  const uint64_t off_want = c.take(kStackWantedRows * H * es), off_want_rows = c.take(kStackWantedRows * 4ull),
+                 off_want_logits = c.take(kStackWantedRows * V * 4ull);
+  s->state_bytes = c.offset;
+  hipError_t err = allocate_session(s, failure_stage, with_weights);
+  if (err != hipSuccess) return err;
+  *failure_stage = 5;
+  const auto f32 = [&](uint64_t off) { return reinterpret_cast<float *>(s->arena + off); };
+  s->stack_cache = s->arena + off_cache;
+  s->stack_tables = reinterpret_cast<uint32_t *>(s->arena + off_tables);
+  s->stack_state = f32(off_rec);
+  s->prompt = reinterpret_cast<uint32_t *>(s->arena + off_prompt);
+  s->slots = reinterpret_cast<Slot *>(s->arena + off_slots);
+  s->state = reinterpret_cast<uint32_t *>(s->arena + off_state);
+  s->x = f32(off_x);
+  s->r = f32(off_r);
+  s->y = f32(off_y);
+  s->qkv = f32(off_in);
+  s->logits = f32(off_logits);
+  s->attn16 = reinterpret_cast<uint16_t *>(s->arena + off_mix16);
+  s->ff16 = reinterpret_cast<uint16_t *>(s->arena + off_ff16);
+  s->rope_freq = f32(off_angles);
+  s->sample_ws = s->arena + off_sample_ws;
+  s->sampler_dev = reinterpret_cast<SamplerDev *>(s->arena + off_sampler_dev);
+  s->sampler_keys = reinterpret_cast<uint64_t *>(s->arena + off_sampler_keys);
+  s->px = f32(off_px);
+  s->py = f32(off_py);
+  s->pqkv = f32(off_pin);
+  s->pxn = s->arena + off_pxn;
+  s->pmix = s->arena + off_pmix;
+  s->pff = s->arena + off_pff;
+  s->prope = f32(off_prope);
+  s->pgemm_ws = s->arena + off_pgemm;
+  s->pwant = s->arena + off_want;
+  s->pwant_rows = reinterpret_cast<uint32_t *>(s->arena + off_want_rows);
+  s->pwant_logits = f32(off_want_logits);
+
+  std::vector<uint32_t> tables(m.table_entries);
+  for (const StackLayer &w : m.layers)
+    if (w.own_cache())
+      for (uint32_t b = 0; b < m.logical_blocks; ++b) tables[w.table_offset + b] = b % w.ring_blocks;
+  if (!tables.empty()) err = hipMemcpy(s->stack_tables, tables.data(), tables.size() * 4, hipMemcpyHostToDevice);
+  if (err == hipSuccess && angles != 0) {
+    err = hipMemcpy(s->rope_freq, m.angle_step.data(), angles * 4, hipMemcpyHostToDevice);
+    if (err == hipSuccess) err = hipMemcpy(s->rope_freq + angles, m.angle_cos.data(), angles * 4, hipMemcpyHostToDevice);
+    if (err == hipSuccess) err = hipMemcpy(s->rope_freq + 2 * angles, m.angle_sin.data(), angles * 4, hipMemcpyHostToDevice);
+  }
+  if (err == hipSuccess) err = hipMemsetAsync(s->stack_cache, 0, m.cache_bytes, s->stream);
+  if (err == hipSuccess && s->stack_state_bytes != 0) err = hipMemsetAsync(s->stack_state, 0, s->stack_state_bytes, s->stream);
+  if (err == hipSuccess) err = hipMemsetAsync(s->slots, 0, static_cast<uint64_t>(s->max_ctx) * sizeof(Slot), s->stream);
+  if (err == hipSuccess) err = hipMemsetAsync(s->state, 0, 64, s->stream);
+  if (err == hipSuccess) err = hipMemsetAsync(s->sample_ws, 0, sample_workspace_bytes(), s->stream);
+  if (err == hipSuccess) err = hipMemsetAsync(s->sampler_dev, 0, sizeof(SamplerDev), s->stream);
+  if (err == hipSuccess) err = hipStreamSynchronize(s->stream);
+  return err;
+}
+
+extern "C" {
+
+int nerva_hip_stack_session_create(const NervaHipStackSessionCreateRequest *request, NervaHipHfDecodeSequenceSessionCreateResult *out,
+                                   NervaHipHfDecodeSequenceSession **session) {
+  return create_stack(request, false, 0, 0.0f, out, session);
+}
+
+int nerva_hip_bench_stack_session_create_synthetic(const NervaHipStackSessionCreateRequest *request, uint64_t seed, float weight_std,
+                                                   NervaHipHfDecodeSequenceSessionCreateResult *out,
+                                                   NervaHipHfDecodeSequenceSession **session) {
+  return create_stack(request, true, seed, weight_std, out, session);
+}
+
+}  // extern "C"

@@ -61,7 +61,10 @@ _ARENA_ORDER = ("rms_attn", "w_q", "q_norm", "w_k", "k_norm", "w_v", "w_o", "rms
 
 def arena_order(weights):
     """The model's tensors in the order the reference lays its weight arena out, which is the byte
-    space weight descriptors address (weights.cu:484-591, session_api_lifecycle.inc.cu:124-148)."""
+    space weight descriptors address (weights.cu:484-591, session_api_lifecycle.inc.cu:124-148); a
+    mixed stack's weights know their own order."""
+    if hasattr(weights, "arena_tensors"):
+        return weights.arena_tensors()
     out = [weights.embeddings]
     for layer in weights.layers:
         out += [layer[k] for k in _ARENA_ORDER if layer.get(k) is not None]
@@ -200,6 +203,45 @@ class DecodeSession:
                                % (res.status, res.hip_error, res.failure_stage))
         return cls(handle, res, cfg["vocab"], cfg["kv_heads"] * cfg["head_dim"])
 
+    @staticmethod
+    def _stack_request(config, max_context, precision):
+        req = abi.NervaHipStackSessionCreateRequest()
+        req.dtype, req.precision, req.hidden, req.vocab_size = 1, precision, config.hidden, config.vocab
+        req.layer_count, req.max_context_tokens, req.norm_eps = len(config.layers), max_context, config.eps
+        layers = config.c_layers()
+        req.layers = layers
+        return req, layers
+
+    @classmethod
+    def _created_stack(cls, rc, res, handle, config):
+        if rc != 0:
+            raise RuntimeError("stack session_create failed: status=%d hip_error=%d stage=%d"
+                               % (res.status, res.hip_error, res.failure_stage))
+        return cls(handle, res, config.vocab, 0)
+
+    @classmethod
+    def create_stack(cls, config, plan, max_context, precision=0, **extra):
+        """A session over a mixed layer stack (stacks.StackConfig) whose weights `plan` describes."""
+        lib = abi.load()
+        req, layers = cls._stack_request(config, max_context, precision)
+        for k, v in list(plan.fields().items()) + list(extra.items()):
+            setattr(req, k, v)
+        res = abi.NervaHipHfDecodeSequenceSessionCreateResult()
+        handle = C.POINTER(abi.NervaHipHfDecodeSequenceSession)()
+        rc = lib.nerva_hip_stack_session_create(C.byref(req), C.byref(res), C.byref(handle))
+        return cls._created_stack(rc, res, handle, config)
+
+    @classmethod
+    def create_stack_synthetic(cls, config, max_context, seed=0x4E45525641, weight_std=0.02, weight_hash=0, precision=0):
+        """The same over device-generated weights."""
+        lib = abi.load()
+        req, layers = cls._stack_request(config, max_context, precision)
+        req.planned_weight_descriptor_hash = weight_hash
+        res = abi.NervaHipHfDecodeSequenceSessionCreateResult()
+        handle = C.POINTER(abi.NervaHipHfDecodeSequenceSession)()
+        rc = lib.nerva_hip_bench_stack_session_create_synthetic(C.byref(req), seed, weight_std, C.byref(res), C.byref(handle))
+        return cls._created_stack(rc, res, handle, config)
+
     def fork_shared_weights(self, detailed_profile=False):
         """A second session on this one's resident weights (request.rs:380-407); carries a sequence
         that is under way over to the child."""
@@ -249,6 +291,27 @@ class DecodeSession:
         res = abi.NervaHipHfDecodeSequenceResult()
         rc = self.lib.nerva_hip_hf_decode_sequence_session_start(C.byref(req), C.byref(res))
         return rc, res
+
+    def extend(self, tokens, wanted=(), residual_layers=0):
+        """Appends given tokens to the sequence (or begins one). Returns (rc, result, logits [wanted, vocab],
+        residual rows [layers, tokens, hidden] or None)."""
+        tokens = np.ascontiguousarray(tokens, np.uint32)
+        places = np.ascontiguousarray(wanted, np.uint32)
+        logits = np.empty((places.size, self.vocab), np.float32)
+        req = abi.NervaHipSessionExtendRequest()
+        req.session, req.tokens, req.token_count = self.handle, tokens.ctypes.data, tokens.size
+        req.wanted, req.wanted_count, req.logits = places.ctypes.data, places.size, logits.ctypes.data
+        residuals = None
+        if residual_layers:
+            residuals = np.empty((residual_layers, tokens.size, self.create_result.hidden), np.float32)
+            req.residuals = residuals.ctypes.data
+        res = abi.NervaHipHfDecodeSequenceResult()
+        rc = self.lib.nerva_hip_session_extend(C.byref(req), C.byref(res))
+        return rc, res, logits, residuals
+
+    def release_sequence(self):
+        """Ends the sequence; the session is free for the next one."""
+        return self.lib.nerva_hip_session_release_sequence(self.handle)
 
     def advance(self, steps, capacity=None):
         out = np.zeros(capacity if capacity is not None else steps, np.uint32)
