@@ -209,6 +209,9 @@ def main():
                     help="prompt block size (0 = the session's choice: 512 tokens at these widths)")
     ap.add_argument("--copy-probe-mib", type=int, default=0,
                     help="also launch one plain copy kernel of this size (memory-counter calibration runs)")
+    ap.add_argument("--stack", nargs="?", const="all", default=None, metavar="SIZE",
+                    help="instead of the workload: a mixed layer stack beside the uniform decoder, at one size of "
+                         "nerva_amd/stackbench.py or at all of them")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py measures one GPU: this path is a single-device decode loop and no multi-GPU "
@@ -220,6 +223,10 @@ def main():
     if rc != 0:
         log("no usable GPU (hip_error=%d): the HIP path cannot run, and there is no CPU fallback" % smoke.hip_error)
         sys.exit(1)
+    if args.stack is not None:
+        from nerva_amd import stackbench
+        stackbench.run(args.prompt, args.steps, args.warmup, None if args.stack == "all" else [args.stack])
+        return
     if args.prefill_block in (128, 256):
         N.Device.set_tuning("prefill_block_tokens", args.prefill_block)
     cfg = dict(N.Qwen3_8B)

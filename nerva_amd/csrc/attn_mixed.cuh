@@ -43,7 +43,7 @@ struct MixedAttnParams {
   uint16_t *out16;             // [tokens][heads * value_dim], or null
   float *out32;                // likewise f32, used when out16 is null
   uint32_t packed_tiles;       // out16: != 0 -> matrix-operand order with that many token tiles
-  void *workspace;             // the wide kernels' split partials (mixed_attn_workspace_bytes)
+  void *workspace;             // the wide kernels' split partials (mixed_attention_workspace_bytes)
   uint32_t last_block;         // highest logical block a launch may meet (sizes the split grid of a captured step)
 };
 
@@ -51,6 +51,12 @@ struct MixedAttnParams {
 hipError_t launch_mixed_publish(uint32_t dtype, const MixedAttnParams &p, hipStream_t stream);
 // Attention of the token rows, whose own keys and values are in the cache. Any shape.
 hipError_t launch_mixed_attention(uint32_t dtype, const MixedAttnParams &p, hipStream_t stream);
+// Wide layers, 16-bit cache (attn_mixed_wide.hip): rotation, cache rows (append) and attention of a decode step (cursor
+// set, one token: two launches) or of a block of token rows (three launches).
+bool mixed_attention_wide(uint32_t heads, uint32_t kv_heads, uint32_t key_dim, uint32_t value_dim);
+uint64_t mixed_attention_workspace_bytes(uint32_t heads, uint32_t max_tokens);
+hipError_t launch_mixed_attention_wide(uint32_t dtype, const MixedAttnParams &p, bool append, hipStream_t stream);
+
 constexpr uint32_t kMixedMaxValueDim = 1024;
 constexpr uint32_t kMixedMaxFolded = 12288;   // kv_heads * key_dim (the folded query lies in LDS as f32)
 

@@ -123,6 +123,20 @@ MixedAttnParams attention_params(Session *s, const StackLayer &layer, const floa
   return a;
 }
 
+// Rotation, cache rows, attention of the token rows in `a`.
+bool takes_wide(const Session *s, const StackLayer &w) {
+  return !wide(s) && mixed_attention_wide(w.spec.heads, w.spec.kv_heads, w.spec.key_dim, w.spec.value_dim) &&
+         tuning(kTuneMixedAttentionWide) != 2;
+}
+uint32_t attention_launches(const Session *s, const StackLayer &w, bool decode) {
+  return takes_wide(s, w) ? (decode ? 2u : 3u) : (w.own_cache() ? 2u : 1u);
+}
+hipError_t attend(Session *s, const StackLayer &w, const MixedAttnParams &a) {
+  if (takes_wide(s, w)) return launch_mixed_attention_wide(s->dtype, a, w.own_cache(), s->stream);
+  hipError_t err = w.own_cache() ? launch_mixed_publish(s->dtype, a, s->stream) : hipSuccess;
+  return err == hipSuccess ? launch_mixed_attention(s->dtype, a, s->stream) : err;
+}
+
 // Final norm, head, sampler of the row in (row.x, s->y): logits, slot[cursor], cursor + 1.
 hipError_t decode_head(Session *s, DecodeRow &row) {
   const StackModel &m = *s->stack;
@@ -173,8 +187,7 @@ hipError_t decode_step_16(Session *s) {
       a.cursor = s->state;
       a.tokens = 1;
       a.out16 = s->attn16;
-      if (err == hipSuccess && w.own_cache()) err = launch_mixed_publish(s->dtype, a, st);
-      if (err == hipSuccess) err = launch_mixed_attention(s->dtype, a, st);
+      if (err == hipSuccess) err = attend(s, w, a);
     } else {
       p.rows = w.spec.width;
       p.out16 = s->attn16;
@@ -303,11 +316,8 @@ struct Block {
       if (wide(s)) a.out32 = static_cast<float *>(s->pmix);
       else a.out16 = static_cast<uint16_t *>(s->pmix);
       a.packed_tiles = out_tiles;
-      if (w.own_cache()) {
-        err = launch_mixed_publish(s->dtype, a, s->stream);
-        launches += 1;
-      }
-      if (err == hipSuccess) err = launch_mixed_attention(s->dtype, a, s->stream);
+      err = attend(s, w, a);
+      launches += attention_launches(s, w, false) - 1;
     } else {
       MinGruRows g{};
       g.zxg = s->pqkv;
@@ -421,7 +431,7 @@ uint64_t nv::stack_step_launches(const Session *s) {
   uint64_t n = 1 + (wide(s) ? 4 : s->sampler.mode == kSamplerGreedy ? 2 : 3);
   for (const StackLayer &w : s->stack->layers) {
     const uint64_t seam = wide(s) ? 1 : 0;
-    n += seam + (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION ? (w.own_cache() ? 4 : 3) : (wide(s) ? 3 : 2));
+    n += seam + (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION ? 2 + attention_launches(s, w, true) : (wide(s) ? 3 : 2));
     if (w.spec.ff != 0) n += seam + 2;
   }
   return n;
@@ -795,6 +805,12 @@ hipError_t nv::stack_setup_state(Session *s, int32_t *failure_stage, bool with_w
   const uint64_t off_px = c.take(T * H * 4), off_py = c.take(T * H * 4), off_pin = c.take(T * m.max_in * 4),
                  off_pxn = c.take(T * H * es), off_pmix = c.take(T * m.max_mix * es), off_pff = c.take(T * m.max_ff * es),
                  off_prope = c.take(T * m.rotation_columns * 4ull + 4), off_pgemm = c.take(s->pgemm_ws_bytes);
+  uint64_t attn_ws_bytes = 0;
+  for (const StackLayer &w : m.layers)
+    if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION && !wide(s) &&
+        mixed_attention_wide(w.spec.heads, w.spec.kv_heads, w.spec.key_dim, w.spec.value_dim))
+      attn_ws_bytes = std::max(attn_ws_bytes, mixed_attention_workspace_bytes(w.spec.heads, kStackBlockTokens));
+  const uint64_t off_attn_ws = c.take(attn_ws_bytes);
   const uint64_t off_want = c.take(kStackWantedRows * H * es), off_want_rows = c.take(kStackWantedRows * 4ull),
                  off_want_logits = c.take(kStackWantedRows * V * 4ull);
   s->state_bytes = c.offset;
@@ -827,6 +843,7 @@ hipError_t nv::stack_setup_state(Session *s, int32_t *failure_stage, bool with_w
   s->pff = s->arena + off_pff;
   s->prope = f32(off_prope);
   s->pgemm_ws = s->arena + off_pgemm;
+  s->attn_ws = s->arena + off_attn_ws;
   s->pwant = s->arena + off_want;
   s->pwant_rows = reinterpret_cast<uint32_t *>(s->arena + off_want_rows);
   s->pwant_logits = f32(off_want_logits);

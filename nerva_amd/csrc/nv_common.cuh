@@ -169,6 +169,7 @@ enum TuningKnob : int {
   kTuneGemmBlockOff,         // 1 = blocks of up to 128 rows use gemm_rows_kernel, never the shared-X kernel
   kTuneGemmBlockWaves,       // shared-X GEMM, gate/up pairs of up to 64 token rows: 4 = never three-wave workgroups
   kTuneGemmBlockRotate,      // shared-X GEMM: 1 + the K-blocks between the starts of consecutive row groups (1: a common start)
+  kTuneMixedAttentionWide,   // mixed stacks: 2 = every attention layer through the general kernel
   kTuneKnobs
 };
 int tuning(TuningKnob knob);

@@ -34,15 +34,14 @@ def xielu(z, p, q):
     return np.where(z > 0.0, softplus(p) * z * z, (softplus(q) + 0.5) * (np.expm1(below) - below)) + 0.5 * z
 
 
-def rotate(head, position, dims, base):
-    """`head` [dim] turned pair by pair; element i goes with element i + dims/2, the rest stays."""
-    out = np.array(head)
-    half = dims // 2
-    for i in range(half):
-        angle = position * base ** (-2.0 * i / dims)
-        u, v = head[i], head[i + half]
-        out[i] = u * np.cos(angle) - v * np.sin(angle)
-        out[i + half] = v * np.cos(angle) + u * np.sin(angle)
+def rotate(heads, position, dims, base):
+    """heads [n, dim] turned pair by pair; element i goes with element i + dims/2, elements from `dims` on stay."""
+    out, half = np.array(heads), dims // 2
+    if half:
+        angle = position * base ** (-2.0 * np.arange(half) / dims)
+        u, v = heads[:, :half], heads[:, half:dims]
+        out[:, :half] = u * np.cos(angle) - v * np.sin(angle)
+        out[:, half:dims] = v * np.cos(angle) + u * np.sin(angle)
     return out
 
 
@@ -79,11 +78,9 @@ def attention_mixer(h, mixer, w, cache, first):
     out = []
     for t, row in enumerate(h):
         p = first + t
-        q = (w["q"] @ row).reshape(H, d)
-        q = np.stack([rotate(x, p, rot["dims"], rot["base"]) for x in q])
+        q = rotate((w["q"] @ row).reshape(H, d), p, rot["dims"], rot["base"])
         if "k" in w:
-            k = (w["k"] @ row).reshape(G, d)
-            cache["k"].append(np.stack([rotate(x, p, rot["dims"], rot["base"]) for x in k]))
+            cache["k"].append(rotate((w["k"] @ row).reshape(G, d), p, rot["dims"], rot["base"]))
             cache["v"].append((w["v"] @ row).reshape(G, dv))
         lo = first_visible(p, mixer["mask"]["size"])
         o = attend(q, np.stack(cache["k"][lo:p + 1]), np.stack(cache["v"][lo:p + 1]), mixer["scale"], w["talk"], w["sink"])
