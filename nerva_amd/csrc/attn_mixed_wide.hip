@@ -30,7 +30,7 @@ namespace {
 
 using namespace attn;
 
-constexpr uint32_t kDecodeSplits = 128, kMinBlocksPerSplit = 2;
+constexpr uint32_t kDecodeSplits = 256, kMinBlocksPerSplit = 2;
 constexpr uint32_t kPromptTokens = 8;          // tokens of a workgroup
 constexpr uint32_t kPromptWorkgroups = 256;    // split the keys until about so many are there
 constexpr uint32_t kPromptSplits = 64;
@@ -75,6 +75,10 @@ __device__ __forceinline__ float rotated_elem(const float *head, const float *cs
   return d < half ? head[d] * cs[d] - head[d + half] * cs[half + d] : head[d] * cs[d - half] + head[d - half] * cs[d];
 }
 
+__device__ __forceinline__ uint32_t pack16(float a, float b) {
+  return enc16_finite<kBF16>(a) | (static_cast<uint32_t>(enc16_finite<kBF16>(b)) << 16);
+}
+
 // ---- decode step -----------------------------------------------------------------------------
 
 constexpr uint32_t kKeysPitch = 68;   // floats of a head's 64 scores in LDS
@@ -83,7 +87,7 @@ __global__ __launch_bounds__(512, 2) void mixed_decode_kernel(MixedAttnParams p,
   constexpr uint32_t DT = kBF16;
   extern __shared__ __align__(16) float lds[];
   const uint32_t H = p.heads;
-  float *s_s = lds, *t_s = s_s + H * kKeysPitch;
+  float *s_s = lds, *t_s = s_s + H * kHD;   // (the scores' room holds the queries first: 128 floats a head)
   uint16_t *w_s = reinterpret_cast<uint16_t *>(t_s + H * H);   // [hi | lo][head][64]
   const uint32_t pos = p.cursor != nullptr ? *p.cursor : p.position;
   if (p.cursor != nullptr && pos >= p.max_steps) return;
@@ -106,15 +110,35 @@ __global__ __launch_bounds__(512, 2) void mixed_decode_kernel(MixedAttnParams p,
     }
     __threadfence_block();   // (a wave reads back only the tiles of its own kv head)
   }
-  for (uint32_t i = threadIdx.x; i < H * H; i += blockDim.x)
-    t_s[i] = p.talk != nullptr ? dec16<DT>(p.talk[i]) : (i / H == i % H ? 1.0f : 0.0f);
+  uint4 kreg[4][4], vreg[4][4];
+  const auto request = [&](uint32_t b) {
+#pragma unroll
+    for (uint32_t t = 0; t < 4; ++t) {
+      const uint64_t tile = kv_tile_offset(0, p.kv_heads, kHD, 0, p.table[min(b + t, b1 - 1)], c) + lane * 8u;
+#pragma unroll
+      for (uint32_t j = 0; j < 4; ++j) kreg[t][j] = *reinterpret_cast<const uint4 *>(kc + tile + j * 512u);
+#pragma unroll
+      for (uint32_t j = 0; j < 4; ++j) vreg[t][j] = *reinterpret_cast<const uint4 *>(vc + tile + j * 512u);
+    }
+  };
+  request(b0);   // the first four blocks are on their way while the queries are prepared
 
-  // queries of this kv head: columns 0..R-1 hi halves, 8..8+R-1 lo halves
+  for (uint32_t i = threadIdx.x; i < H * H; i += blockDim.x)   // M transposed: a wave's heads of one source lie together
+    t_s[i % H * H + i / H] = p.talk != nullptr ? dec16<DT>(p.talk[i]) : (i / H == i % H ? 1.0f : 0.0f);
+  // queries of this kv head, rotated and scaled, through LDS (the scores' room): columns 0..R-1 hi halves, 8..8+R-1 lo
+  float *q_s = s_s + c * R * kHD;
+#pragma unroll
+  for (int r = 0; r < R; ++r)
+#pragma unroll
+    for (uint32_t i = 0; i < 2; ++i) {
+      const uint32_t d = lane + 64u * i;
+      q_s[r * kHD + d] = rotated_elem(p.proj + p.q_col + (c * R + r) * kHD, p.rope_cs, p.rot_dims, d) * (p.scale * kLog2e);
+    }
+  __syncthreads();
   uint4 qx[4];
   {
     const uint32_t r = n & 7u;
-    const float *head = p.proj + p.q_col + (c * R + min(r, static_cast<uint32_t>(R - 1))) * kHD;
-    const float scale = p.scale * kLog2e;
+    const float *head = q_s + min(r, static_cast<uint32_t>(R - 1)) * kHD;
 #pragma unroll
     for (uint32_t j = 0; j < 4; ++j) {
       uint32_t w[4];
@@ -122,13 +146,14 @@ __global__ __launch_bounds__(512, 2) void mixed_decode_kernel(MixedAttnParams p,
       for (uint32_t e = 0; e < 4; ++e) {
         const uint32_t d = j * 32u + q4 * 8u + 2u * e;
         uint16_t h0, l0, h1, l1;
-        split16<DT>(rotated_elem(head, p.rope_cs, p.rot_dims, d) * scale, h0, l0);
-        split16<DT>(rotated_elem(head, p.rope_cs, p.rot_dims, d + 1) * scale, h1, l1);
+        split16<DT>(head[d], h0, l0);
+        split16<DT>(head[d + 1], h1, l1);
         w[e] = n < 8u ? (h0 | (static_cast<uint32_t>(h1) << 16)) : (l0 | (static_cast<uint32_t>(l1) << 16));
       }
       qx[j] = r < static_cast<uint32_t>(R) ? make_uint4(w[0], w[1], w[2], w[3]) : make_uint4(0u, 0u, 0u, 0u);
     }
   }
+  __syncthreads();   // the scores take the queries' room
 
   const uint32_t lo = first_seen(p, pos);
   float m[R], l[R];
@@ -142,15 +167,7 @@ __global__ __launch_bounds__(512, 2) void mixed_decode_kernel(MixedAttnParams p,
   for (int s = 0; s < 8; ++s) acc[s] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
 
   for (uint32_t b = b0; b < b1; b += 4) {
-    uint4 kreg[4][4], vreg[4][4];
-#pragma unroll
-    for (uint32_t t = 0; t < 4; ++t) {
-      const uint64_t tile = kv_tile_offset(0, p.kv_heads, kHD, 0, p.table[min(b + t, b1 - 1)], c) + lane * 8u;
-#pragma unroll
-      for (uint32_t j = 0; j < 4; ++j) kreg[t][j] = *reinterpret_cast<const uint4 *>(kc + tile + j * 512u);
-#pragma unroll
-      for (uint32_t j = 0; j < 4; ++j) vreg[t][j] = *reinterpret_cast<const uint4 *>(vc + tile + j * 512u);
-    }
+    if (b != b0) request(b);
 #pragma unroll
     for (uint32_t t = 0; t < 4; ++t) {
       f32x4_t s = {0.0f, 0.0f, 0.0f, 0.0f};
@@ -171,7 +188,7 @@ __global__ __launch_bounds__(512, 2) void mixed_decode_kernel(MixedAttnParams p,
     for (uint32_t g = 0; g < H; ++g) {
       const float s = s_s[g * kKeysPitch + lane];
 #pragma unroll
-      for (int r = 0; r < R; ++r) mixed[r] = fmaf(t_s[(c * R + r) * H + g], s, mixed[r]);
+      for (int r = 0; r < R; ++r) mixed[r] = fmaf(t_s[g * H + c * R + r], s, mixed[r]);
     }
     float keep[R];
 #pragma unroll
@@ -251,10 +268,6 @@ __global__ __launch_bounds__(kBlock) void mixed_prepare_kernel(MixedAttnParams p
 // Scores in LDS: [key of 32][token of 8][head of 32], the pitches chosen so that a wave's accesses spread over the banks.
 constexpr uint32_t kTokenPitch = kWideHeads + 4, kKeyPitch = kPromptTokens * kTokenPitch + 4;
 constexpr size_t kPromptLds = 2u * 32u * kKeyPitch * sizeof(float);
-
-__device__ __forceinline__ uint32_t pack16(float a, float b) {
-  return enc16_finite<kBF16>(a) | (static_cast<uint32_t>(enc16_finite<kBF16>(b)) << 16);
-}
 
 template <int R>
 __global__ __launch_bounds__(512, 2) void mixed_prompt_kernel(MixedAttnParams p, const uint16_t *q16, uint32_t splits) {
@@ -439,47 +452,99 @@ __global__ __launch_bounds__(512, 2) void mixed_prompt_kernel(MixedAttnParams p,
 
 // ---- merge -----------------------------------------------------------------------------------
 
-// Grid (head, token): PARTS groups of 128 lanes share the splits.
-template <int PARTS, bool PROMPT>
-__global__ __launch_bounds__(PARTS *kHD) void mixed_merge_kernel(MixedAttnParams p, uint32_t splits) {
-  constexpr uint32_t DT = kBF16;
-  __shared__ float f_s[kDecodeSplits], sum_s[PARTS][kHD];
-  const uint32_t h = blockIdx.x, t = blockIdx.y, d = threadIdx.x % kHD, part = threadIdx.x / kHD, H = p.heads;
-  uint32_t active;
-  if constexpr (PROMPT) {
-    active = prompt_range(p, t / kPromptTokens, splits).active;
-  } else {
-    const uint32_t pos = p.cursor != nullptr ? *p.cursor : p.position;
-    if (p.cursor != nullptr && pos >= p.max_steps) return;
-    active = decode_range(p, pos, splits).active;
+__device__ __forceinline__ void merged_store(const MixedAttnParams &p, uint32_t t, uint32_t e, float4 o) {
+  if (p.gate_col != kNoColumn) {
+    const float4 g = *reinterpret_cast<const float4 *>(p.proj + static_cast<uint64_t>(t) * p.proj_stride + p.gate_col + e);
+    o.x *= sigmoid(g.x);
+    o.y *= sigmoid(g.y);
+    o.z *= sigmoid(g.z);
+    o.w *= sigmoid(g.w);
   }
+  uint16_t *out = p.out16 + (p.packed_tiles != 0 ? gemm_x_packed_index(p.packed_tiles, t, e) : static_cast<uint64_t>(t) * p.heads * kHD + e);
+  *reinterpret_cast<uint2 *>(out) = make_uint2(pack16(o.x, o.y), pack16(o.z, o.w));   // (four columns stay together in operand order)
+}
+
+// Decode step: one workgroup per head; sixteen groups of 32 lanes share the splits, four columns a lane.
+constexpr uint32_t kMergeGroups = 16;
+__global__ __launch_bounds__(kMergeGroups * 32) void mixed_decode_merge_kernel(MixedAttnParams p, uint32_t splits) {
+  __shared__ float f_s[kDecodeSplits], red[kMergeGroups * 32 / kWave];
+  __shared__ float4 sum_s[kMergeGroups][32];
+  const uint32_t h = blockIdx.x, H = p.heads, tid = threadIdx.x, group = tid / 32u, c4 = tid % 32u;
+  const uint32_t pos = p.cursor != nullptr ? *p.cursor : p.position;
+  if (p.cursor != nullptr && pos >= p.max_steps) return;
+  const uint32_t active = decode_range(p, pos, splits).active;
+  const Partials in = partials_of(p.workspace, static_cast<uint64_t>(splits) * H);
+  const float sink = p.sink != nullptr ? dec16<kBF16>(p.sink[h]) * kLog2e : -INFINITY;
+  // one split a lane (kDecodeSplits lanes are enough)
+  const float ms = tid < active ? in.m[tid * H + h] : -INFINITY, ls = tid < active ? in.l[tid * H + h] : 0.0f;
+  float top = wave_max(ms);
+  if (tid % kWave == 0) red[tid / kWave] = top;
+  __syncthreads();
+  top = sink;
+#pragma unroll
+  for (uint32_t w = 0; w < kMergeGroups * 32 / kWave; ++w) top = fmaxf(top, red[w]);
+  const float f = tid < active ? attn_exp2(ms - top) : 0.0f;
+  if (tid < kDecodeSplits) f_s[tid] = f;
+  const float part = wave_sum(ls * f);
+  __syncthreads();
+  if (tid % kWave == 0) red[tid / kWave] = part;
+  __syncthreads();
+  float total = p.sink != nullptr ? attn_exp2(sink - top) : 0.0f;
+#pragma unroll
+  for (uint32_t w = 0; w < kMergeGroups * 32 / kWave; ++w) total += red[w];
+  float4 o = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+#pragma unroll 8
+  for (uint32_t s = group; s < active; s += kMergeGroups) {
+    const float4 v = *reinterpret_cast<const float4 *>(in.sum + (static_cast<uint64_t>(s) * H + h) * kHD + c4 * 4u);
+    const float w = f_s[s];
+    o.x = fmaf(v.x, w, o.x);
+    o.y = fmaf(v.y, w, o.y);
+    o.z = fmaf(v.z, w, o.z);
+    o.w = fmaf(v.w, w, o.w);
+  }
+  sum_s[group][c4] = o;
+  __syncthreads();
+  if (group != 0) return;
+#pragma unroll
+  for (uint32_t i = 1; i < kMergeGroups; ++i) {
+    const float4 v = sum_s[i][c4];
+    o.x += v.x;
+    o.y += v.y;
+    o.z += v.z;
+    o.w += v.w;
+  }
+  const float inv = 1.0f / total;
+  merged_store(p, 0, h * kHD + c4 * 4u, make_float4(o.x * inv, o.y * inv, o.z * inv, o.w * inv));
+}
+
+// Prompt blocks: 32 lanes per (token, head), four columns a lane, the splits in order.
+__global__ __launch_bounds__(kBlock) void mixed_prompt_merge_kernel(MixedAttnParams p, uint32_t splits) {
+  const uint32_t H = p.heads, id = blockIdx.x * (kBlock / 32u) + threadIdx.x / 32u, c4 = threadIdx.x % 32u;
+  const uint32_t t = id / H, h = id % H;
+  if (t >= p.tokens) return;
+  const uint32_t active = prompt_range(p, t / kPromptTokens, splits).active;
   const Partials in = partials_of(p.workspace, static_cast<uint64_t>(p.tokens) * splits * H);
   const uint64_t base = static_cast<uint64_t>(t) * splits * H + h;
-  const float sink = p.sink != nullptr ? dec16<DT>(p.sink[h]) * kLog2e : -INFINITY;
-  float top = sink;
-  for (uint32_t s = 0; s < active; ++s) top = fmaxf(top, in.m[base + static_cast<uint64_t>(s) * H]);
-  float total = p.sink != nullptr ? attn_exp2(sink - top) : 0.0f;
+  float top = p.sink != nullptr ? dec16<kBF16>(p.sink[h]) * kLog2e : -INFINITY;
+  float total = p.sink != nullptr ? 1.0f : 0.0f;
+  float4 o = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+#pragma unroll 4
   for (uint32_t s = 0; s < active; ++s) {
-    const float ms = in.m[base + static_cast<uint64_t>(s) * H];
-    const float f = ms > -INFINITY ? attn_exp2(ms - top) : 0.0f;
-    total = fmaf(in.l[base + static_cast<uint64_t>(s) * H], f, total);
-    if (threadIdx.x == 0) f_s[s] = f;
+    const uint64_t at = base + static_cast<uint64_t>(s) * H;
+    const float ms = in.m[at], ls = in.l[at];
+    const float4 v = *reinterpret_cast<const float4 *>(in.sum + at * kHD + c4 * 4u);
+    const float next = fmaxf(top, ms);
+    const float keep = top > -INFINITY ? attn_exp2(top - next) : 0.0f;
+    const float f = ms > -INFINITY ? attn_exp2(ms - next) : 0.0f;   // (a token may have seen no key of a split)
+    top = next;
+    total = total * keep + ls * f;
+    o.x = o.x * keep + v.x * f;
+    o.y = o.y * keep + v.y * f;
+    o.z = o.z * keep + v.z * f;
+    o.w = o.w * keep + v.w * f;
   }
-  __syncthreads();
-  float o = 0.0f;
-#pragma unroll 8
-  for (uint32_t s = part; s < active; s += PARTS) o = fmaf(in.sum[(base + static_cast<uint64_t>(s) * H) * kHD + d], f_s[s], o);
-  if constexpr (PARTS > 1) {
-    sum_s[part][d] = o;
-    __syncthreads();
-    if (part != 0) return;
-#pragma unroll
-    for (int i = 1; i < PARTS; ++i) o += sum_s[i][d];
-  }
-  o = total > 0.0f ? o / total : 0.0f;
-  const uint32_t e = h * kHD + d;
-  if (p.gate_col != kNoColumn) o *= sigmoid(p.proj[static_cast<uint64_t>(t) * p.proj_stride + p.gate_col + e]);
-  p.out16[p.packed_tiles != 0 ? gemm_x_packed_index(p.packed_tiles, t, e) : static_cast<uint64_t>(t) * H * kHD + e] = enc16<DT>(o);
+  const float inv = 1.0f / total;
+  merged_store(p, t, h * kHD + c4 * 4u, make_float4(o.x * inv, o.y * inv, o.z * inv, o.w * inv));
 }
 
 uint32_t decode_splits(const MixedAttnParams &p) {
@@ -495,11 +560,11 @@ uint64_t partial_bytes(uint64_t entries) { return entries * (kHD + 2) * sizeof(f
 template <int R>
 hipError_t launch_decode(const MixedAttnParams &p, uint32_t append, hipStream_t stream) {
   const uint32_t splits = decode_splits(p);
-  const size_t lds = (p.heads * kKeysPitch + p.heads * p.heads) * sizeof(float) + 2u * p.heads * 64u * sizeof(uint16_t);
+  const size_t lds = (p.heads * static_cast<uint32_t>(kHD) + p.heads * p.heads) * sizeof(float) + 2u * p.heads * 64u * sizeof(uint16_t);
   hipLaunchKernelGGL(mixed_decode_kernel<R>, dim3(splits), dim3(p.kv_heads * kWave), lds, stream, p, splits, append);
   hipError_t err = hipGetLastError();
   if (err != hipSuccess) return err;
-  hipLaunchKernelGGL((mixed_merge_kernel<4, false>), dim3(p.heads, 1), dim3(4 * kHD), 0, stream, p, splits);
+  hipLaunchKernelGGL(mixed_decode_merge_kernel, dim3(p.heads), dim3(kMergeGroups * 32), 0, stream, p, splits);
   return hipGetLastError();
 }
 
@@ -522,7 +587,9 @@ hipError_t launch_prompt(const MixedAttnParams &p, uint32_t append, hipStream_t 
                      static_cast<const uint16_t *>(q16), splits);
   err = hipGetLastError();
   if (err != hipSuccess) return err;
-  hipLaunchKernelGGL((mixed_merge_kernel<1, true>), dim3(p.heads, p.tokens), dim3(kHD), 0, stream, p, splits);
+  constexpr uint32_t kRowsPerBlock = kBlock / 32u;
+  hipLaunchKernelGGL(mixed_prompt_merge_kernel, dim3((p.tokens * p.heads + kRowsPerBlock - 1) / kRowsPerBlock), dim3(kBlock), 0, stream, p,
+                     splits);
   return hipGetLastError();
 }
 

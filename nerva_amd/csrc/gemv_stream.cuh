@@ -426,7 +426,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
 // Register budget as resident waves per SIMD (= workgroups per CU): 6 with a 16-bit input,
 // 5 with the RMSNorm prologue, which holds the f32 activations and the norm weights in
 // registers across the first weight requests (a budget of 6 makes it spill), 4 with the join
-// prologue, which holds two f32 rows and the weights and biases of two norms.
+// prologue, which holds two f32 rows and the weights and biases of two norms: one 16-wave workgroup a CU.
 constexpr int fast_waves_per_simd(int prologue) { return prologue == kProJoin ? 4 : prologue == kProRmsNorm ? 5 : 6; }
 constexpr int kFastMaxCols = 12288;  // x staged through at most 6 x 16 B per lane in registers ...
 constexpr int kFastMaxColsLoop = 30720;  // ... or, with a 16-bit input, copied into LDS behind the first weight requests
@@ -468,7 +468,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   const int wave = threadIdx.x / kWave;
   const uint32_t cols = p.cols;
   const uint32_t units = p.rows;  // NR == 1: rows; kEpiSwiglu (NR == 2): gate/up pairs; kEpiMinGru (NR == 3): triples
-  const uint32_t wave_global = blockIdx.x * WG + wave;
+  // (kProJoin: consecutive units go to different workgroups - one per CU - so that every CU has the same share to a row)
+  const uint32_t wave_global = PRO == kProJoin ? wave * gridDim.x + blockIdx.x : blockIdx.x * WG + wave;
   const uint32_t wave_stride = gridDim.x * WG;
   const uint32_t bpr = cols / (kWave * 8 * B);  // request batches per row
   const uint32_t my_units = wave_global < units ? (units - wave_global + wave_stride - 1) / wave_stride : 0u;
@@ -480,7 +481,7 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   float4 xa[PRO == kProRmsNorm ? 2 : 1], xb[PRO == kProRmsNorm ? 2 : 1];
   uint4 gw[PRO == kProRmsNorm ? 2 : 1];
   const bool norm_in_regs = cols <= TB * 16;
-  JoinRegs join[PRO == kProJoin ? 2 : 1];   // (the launcher keeps cols <= TB * 16 here)
+  JoinRegs join[1];   // (kProJoin: the launcher keeps cols <= TB * 8)
   // (the same for every wave of the launch; a constant in the variant with exact start-up waits, which only
   // runs at 4096 columns, so its request counts stay countable)
   const bool x_in_regs = EXACT || cols <= static_cast<uint32_t>(kFastMaxCols);
@@ -494,8 +495,7 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
       }
     }
   } else if constexpr (PRO == kProJoin) {
-#pragma unroll
-    for (int i = 0; i < 2; ++i) join_load8(p.join, (i * TB + threadIdx.x) * 8, cols, join[i]);
+    join_load8(p.join, threadIdx.x * 8, cols, join[0]);
   } else {
     if (norm_in_regs) {
 #pragma unroll
@@ -573,7 +573,7 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
         *reinterpret_cast<uint4 *>(xs + c) = *reinterpret_cast<const uint4 *>(p.x16 + c);
     }
   } else if constexpr (PRO == kProJoin) {
-    join_norm_regs<DT, WG>(p.join, cols, blockIdx.x == 0, join, red, xs);
+    join_norm_regs<DT, WG, 1>(p.join, cols, blockIdx.x == 0, join, red, xs);
   } else {
     float ss = 0.0f;
     if (norm_in_regs) {

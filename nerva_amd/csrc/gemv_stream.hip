@@ -18,6 +18,7 @@ constexpr int kDefaultNR = 1;
 constexpr int kDefaultU = NV_GEMV_U;  // chunks of 1 KiB in flight per wave per request batch
 constexpr bool kDefaultDot2 = false;
 constexpr uint32_t kCus = 256;                     // gfx950: 8 XCDs x 32 CUs
+constexpr uint32_t kJoinFastCols = 16u * kWave * 8u;   // widest seam a 16-wave workgroup holds at eight columns a lane
 constexpr uint32_t kDefaultMaxBlocks = kCus * 6u;  // generic kernels: 6 workgroups per CU
 
 // One workgroup: reduce the per-workgroup candidates, publish the token.
@@ -76,22 +77,30 @@ hipError_t launch_one(const GemvParams &p, const GemvPlan &plan, size_t lds, hip
 #define NV_GEMV_LAUNCH(BB, EX, W, XR, RT)                                                                      \
   hipLaunchKernelGGL((gemv_fast_kernel<DT, PRO, EPI, NR, BB, EX, W, XR, RT>), dim3((waves + W - 1) / W),        \
                      dim3(W * kWave), lds, stream, p)
-    if (plan.rotated) {
+    if constexpr (PRO == kProJoin) {   // one 16-wave workgroup a CU (the plan)
+      if (wg != 16 || p.cols > kJoinFastCols) return hipErrorInvalidValue;
+      if constexpr (EPI == kEpiArgmax) {
+        if (plan.rotated) NV_GEMV_LAUNCH(1, false, 16, false, true);
+        else NV_GEMV_LAUNCH(2, false, 16, false, false);
+      } else if constexpr (EPI == kEpiMinGru) {   // three rows at a time
+        if (plan.rotated) NV_GEMV_LAUNCH(1, false, 16, false, true);
+        else NV_GEMV_LAUNCH(1, false, 16, false, false);
+      } else {
+        if (plan.rotated) NV_GEMV_LAUNCH(2, false, 16, false, true);
+        else NV_GEMV_LAUNCH(2, false, 16, false, false);
+      }
+    } else if (plan.rotated) {
       // (which launches walk rotated, and with how many chunks a batch, is the plan's choice)
       if constexpr (EPI == kEpiSwiglu) {
         if (wg == 16) NV_GEMV_LAUNCH(2, false, 16, false, true);
         else NV_GEMV_LAUNCH(2, false, 4, false, true);
-      } else if constexpr (PRO != kProX16 && EPI == kEpiArgmax) {
+      } else if constexpr (PRO == kProRmsNorm && EPI == kEpiArgmax) {
         NV_GEMV_LAUNCH(1, false, 16, false, true);
       } else if constexpr (PRO == kProRmsNorm && EPI == kEpiF32) {
         NV_GEMV_LAUNCH(2, false, 4, false, true);
       } else {
         return hipErrorInvalidValue;
       }
-    } else if constexpr (EPI == kEpiMinGru) {
-      // three rows an output, two chunks of each a batch
-      if (wg == 16) NV_GEMV_LAUNCH(2, false, 16, false, false);
-      else NV_GEMV_LAUNCH(2, false, 4, false, false);
     } else if (plan.chunks == 2 && NR == 1) {
       // rows that are whole batches of 1024 columns but not of 2048 (hidden 5120, MLP width 25600): two chunks a batch
       if (wg == 16) NV_GEMV_LAUNCH(2, false, 16, false, false);
@@ -161,8 +170,10 @@ bool aligned16(const void *ptr) { return (reinterpret_cast<uintptr_t>(ptr) & 15u
 // launches measured the same (qkv, o, down: within 0.1 us) or worse (gate_up 32.8 -> 34.6 us: one workgroup of
 // 16 waves per CU instead of five of 4) with 16.
 int fast_workgroup_waves(int prologue, int epilogue, uint32_t rows, uint32_t cols) {
-  if (prologue == kProJoin && cols > kWavesPerBlock * kWave * 16u) return 16;   // the seam's row in the lanes' registers
-  return prologue != kProX16 && epilogue == kEpiArgmax && rows >= 65536u ? 16 : kWavesPerBlock;
+  // The seam's prologue reads two f32 rows and four norm vectors (64 KiB at 4096 columns) in every workgroup: one
+  // workgroup of 16 waves a CU, looping over its rows.
+  if (prologue == kProJoin) return 16;
+  return prologue == kProRmsNorm && epilogue == kEpiArgmax && rows >= 65536u ? 16 : kWavesPerBlock;
 }
 
 }  // namespace
@@ -175,7 +186,7 @@ GemvPlan gemv_plan(int prologue, int epilogue, uint32_t rows, uint32_t cols, boo
   plan.mode = !vec ? kScalar : (cols % (kWave * 8) == 0 ? kVecFull : kVecGuarded);
   const uint32_t fast_cols = kWave * 8 * 2;
   const uint32_t max_cols = prologue == kProX16 ? kFastMaxColsLoop : kFastMaxCols;
-  if (plan.mode == kVecFull && cols % fast_cols == 0 && cols <= max_cols && !(tuning && tuning->force_generic))
+  if (plan.mode == kVecFull && cols % fast_cols == 0 && cols <= (prologue == kProJoin ? kJoinFastCols : max_cols) && !(tuning && tuning->force_generic))
     plan.mode = kFast;
   // one wave per unit (a row, or a gate/up pair)
   const uint32_t want = (rows + kWavesPerBlock - 1) / kWavesPerBlock;
@@ -187,7 +198,9 @@ GemvPlan gemv_plan(int prologue, int epilogue, uint32_t rows, uint32_t cols, boo
     const uint32_t by_lds = (160u * 1024u) / (cols * 2u + 1024u);
     const uint32_t resident =
         kCus * std::min<uint32_t>(static_cast<uint32_t>(fast_waves_per_simd(prologue)), std::max(by_lds, 1u));
-    if (want <= resident) {
+    if (prologue == kProJoin) {
+      blocks = std::min(want, kCus * 4u);  // (four-wave units: 256 workgroups of 16 waves)
+    } else if (want <= resident) {
       blocks = want;                       // everything is on the machine at once, one unit per wave
     } else if (want <= 2 * resident) {
       blocks = (want + 1) / 2;             // exactly two units per wave, pipelined in one round
@@ -204,14 +217,17 @@ GemvPlan gemv_plan(int prologue, int epilogue, uint32_t rows, uint32_t cols, boo
   plan.chunks = epilogue == kEpiSwiglu ? 2 : 4;
   if (plan.mode == kFast) {
     plan.wg_waves = nv::tuning(kTuneGemvWorkgroupWaves);
-    if (plan.wg_waves != 4 && plan.wg_waves != 16) plan.wg_waves = fast_workgroup_waves(prologue, epilogue, rows, cols);
+    if ((plan.wg_waves != 4 && plan.wg_waves != 16) || prologue == kProJoin) plan.wg_waves = fast_workgroup_waves(prologue, epilogue, rows, cols);
     if (epilogue != kEpiSwiglu && cols % (kWave * 8 * 4) != 0) plan.chunks = 2;
     // The rotated walk (see the kernel), where it measured faster; "gemv_rotated_walk" = 2 keeps the plain walk.
     const bool auto_grid = !(tuning && tuning->max_blocks > 0);
     if (nv::tuning(kTuneGemvRotatedWalk) != 2) {
-      if (epilogue == kEpiSwiglu) {
+      if (prologue == kProJoin) {
+        plan.rotated = true;                                  // 2 KiB of each row a batch, the head's 1 KiB
+        plan.chunks = epilogue == kEpiArgmax || epilogue == kEpiMinGru ? 1 : 2;
+      } else if (epilogue == kEpiSwiglu) {
         plan.rotated = true;                                  // gate/up pair: 2 KiB of each row a batch
-      } else if (prologue != kProX16 && epilogue == kEpiArgmax && plan.wg_waves == 16 && plan.chunks == 4) {
+      } else if (prologue == kProRmsNorm && epilogue == kEpiArgmax && plan.wg_waves == 16 && plan.chunks == 4) {
         plan.rotated = true;                                  // LM head: 1 KiB a batch
         plan.chunks = 1;
       } else if (prologue == kProRmsNorm && epilogue == kEpiF32 && plan.wg_waves == 4 && cols == 4096u && auto_grid &&

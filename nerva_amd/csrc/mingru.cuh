@@ -1,8 +1,8 @@
 // minGRU over a block of token rows: the gates of every token are known before the recurrence starts (they read the
 // token alone), so S_t = (1 - z_t) S_{t-1} + z_t c_t is a first-order linear recurrence that a block of tokens
-// evaluates in pieces: every wave of a workgroup takes a run of consecutive tokens for 64 channels and reduces it to
-// (product of 1 - z, result from a zero state); the runs' results chain through LDS; then each wave walks its run again
-// from the state it now knows and writes the gated outputs. A decode step has the recurrence in the epilogue of its
+// evaluates in pieces: half a wave takes a run of consecutive tokens for 32 channels and reduces it to (product of 1 - z,
+// result from a zero state); the runs' results chain through LDS; then each walks its run again - from registers, for
+// blocks of up to 512 tokens - from the state it now knows and writes the gated outputs. A decode step has the recurrence in the epilogue of its
 // projection (gemv_stream.cuh) instead.
 #pragma once
 

@@ -138,8 +138,8 @@ __device__ __forceinline__ void join_norm_row(const JoinNorm &j, uint32_t cols, 
     for (uint32_t c = threadIdx.x; c < cols; c += TB) j.x_out[c] = joined(c);
 }
 
-// Eight consecutive columns of everything the seam reads, requested at once (the lean GEMV holds two of these per
-// lane across its first weight requests).
+// Eight consecutive columns of everything the seam reads, requested at once (the lean GEMV holds them across its first
+// weight requests).
 struct JoinRegs {
   float4 xa, xb, ya, yb;
   uint4 post_w, post_b, pre_w, pre_b;
@@ -164,18 +164,18 @@ __device__ __forceinline__ void unpack8(const uint4 &w, float (&o)[8]) {
   unpack2<DT>(w.z, o[4], o[5]);
   unpack2<DT>(w.w, o[6], o[7]);
 }
-// cols % 8 == 0, cols <= WG * 64 * 16: h into LDS as 16-bit values, x' to memory where `store`.
-template <uint32_t DT, int WG>
-__device__ __forceinline__ void join_norm_regs(const JoinNorm &j, uint32_t cols, bool store, const JoinRegs (&r)[2], float *scratch,
+// cols % 8 == 0, cols <= WG * 64 * 8 * N: h into LDS as 16-bit values, x' to memory where `store`.
+template <uint32_t DT, int WG, int N>
+__device__ __forceinline__ void join_norm_regs(const JoinNorm &j, uint32_t cols, bool store, const JoinRegs (&r)[N], float *scratch,
                                                uint16_t *xs) {
   constexpr uint32_t TB = WG * kWave;
   const auto at = [&](int i) { return (static_cast<uint32_t>(i) * TB + threadIdx.x) * 8u; };
   const auto in = [&](int i) { return at(i / 8) < cols; };
-  float v[16];
+  float v[8 * N];
   float mean, rstd;
   if (j.y != nullptr) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < N; ++i) {
       const bool on = at(i) < cols;
       const float t[8] = {r[i].ya.x, r[i].ya.y, r[i].ya.z, r[i].ya.w, r[i].yb.x, r[i].yb.y, r[i].yb.z, r[i].yb.w};
 #pragma unroll
@@ -183,7 +183,7 @@ __device__ __forceinline__ void join_norm_regs(const JoinNorm &j, uint32_t cols,
     }
     row_moments<WG>(v, in, cols, j.eps, scratch, mean, rstd);
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < N; ++i) {
       const bool on = at(i) < cols;
       float w[8], b[8];
       unpack8<DT>(r[i].post_w, w);
@@ -194,7 +194,7 @@ __device__ __forceinline__ void join_norm_regs(const JoinNorm &j, uint32_t cols,
     }
   } else {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < N; ++i) {
       const bool on = at(i) < cols;
       const float t[8] = {r[i].xa.x, r[i].xa.y, r[i].xa.z, r[i].xa.w, r[i].xb.x, r[i].xb.y, r[i].xb.z, r[i].xb.w};
 #pragma unroll
@@ -203,7 +203,7 @@ __device__ __forceinline__ void join_norm_regs(const JoinNorm &j, uint32_t cols,
   }
   if (store && j.x_out != nullptr) {
 #pragma unroll
-    for (int i = 0; i < 2; ++i) {
+    for (int i = 0; i < N; ++i) {
       if (at(i) < cols) {
         *reinterpret_cast<float4 *>(j.x_out + at(i)) = make_float4(v[8 * i], v[8 * i + 1], v[8 * i + 2], v[8 * i + 3]);
         *reinterpret_cast<float4 *>(j.x_out + at(i) + 4) = make_float4(v[8 * i + 4], v[8 * i + 5], v[8 * i + 6], v[8 * i + 7]);
@@ -212,7 +212,7 @@ __device__ __forceinline__ void join_norm_regs(const JoinNorm &j, uint32_t cols,
   }
   row_moments<WG>(v, in, cols, j.eps, scratch, mean, rstd);
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
+  for (int i = 0; i < N; ++i) {
     if (at(i) < cols) {
       float w[8], b[8];
       unpack8<DT>(r[i].pre_w, w);

@@ -48,7 +48,7 @@ __global__ __launch_bounds__(WG *kWave) void join_rows_vec_kernel(JoinRows p) {
   JoinRegs r[2];
 #pragma unroll
   for (int i = 0; i < 2; ++i) join_load8(j, (static_cast<uint32_t>(i) * TB + threadIdx.x) * 8u, cols, r[i]);
-  join_norm_regs<DT, WG>(j, cols, true, r, red, h);
+  join_norm_regs<DT, WG, 2>(j, cols, true, r, red, h);
   // (every lane reads back the pieces it wrote itself)
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
