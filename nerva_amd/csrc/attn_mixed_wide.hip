@@ -185,7 +185,8 @@ __global__ __launch_bounds__(512, 2) void mixed_decode_kernel(MixedAttnParams p,
     float mixed[R];
 #pragma unroll
     for (int r = 0; r < R; ++r) mixed[r] = 0.0f;
-    for (uint32_t g = 0; g < H; ++g) {
+#pragma unroll 8
+    for (uint32_t g = 0; g < H; ++g) {   // (16 or 32 heads)
       const float s = s_s[g * kKeysPitch + lane];
 #pragma unroll
       for (int r = 0; r < R; ++r) mixed[r] = fmaf(t_s[g * H + c * R + r], s, mixed[r]);
@@ -475,7 +476,12 @@ __global__ __launch_bounds__(kMergeGroups * 32) void mixed_decode_merge_kernel(M
   const uint32_t active = decode_range(p, pos, splits).active;
   const Partials in = partials_of(p.workspace, static_cast<uint64_t>(splits) * H);
   const float sink = p.sink != nullptr ? dec16<kBF16>(p.sink[h]) * kLog2e : -INFINITY;
-  // one split a lane (kDecodeSplits lanes are enough)
+  // every request first: the lane's share of the sums, and one split's maximum and denominator (kDecodeSplits lanes
+  // are enough)
+  float4 v[kDecodeSplits / kMergeGroups];
+#pragma unroll
+  for (uint32_t i = 0; i < kDecodeSplits / kMergeGroups; ++i)
+    v[i] = *reinterpret_cast<const float4 *>(in.sum + (static_cast<uint64_t>(min(group + i * kMergeGroups, active - 1)) * H + h) * kHD + c4 * 4u);
   const float ms = tid < active ? in.m[tid * H + h] : -INFINITY, ls = tid < active ? in.l[tid * H + h] : 0.0f;
   float top = wave_max(ms);
   if (tid % kWave == 0) red[tid / kWave] = top;
@@ -493,25 +499,24 @@ __global__ __launch_bounds__(kMergeGroups * 32) void mixed_decode_merge_kernel(M
 #pragma unroll
   for (uint32_t w = 0; w < kMergeGroups * 32 / kWave; ++w) total += red[w];
   float4 o = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
-#pragma unroll 8
-  for (uint32_t s = group; s < active; s += kMergeGroups) {
-    const float4 v = *reinterpret_cast<const float4 *>(in.sum + (static_cast<uint64_t>(s) * H + h) * kHD + c4 * 4u);
-    const float w = f_s[s];
-    o.x = fmaf(v.x, w, o.x);
-    o.y = fmaf(v.y, w, o.y);
-    o.z = fmaf(v.z, w, o.z);
-    o.w = fmaf(v.w, w, o.w);
+#pragma unroll
+  for (uint32_t i = 0; i < kDecodeSplits / kMergeGroups; ++i) {
+    const float w = f_s[group + i * kMergeGroups];   // zero past the active splits
+    o.x = fmaf(v[i].x, w, o.x);
+    o.y = fmaf(v[i].y, w, o.y);
+    o.z = fmaf(v[i].z, w, o.z);
+    o.w = fmaf(v[i].w, w, o.w);
   }
   sum_s[group][c4] = o;
   __syncthreads();
   if (group != 0) return;
 #pragma unroll
   for (uint32_t i = 1; i < kMergeGroups; ++i) {
-    const float4 v = sum_s[i][c4];
-    o.x += v.x;
-    o.y += v.y;
-    o.z += v.z;
-    o.w += v.w;
+    const float4 a = sum_s[i][c4];
+    o.x += a.x;
+    o.y += a.y;
+    o.z += a.z;
+    o.w += a.w;
   }
   const float inv = 1.0f / total;
   merged_store(p, 0, h * kHD + c4 * 4u, make_float4(o.x * inv, o.y * inv, o.z * inv, o.w * inv));

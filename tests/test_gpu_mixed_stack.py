@@ -387,3 +387,18 @@ def test_trace_replay_from_a_folder(tmp_path, dtype):
             if places:
                 got = np.fromfile(path, "<f4").reshape(len(places), cfg["vocab"])
                 assert M.errors(got, want[name][[first + w for w in places]]).max() < (EXACT if dtype == "float32" else HALF)
+
+
+def test_generation_from_a_folder(tmp_path):
+    """bin/generate over a folder gives the tokens of a session over the same weights in memory."""
+    cfg = M.config([M.attention(), M.mingru()])
+    tensors, prompt = M.weights(cfg, seed=21), tokens_of(cfg, 9)
+    M.write_folder(str(tmp_path), cfg, tensors)
+    s = M.session(cfg, tensors, 32, 1)
+    rc, _ = s.start(prompt)
+    rc, _, tokens = s.advance(12)
+    s.destroy()
+    run = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "generate"), "--model", str(tmp_path), "--dtype", "float32", "--steps", "12",
+                          "--prompt", ",".join(str(t) for t in prompt)], capture_output=True, text=True, timeout=100)
+    assert run.returncode == 0, run.stderr[-2000:]
+    assert run.stdout.strip() == ",".join(str(t) for t in tokens)
