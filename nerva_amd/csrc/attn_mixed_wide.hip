@@ -30,7 +30,7 @@ namespace {
 
 using namespace attn;
 
-constexpr uint32_t kDecodeSplits = 256, kMinBlocksPerSplit = 2;
+constexpr uint32_t kDecodeSplits = 256, kMinBlocksPerSplit = 4;
 constexpr uint32_t kPromptTokens = 8;          // tokens of a workgroup
 constexpr uint32_t kPromptWorkgroups = 256;    // split the keys until about so many are there
 constexpr uint32_t kPromptSplits = 64;

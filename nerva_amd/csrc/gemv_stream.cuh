@@ -517,7 +517,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   const uint16_t *wp[NR];
   uint4 buf0[NR][B], buf1[NR][B];
   float res0 = 0.0f, res1 = 0.0f;     // residual element (recurrent state) requested with a row's first batch
-  float zb0 = 0.0f, zb1 = 0.0f, ub0 = 0.0f, ub1 = 0.0f;   // kEpiMinGru: the row's two biases, likewise
+  uint16_t zb0 = 0, zb1 = 0, ub0 = 0, ub1 = 0;   // kEpiMinGru: the row's two biases, likewise (widened where they are used:
+                                                // here that would wait for them ahead of the weight requests)
 #define NV_FAST_ISSUE(DST, RES, ZB, UB)                                                                 \
   do {                                                                                            \
     if (ib == 0) {                                                                                \
@@ -529,8 +530,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
       }                                                                                           \
       if constexpr (EPI == kEpiMinGru) {                                                          \
         RES = p.state[iu];                                                                        \
-        ZB = dec16<DT>(p.bias[iu]);                                                               \
-        UB = dec16<DT>(p.bias2[iu]);                                                              \
+        ZB = p.bias[iu];                                                                          \
+        UB = p.bias2[iu];                                                                         \
       }                                                                                           \
     }                                                                                             \
     _Pragma("unroll") for (int u = 0; u < B; ++u)                                                 \
@@ -633,7 +634,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
   Best best{0.0f, 0u, 0u};
   uint32_t cu = wave_global, cb = 0;  // batch being consumed: unit, batch within the row
   float acc[NR];
-  float res_cur = 0.0f, zb_cur = 0.0f, ub_cur = 0.0f;
+  float res_cur = 0.0f;
+  uint16_t zb_cur = 0, ub_cur = 0;
   XieluParams act{};
   if constexpr (EPI == kEpiXielu) act = xielu_params<DT>(p.act);
 #define NV_FAST_CONSUME(SRC, RES, ZB, UB)                                                               \
@@ -667,7 +669,8 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) voi
           }                                                                                       \
           p.out16[cu] = enc16<DT>(silu(g) * u);                                                   \
         } else if constexpr (EPI == kEpiMinGru) {                                                 \
-          const float next = mingru_step(acc[0] + zb_cur, acc[NR > 1 ? 1 : 0] + ub_cur, res_cur); \
+          const float next =                                                                      \
+              mingru_step(acc[0] + dec16<DT>(zb_cur), acc[NR > 1 ? 1 : 0] + dec16<DT>(ub_cur), res_cur); \
           p.state[cu] = next;                                                                     \
           p.out16[cu] = enc16<DT>(next * silu(acc[NR - 1]));                                      \
         } else {                                                                                  \

@@ -857,6 +857,45 @@ def test_block_prefill_edge_lengths_match_token_walk(length, monkeypatch):
     assert tb[0] == tw[0] or top[-1] - top[-2] < E2E_REL_L2 * np.max(np.abs(lw))
 
 
+@pytest.mark.parametrize("geom", [GEOMETRIES[0], GEOMETRIES[5]], ids=["token walk", "blocks"])
+def test_extend_appends_given_tokens_to_a_running_sequence(geom):
+    """extend() in portions of several sizes leaves the cache, the logits at the places asked for and the next token as
+    start() over the whole prompt does; a session without a sequence begins one, and a released one starts anew."""
+    dtype, hidden, heads, kv, hd, inter, vocab, layers, theta, qk_norm, bias = geom
+    weights, _ = random_model(dtype, hidden, heads, kv, hd, inter, vocab, layers, 31, theta, qk_norm, bias)
+    prompt = np.random.default_rng(4).integers(0, vocab, 150).astype(np.uint32)
+    solo, s = N.DecodeSession.create(weights, 160), N.DecodeSession.create(weights, 160)
+    want = {}
+    for place in (0, 39, 40, 42, 100, 149):
+        rc, _ = solo.start(prompt[:place + 1])
+        assert rc == 0
+        want[place] = solo.logits()
+    rc, _, tokens = solo.advance(4)
+    assert rc == 0
+    rows = [solo.kv_row(layers - 1, t) for t in (0, 40, 41, 99, 148)]
+    for _ in range(2):
+        at = 0
+        for size in (40, 1, 2, 90, 17):
+            places = [p - at for p in want if at <= p < at + size]
+            rc, res, logits, _ = s.extend(prompt[at:at + size], places)
+            assert rc == 0 and res.kv_tokens == at + size
+            for p, row in zip(places, logits):
+                assert rel_l2(row, want[at + p]) <= E2E_REL_L2, at + p
+            at += size
+        for token, (k, v) in zip((0, 40, 41, 99, 148), rows):
+            gk, gv = s.kv_row(layers - 1, token)
+            assert rel_l2(O.decode16(dtype, gk), O.decode16(dtype, k)) <= E2E_REL_L2
+            assert rel_l2(O.decode16(dtype, gv), O.decode16(dtype, v)) <= E2E_REL_L2
+        rc, _, out = s.advance(4)
+        assert rc == 0
+        top = np.sort(want[149])
+        assert out[0] == tokens[0] or top[-1] - top[-2] < E2E_REL_L2 * np.max(np.abs(want[149]))
+        assert s.release_sequence() == 0
+    assert s.extend(prompt[:3], (), residual_layers=layers)[0] == -1   # residual rows are a mixed stack's
+    solo.destroy()
+    s.destroy()
+
+
 def test_prefill_block_size_changes_only_the_block_boundaries():
     """A session whose four projections have the kernels for them prefills 512 tokens at a time (256 where only the
     kernel for those blocks takes its widths); the hook "prefill_block_tokens" = 256 or 128 keeps the smaller
