@@ -426,7 +426,8 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
 // Register budget as resident waves per SIMD (= workgroups per CU): 6 with a 16-bit input,
 // 5 with the RMSNorm prologue, which holds the f32 activations and the norm weights in
 // registers across the first weight requests (a budget of 6 makes it spill), 4 with the join
-// prologue, which holds two f32 rows and the weights and biases of two norms: one 16-wave workgroup a CU.
+// prologue, which holds two f32 rows and the weights and biases of two norms: one 16-wave workgroup a CU, or an
+// 8-wave one with twice the registers.
 constexpr int fast_waves_per_simd(int prologue) { return prologue == kProJoin ? 4 : prologue == kProRmsNorm ? 5 : 6; }
 constexpr int kFastMaxCols = 12288;  // x staged through at most 6 x 16 B per lane in registers ...
 constexpr int kFastMaxColsLoop = 30720;  // ... or, with a 16-bit input, copied into LDS behind the first weight requests
@@ -436,7 +437,7 @@ constexpr int kFastMaxColsLoop = 30720;  // ... or, with a 16-bit input, copied 
 // without a row asks for the last row's data and drops it - so that the compiler can count the requests
 // behind the activation loads and waits for exactly those before the prologue, which then runs under
 // the weights' latency. With the requests under `if (total > n)` it waits for everything.
-// WG: waves per workgroup (4 or 16). Every workgroup fetches the whole input vector (and for the RMSNorm
+// WG: waves per workgroup (4 or 16; 8 with the join prologue). Every workgroup fetches the whole input vector (and for the RMSNorm
 // prologue the norm weights) for itself, so fewer, larger workgroups move that much less through the L2s ahead of
 // the weights; the waves' work is the same whatever the size (wave_global = workgroup x WG + wave).
 // ROT: a unit's walk over its columns starts at batch (unit mod batches per row) and wraps, so the waves of a
@@ -455,7 +456,7 @@ constexpr int kFastMaxColsLoop = 30720;  // ... or, with a 16-bit input, copied 
 // one wave per SIMD less.
 template <uint32_t DT, int PRO, int EPI, int NR, int B, bool EXACT = false, int WG = kWavesPerBlock, bool XREG = false,
           bool ROT = false>
-__global__ __launch_bounds__(WG *kWave, XREG ? 4 : fast_waves_per_simd(PRO)) void gemv_fast_kernel(GemvParams p) {
+__global__ __launch_bounds__(WG *kWave, XREG ? 4 : PRO == kProJoin && WG == 8 ? 2 : fast_waves_per_simd(PRO)) void gemv_fast_kernel(GemvParams p) {
   static_assert(!(ROT && (XREG || EXACT)), "the rotated walk has no exact-start or register-input variant");
   constexpr int TB = WG * kWave;
   constexpr uint32_t kXregBpr = 8 / B;   // batches per 4096-column row
@@ -763,7 +764,7 @@ hipError_t launch_gemv(uint32_t dtype, int prologue, int epilogue, const GemvPar
 struct GemvPlan {
   int mode;         // kScalar / kVecGuarded / kVecFull / kFast
   uint32_t blocks;  // four-wave workgroups' worth of waves
-  int wg_waves;     // waves per workgroup the launch uses (kFast: 4 or 16)
+  int wg_waves;     // waves per workgroup the launch uses (kFast: 4, 8 or 16)
   uint32_t grid;    // workgroups launched: ceil(blocks * 4 / wg_waves)
   bool rotated;     // kFast: the rotated walk (see gemv_fast_kernel)
   int chunks;       // kFast: 1 KiB chunks per row and request batch

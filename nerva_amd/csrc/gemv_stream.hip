@@ -77,9 +77,18 @@ hipError_t launch_one(const GemvParams &p, const GemvPlan &plan, size_t lds, hip
 #define NV_GEMV_LAUNCH(BB, EX, W, XR, RT)                                                                      \
   hipLaunchKernelGGL((gemv_fast_kernel<DT, PRO, EPI, NR, BB, EX, W, XR, RT>), dim3((waves + W - 1) / W),        \
                      dim3(W * kWave), lds, stream, p)
-    if constexpr (PRO == kProJoin) {   // one 16-wave workgroup a CU (the plan)
-      if (wg != 16 || p.cols > kJoinFastCols) return hipErrorInvalidValue;
-      if constexpr (EPI == kEpiArgmax) {
+    if constexpr (PRO == kProJoin) {   // one workgroup a CU (the plan)
+      if ((wg != 16 && wg != 8) || p.cols > static_cast<uint32_t>(wg) * kWave * 8u) return hipErrorInvalidValue;
+      if (wg == 8) {
+        if constexpr (EPI == kEpiArgmax) {
+          return hipErrorInvalidValue;
+        } else if constexpr (EPI == kEpiMinGru) {
+          NV_GEMV_LAUNCH(2, false, 8, false, true);
+        } else {
+          if (plan.chunks == 4) NV_GEMV_LAUNCH(4, false, 8, false, true);
+          else NV_GEMV_LAUNCH(2, false, 8, false, true);
+        }
+      } else if constexpr (EPI == kEpiArgmax) {
         if (plan.rotated) NV_GEMV_LAUNCH(1, false, 16, false, true);
         else NV_GEMV_LAUNCH(2, false, 16, false, false);
       } else if constexpr (EPI == kEpiMinGru) {   // three rows at a time
@@ -164,15 +173,21 @@ hipError_t launch_pro(int prologue, int epilogue, const GemvParams &p, const Gem
 
 bool aligned16(const void *ptr) { return (reinterpret_cast<uintptr_t>(ptr) & 15u) == 0; }
 
-// Waves per workgroup the lean kernel is launched with (4 or 16), per shape. Every workgroup fetches the input
+// Waves per workgroup the lean kernel is launched with, per shape. Every workgroup fetches the input
 // vector and the norm weights for itself (24 KiB at 4096 columns); the LM head's 2048 looping workgroups move
 // 49 MB of that ahead of their weights, as 512 workgroups of 16 waves 12 MB: 197 -> 190 us. The step's other
 // launches measured the same (qkv, o, down: within 0.1 us) or worse (gate_up 32.8 -> 34.6 us: one workgroup of
 // 16 waves per CU instead of five of 4) with 16.
 int fast_workgroup_waves(int prologue, int epilogue, uint32_t rows, uint32_t cols) {
-  // The seam's prologue reads two f32 rows and four norm vectors (64 KiB at 4096 columns) in every workgroup: one
-  // workgroup of 16 waves a CU, looping over its rows.
-  if (prologue == kProJoin) return 16;
+  // The seam's prologue reads two f32 rows and four norm vectors (64 KiB at 4096 columns) in every workgroup, so it
+  // runs in one workgroup a CU that loops over its rows: of eight waves where eight columns a lane cover the row - their
+  // register budget takes whole 2048-column batches - else of sixteen. Measured against sixteen everywhere, decode step
+  // of 12 layers: 1.060 -> 1.040 ms at width 4096, 0.530 -> 0.507 at 2048 (four waves, 64 KiB in each of up to 3072
+  // workgroups: 1.56 and 0.95). The eight-wave kernels walk rotated only.
+  if (prologue == kProJoin)
+    return cols <= 8u * kWave * 8u && epilogue != kEpiArgmax && tuning(kTuneGemvWorkgroupWaves) != 16 && tuning(kTuneGemvRotatedWalk) != 2
+               ? 8
+               : 16;
   return prologue == kProRmsNorm && epilogue == kEpiArgmax && rows >= 65536u ? 16 : kWavesPerBlock;
 }
 
@@ -199,7 +214,8 @@ GemvPlan gemv_plan(int prologue, int epilogue, uint32_t rows, uint32_t cols, boo
     const uint32_t resident =
         kCus * std::min<uint32_t>(static_cast<uint32_t>(fast_waves_per_simd(prologue)), std::max(by_lds, 1u));
     if (prologue == kProJoin) {
-      blocks = std::min(want, kCus * 4u);  // (four-wave units: 256 workgroups of 16 waves)
+      // (in units of four waves)
+      blocks = std::min(want, kCus * static_cast<uint32_t>(fast_workgroup_waves(prologue, epilogue, rows, cols)) / 4u);
     } else if (want <= resident) {
       blocks = want;                       // everything is on the machine at once, one unit per wave
     } else if (want <= 2 * resident) {
@@ -224,7 +240,7 @@ GemvPlan gemv_plan(int prologue, int epilogue, uint32_t rows, uint32_t cols, boo
     if (nv::tuning(kTuneGemvRotatedWalk) != 2) {
       if (prologue == kProJoin) {
         plan.rotated = true;                                  // 2 KiB of each row a batch, the head's 1 KiB
-        plan.chunks = epilogue == kEpiArgmax || epilogue == kEpiMinGru ? 1 : 2;
+        plan.chunks = plan.wg_waves == 8 && cols % 2048u == 0 ? 4 : epilogue == kEpiArgmax || epilogue == kEpiMinGru ? 1 : 2;
       } else if (epilogue == kEpiSwiglu) {
         plan.rotated = true;                                  // gate/up pair: 2 KiB of each row a batch
       } else if (prologue == kProRmsNorm && epilogue == kEpiArgmax && plan.wg_waves == 16 && plan.chunks == 4) {
