@@ -47,6 +47,13 @@ struct MixedAttnParams {
   uint32_t last_block;         // highest logical block a launch may meet (sizes the split grid of a captured step)
 };
 
+// Element d of a head after rotation; cs = cos | sin of the row's angles.
+__device__ __forceinline__ float rotated_elem(const float *head, const float *cs, uint32_t rot_dims, uint32_t d) {
+  if (d >= rot_dims) return head[d];
+  const uint32_t half = rot_dims / 2;
+  return d < half ? head[d] * cs[d] - head[d + half] * cs[half + d] : head[d] * cs[d - half] + head[d - half] * cs[d];
+}
+
 // Rotates the token rows' keys and writes keys and values to the cache.
 hipError_t launch_mixed_publish(uint32_t dtype, const MixedAttnParams &p, hipStream_t stream);
 // Attention of the token rows, whose own keys and values are in the cache. Any shape.

@@ -18,13 +18,6 @@ __device__ __forceinline__ float cache_load(const void *base, uint64_t at) {
   if constexpr (F32) return static_cast<const float *>(base)[at];
   else return dec16<DT>(static_cast<const uint16_t *>(base)[at]);
 }
-// Element d of a head after rotation; cs = cos | sin of the row's angles.
-__device__ __forceinline__ float rotated(const float *head, const float *cs, uint32_t rot_dims, uint32_t d) {
-  if (d >= rot_dims) return head[d];
-  const uint32_t half = rot_dims / 2;
-  return d < half ? head[d] * cs[d] - head[d + half] * cs[half + d] : head[d] * cs[d - half] + head[d - half] * cs[d];
-}
-
 template <uint32_t DT, bool F32>
 __global__ __launch_bounds__(kBlock) void mixed_publish_kernel(MixedAttnParams p) {
   const uint32_t t = blockIdx.x;
@@ -37,7 +30,7 @@ __global__ __launch_bounds__(kBlock) void mixed_publish_kernel(MixedAttnParams p
   for (uint32_t i = threadIdx.x; i < nk; i += kBlock) {
     const uint32_t h = i / p.key_dim, d = i % p.key_dim;
     cache_store<DT, F32>(p.k_cache, kv_tile_offset(0, p.kv_heads, p.key_dim, 0, block, h) + kv_k_elem(p.key_dim, row, d),
-                         rotated(src + p.k_col + h * p.key_dim, cs, p.rot_dims, d));
+                         rotated_elem(src + p.k_col + h * p.key_dim, cs, p.rot_dims, d));
   }
   for (uint32_t i = threadIdx.x; i < nv_; i += kBlock) {
     const uint32_t h = i / p.value_dim, d = i % p.value_dim;
@@ -66,7 +59,7 @@ __global__ __launch_bounds__(kBlock) void mixed_attention_kernel(MixedAttnParams
     for (uint32_t r = 0; r < group; ++r) {
       const uint32_t g = c * group + r;
       const float m = p.talk != nullptr ? dec16<DT>(p.talk[h * p.heads + g]) : (g == h ? 1.0f : 0.0f);
-      sum = fmaf(m, rotated(src + p.q_col + g * D, cs, p.rot_dims, d), sum);
+      sum = fmaf(m, rotated_elem(src + p.q_col + g * D, cs, p.rot_dims, d), sum);
     }
     q_s[i] = sum * p.scale;
   }

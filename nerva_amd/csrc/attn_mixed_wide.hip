@@ -69,12 +69,6 @@ __device__ __forceinline__ Range prompt_range(const MixedAttnParams &p, uint32_t
   return split_range(b0, ((p.position + t1) / kKvBlockTokens - b0) / 2 + 1, splits, 1);
 }
 
-__device__ __forceinline__ float rotated_elem(const float *head, const float *cs, uint32_t rot_dims, uint32_t d) {
-  if (d >= rot_dims) return head[d];
-  const uint32_t half = rot_dims / 2;
-  return d < half ? head[d] * cs[d] - head[d + half] * cs[half + d] : head[d] * cs[d - half] + head[d - half] * cs[d];
-}
-
 __device__ __forceinline__ uint32_t pack16(float a, float b) {
   return enc16_finite<kBF16>(a) | (static_cast<uint32_t>(enc16_finite<kBF16>(b)) << 16);
 }

@@ -151,14 +151,14 @@ hipError_t launch_epi(int epilogue, const GemvParams &p, const GemvPlan &plan, s
       default: return hipErrorInvalidValue;
     }
   } else {
-  switch (epilogue) {
-    case kEpiF32: return launch_one<DT, PRO, kEpiF32, MODE>(p, plan, lds, stream);
-    case kEpiResidual: return launch_one<DT, PRO, kEpiResidual, MODE>(p, plan, lds, stream);
-    case kEpiSwiglu: return launch_one<DT, PRO, kEpiSwiglu, MODE>(p, plan, lds, stream);
-    case kEpiOut16: return launch_one<DT, PRO, kEpiOut16, MODE>(p, plan, lds, stream);
-    case kEpiArgmax: return launch_one<DT, PRO, kEpiArgmax, MODE>(p, plan, lds, stream);
-    default: return hipErrorInvalidValue;
-  }
+    switch (epilogue) {
+      case kEpiF32: return launch_one<DT, PRO, kEpiF32, MODE>(p, plan, lds, stream);
+      case kEpiResidual: return launch_one<DT, PRO, kEpiResidual, MODE>(p, plan, lds, stream);
+      case kEpiSwiglu: return launch_one<DT, PRO, kEpiSwiglu, MODE>(p, plan, lds, stream);
+      case kEpiOut16: return launch_one<DT, PRO, kEpiOut16, MODE>(p, plan, lds, stream);
+      case kEpiArgmax: return launch_one<DT, PRO, kEpiArgmax, MODE>(p, plan, lds, stream);
+      default: return hipErrorInvalidValue;
+    }
   }
 }
 

@@ -504,10 +504,9 @@ uint32_t widest_chunk(const std::vector<StackLayer> &layers, size_t l) {
   return widest;
 }
 
-bool layer_valid(const NervaHipStackLayer *layers, uint32_t count, uint32_t l, uint32_t hidden) {
+bool layer_valid(const NervaHipStackLayer *layers, uint32_t count, uint32_t l) {
   const NervaHipStackLayer &d = layers[l];
   if (static_cast<uint64_t>(d.ff) * 2 > 60 * 1024) return false;
-  (void)hidden;
   if (d.mixer == NERVA_HIP_MIXER_MINGRU) return d.width != 0 && static_cast<uint64_t>(d.width) * 2 <= 60 * 1024;
   if (d.mixer != NERVA_HIP_MIXER_ATTENTION) return false;
   if (d.heads == 0 || d.kv_heads == 0 || d.heads % d.kv_heads != 0 || d.key_dim == 0 || d.value_dim == 0 || d.rotary_dims % 2 != 0 ||
@@ -533,7 +532,7 @@ bool create_checks(const NervaHipStackSessionCreateRequest *rq, bool synthetic, 
     return false;
   }
   for (uint32_t l = 0; l < rq->layer_count; ++l)
-    if (!layer_valid(rq->layers, rq->layer_count, l, rq->hidden)) return false;
+    if (!layer_valid(rq->layers, rq->layer_count, l)) return false;
   // the weights come through a complete plan
   return synthetic || (rq->planned_weight_blocks != 0 && rq->planned_weight_bytes != 0 && rq->planned_weight_descriptors != nullptr &&
                        rq->planned_weight_descriptor_count == rq->planned_weight_blocks && rq->planned_weight_descriptor_hash != 0);
