@@ -624,6 +624,16 @@ pub struct NervaHipStackLayer {
     pub kv_layer: u32,
     pub width: u32,
     pub ff: u32,
+    pub q_rank: u32,
+    pub kv_rank: u32,
+    pub rotary_key_dim: u32,
+    pub window_tokens: u32,
+    pub experts: u32,
+    pub experts_per_token: u32,
+    pub expert_ff: u32,
+    pub expert_limit: f32,
+    pub shared_ff: u32,
+    pub shared_limit: f32,
 }
 
 #[repr(C)]
@@ -636,6 +646,9 @@ pub struct NervaHipStackSessionCreateRequest {
     pub layer_count: u32,
     pub max_context_tokens: u32,
     pub norm_eps: f32,
+    pub arrangement: u32,
+    pub embedding_scale: f32,
+    pub logit_scale: f32,
     pub layers: *const NervaHipStackLayer,
     pub planned_weight_blocks: u32,
     pub planned_gpu_resident_blocks: u32,

@@ -449,42 +449,65 @@ int nerva_hip_deepseek_moe_forward(const NervaHipDeepSeekMoeForwardRequest *requ
  * that (start / advance / run / extend / fork / batch_advance_one / destroy, the sampler, the token slots) is the
  * session interface above.
  *
- * Every sublayer f sits between two layer norms (weight and bias): x <- x + N_post(f(N_pre(x))). A layer is a mixer,
- * then - where ff != 0 - a feed-forward down(xielu(up(.))). Mixers:
+ * A layer is a mixer and a feed-forward or none, in one of two arrangements:
+ *   SANDWICH  one after the other, each between two layer norms (weight and bias): x <- x + N_post(f(N_pre(x))). The
+ *             output is the final layer norm and the embedding matrix.
+ *   PARALLEL  both read the same row, each through an RMS norm of its own: x <- x + (mixer(N1(x)) + ff(N2(x))). The
+ *             output is the final RMS norm, a head matrix and logit_scale.
+ * Feed-forwards: dense, down(xielu(up(.))) (ff != 0), or routed experts (experts != 0, PARALLEL only): every token goes
+ * through the `experts_per_token` experts with the largest sigmoid(router(.)), weighted by these scores over their sum; an
+ * expert is down(g sigmoid(1.702 g) (u + 1)) with g = min(gate(.), limit), u = clamp(up(.), -limit, limit); where
+ * shared_ff != 0 an expert of that width takes every token besides. Mixers:
  *   ATTENTION  grouped-query attention; the heads' scores are mixed by a learned [heads][heads] matrix before the
  *              softmax; the softmax has a learned sink per head in its denominator; the heads are gated by
  *              sigmoid(gate(.)); rotation on the first rotary_dims of a head; with chunk_tokens != 0 a query sees its
  *              own chunk of positions only; kv_layer names another layer whose keys and values are used
  *              (NERVA_HIP_OWN_KEYS: its own).
  *   MINGRU     gated recurrence of `width` channels with an f32 state (csrc/activations.cuh), gated by silu(gate(.)).
- * The output is the final layer norm and the embedding matrix. Computed in f32 whatever the precision: norms, the
- * residual, rotation, scores and weights, recurrence.
+ *   LATENT     attention over normalised latents: queries from an RMS-normed latent of q_rank, unrotated keys (key_dim
+ *              per head) and values from one of kv_rank, one rotated key part of rotary_key_dim for all heads (rotation
+ *              on its first rotary_dims), which a head's query meets with its own last rotary_key_dim elements; with
+ *              window_tokens != 0 a query sees that many tokens, itself included; the heads are gated by
+ *              sigmoid(gate(.)). Cached are the latent and the rotated key part (csrc/attn_latent.cuh).
+ * The embedding row is multiplied by embedding_scale. Computed in f32 whatever the precision: norms, the residual,
+ * rotation, scores and weights, routing, recurrence.
  * ---------------------------------------------------------------------- */
 #define NERVA_HIP_MIXER_ATTENTION 1u
 #define NERVA_HIP_MIXER_MINGRU 2u
+#define NERVA_HIP_MIXER_LATENT 3u
+#define NERVA_HIP_STACK_SANDWICH 0u
+#define NERVA_HIP_STACK_PARALLEL 1u
 #define NERVA_HIP_OWN_KEYS 4294967295u
 #define NERVA_HIP_PRECISION_16 0u /* 16-bit inputs of the matrix products, 16-bit keys and values */
 #define NERVA_HIP_PRECISION_32 1u /* f32 throughout (weights stay 16-bit values): a checking mode, not a fast one */
 
 typedef struct NervaHipStackLayer {
   uint32_t mixer;                                  /* NERVA_HIP_MIXER_* */
-  uint32_t heads, kv_heads, key_dim, value_dim;    /* attention */
+  uint32_t heads, kv_heads, key_dim, value_dim;    /* attention; latent (key_dim: the unrotated elements; no kv_heads) */
   uint32_t rotary_dims;
   float rotary_base, score_scale;
   uint32_t chunk_tokens, kv_layer;
   uint32_t width;                                  /* minGRU */
-  uint32_t ff;                                     /* feed-forward width, 0 = none */
+  uint32_t ff;                                     /* dense feed-forward's width, 0 = none */
+  uint32_t q_rank, kv_rank, rotary_key_dim, window_tokens;   /* latent */
+  uint32_t experts, experts_per_token, expert_ff;  /* routed experts, 0 = none */
+  float expert_limit;
+  uint32_t shared_ff;                              /* expert for every token, 0 = none */
+  float shared_limit;
 } NervaHipStackLayer;
 
 /* The weights come through a declared weight plan (NervaHipHfDecodeSequenceWeightBlock) over this order of 16-bit
- * tensors: embedding; per layer norm1 w, b, norm1b w, b, [norm2 w, b, norm2b w, b], then attention: q, [k, v,] gate,
- * mixing, sinks, o - or minGRU: z, x, gate, z bias, x bias, o - then [up, down, activation (2 numbers)]; final norm
- * w, b. */
+ * tensors: embedding; per layer norm1 w, b, norm1b w, b, [norm2 w, b, norm2b w, b] (PARALLEL: norm1 w, [norm2 w]), then
+ * attention: q, [k, v,] gate, mixing, sinks, o - or minGRU: z, x, gate, z bias, x bias, o - or latent: dq, dkv, gate,
+ * norm of dq, norm of dkv, uq, uk, uv, o - then [up, down, activation (2 numbers)] or [router, per expert gate, up, down,
+ * [shared gate, up, down]]; final norm w, b (PARALLEL: w, then the head). */
 typedef struct NervaHipStackSessionCreateRequest {
   uint32_t dtype;      /* NERVA_HIP_DTYPE_BF16 */
   uint32_t precision;  /* NERVA_HIP_PRECISION_* */
   uint32_t hidden, vocab_size, layer_count, max_context_tokens;
   float norm_eps;
+  uint32_t arrangement;                   /* NERVA_HIP_STACK_* */
+  float embedding_scale, logit_scale;     /* SANDWICH: logit_scale 1 */
   const NervaHipStackLayer *layers;
   uint32_t planned_weight_blocks, planned_gpu_resident_blocks, planned_gpu_staged_blocks;
   uint64_t planned_weight_bytes, planned_gpu_resident_weight_bytes, planned_gpu_staged_weight_bytes;

@@ -22,6 +22,13 @@ __device__ __forceinline__ float xielu(float z, const XieluParams &a) {
   return (z > 0.0f ? a.above * z * z : a.below * (expm1f(low) - low)) + 0.5f * z;
 }
 
+// Gated linear unit with bounds: the gate from above, the linear part on both sides and moved up by one.
+__device__ __forceinline__ float clamped_glu(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g * sigmoid(1.702f * g) * (u + 1.0f);
+}
+
 // minGRU: gate and candidate from the current token alone (pre-activations with their biases added).
 __device__ __forceinline__ float mingru_candidate(float u) { return u >= 0.0f ? u + 0.5f : sigmoid(u); }
 __device__ __forceinline__ float mingru_step(float z_pre, float u, float state) {

@@ -15,12 +15,15 @@
 namespace nv {
 
 // Tensors of one layer in device memory. Row-concatenated: w_in is [q; k; v; gate] ([q; gate] where the keys are
-// another layer's) or [z; candidate; gate].
+// another layer's), [z; candidate; gate] or [query latent; latent and rotated key part; gate].
 struct StackLayer {
   NervaHipStackLayer spec{};
-  const uint16_t *norm[8] = {};   // norm1 w, b, norm1b w, b, norm2 w, b, norm2b w, b
+  const uint16_t *norm[8] = {};   // norm1 w, b, norm1b w, b, norm2 w, b, norm2b w, b (parallel layers: norm1 w, norm2 w)
   const uint16_t *w_in = nullptr, *w_out = nullptr, *talk = nullptr, *sink = nullptr, *z_bias = nullptr, *x_bias = nullptr,
                  *w_up = nullptr, *w_down = nullptr, *act = nullptr;
+  const uint16_t *q_norm = nullptr, *kv_norm = nullptr, *w_uq = nullptr, *w_uk = nullptr, *w_uv = nullptr;   // latent attention
+  // experts: [experts][gate rows; up rows] and [experts][down], the shared one likewise
+  const uint16_t *router = nullptr, *e_in = nullptr, *e_out = nullptr, *shared_in = nullptr, *shared_out = nullptr;
   uint32_t in_rows = 0, out_cols = 0;
   uint32_t q_col = 0, k_col = 0, v_col = 0, gate_col = 0;
   uint32_t rotation = 0;          // first column of the layer's angles in a token's rotation row
@@ -30,14 +33,21 @@ struct StackLayer {
   uint32_t table_offset = 0;             // entries into the session's block tables
   uint32_t ring_blocks = 0;
   uint64_t state_offset = 0;             // floats into the session's recurrent state (minGRU)
-  bool own_cache() const { return spec.mixer == NERVA_HIP_MIXER_ATTENTION && spec.kv_layer == NERVA_HIP_OWN_KEYS; }
+  bool own_cache() const {
+    return spec.mixer == NERVA_HIP_MIXER_LATENT || (spec.mixer == NERVA_HIP_MIXER_ATTENTION && spec.kv_layer == NERVA_HIP_OWN_KEYS);
+  }
+  uint32_t q_rows() const { return spec.heads * (spec.key_dim + spec.rotary_key_dim); }   // latent attention
 };
 
 struct StackModel {
   std::vector<StackLayer> layers;
   uint32_t precision = NERVA_HIP_PRECISION_16;
+  uint32_t arrangement = NERVA_HIP_STACK_SANDWICH;
+  float embedding_scale = 1.0f, logit_scale = 1.0f;
   const uint16_t *final_w = nullptr, *final_b = nullptr;
-  uint32_t max_in = 0, max_mix = 0, max_ff = 0;   // widest input projection, mixer output, feed-forward
+  // widest input projection, mixer output, feed-forward (activations of a token), query latent, queries, router, choices
+  uint32_t max_in = 0, max_mix = 0, max_ff = 0, max_q_rank = 0, max_q = 0, max_experts = 0, max_top = 0;
+  uint64_t plan_bytes = 0;                        // routing of a block (moe_rows.cuh)
   std::vector<float> angle_step;                  // per angle: radians per position
   std::vector<uint32_t> angle_cos, angle_sin;     // ... and its two columns in a token's rotation row
   uint32_t rotation_columns = 0;

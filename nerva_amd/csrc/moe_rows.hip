@@ -1,0 +1,368 @@
+// Routed experts over blocks of token rows (see moe_rows.cuh).
+#include "moe_rows.cuh"
+
+#include <algorithm>
+
+#include "activations.cuh"
+
+namespace nv {
+
+namespace {
+
+typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
+typedef float f32x4_t __attribute__((ext_vector_type(4)));
+
+__device__ __forceinline__ f32x4_t mfma_k32(const uint4 &a, const uint4 &b, f32x4_t c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, a), __builtin_bit_cast(bf16x8_t, b), c, 0, 0, 0);
+}
+
+// ---- routing ---------------------------------------------------------------------------------
+
+// One wave per token: scores in registers, `top` rounds of a wave-wide maximum.
+constexpr uint32_t kScoreRegs = kMaxExperts / kWave;
+__global__ __launch_bounds__(kBlock) void moe_route_rows_kernel(MoeRouteRows p) {
+  const uint32_t t = blockIdx.x * kWavesPerBlock + threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  if (t >= p.tokens) return;
+  const float *z = p.logits + static_cast<uint64_t>(t) * p.experts;
+  float s[kScoreRegs];
+#pragma unroll
+  for (uint32_t i = 0; i < kScoreRegs; ++i) {
+    const uint32_t e = i * kWave + lane;
+    s[i] = -1.0f;
+    if (i * kWave < p.experts && e < p.experts) s[i] = 1.0f / (1.0f + expf(-z[e]));
+  }
+  float sum = 0.0f, mine = 0.0f;   // lane k keeps choice k
+  uint32_t mine_id = 0;
+  for (uint32_t k = 0; k < p.top; ++k) {
+    Best b{0.0f, 0u, 0u};
+#pragma unroll
+    for (uint32_t i = 0; i < kScoreRegs; ++i) {
+      if (i * kWave >= p.experts) break;
+      const Best c{s[i], i * kWave + lane, s[i] >= 0.0f ? 1u : 0u};
+      if (better(c, b)) b = c;
+    }
+    b = wave_best(b);
+    // (scores that are no numbers: some expert that exists, so that every slot has one)
+    const uint32_t e = b.has != 0 ? b.index : k;
+#pragma unroll
+    for (uint32_t i = 0; i < kScoreRegs; ++i)
+      if (i * kWave + lane == e) s[i] = -1.0f;
+    sum += b.value;
+    if (lane == k) {
+      mine = b.value;
+      mine_id = e;
+    }
+  }
+  if (lane < p.top) {
+    p.plan.ids[static_cast<uint64_t>(t) * p.top + lane] = mine_id;
+    p.plan.weights[static_cast<uint64_t>(t) * p.top + lane] = mine / (sum + 1e-20f);
+  }
+}
+
+// One workgroup: counts per expert, places, tiles.
+constexpr uint32_t kSortThreads = 1024;
+__global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(MoeRouteRows p) {
+  __shared__ uint32_t count[kMaxExperts], first[kMaxExperts], tile_at[kMaxExperts], wave_total[2][kSortThreads / kWave];
+  const uint32_t slots = p.tokens * p.top, tid = threadIdx.x;
+  for (uint32_t e = tid; e < kMaxExperts; e += kSortThreads) count[e] = 0;
+  __syncthreads();
+  for (uint32_t i = tid; i < slots; i += kSortThreads) atomicAdd(&count[min(p.plan.ids[i], p.experts - 1)], 1u);
+  __syncthreads();
+  // exclusive sums over the experts (one each), of slots and of tiles
+  static_assert(kMaxExperts == kSortThreads, "one expert a thread");
+  const uint32_t n = count[tid], tiles = (n + kExpertTile - 1) / kExpertTile;
+  uint32_t a = n, b = tiles;
+#pragma unroll
+  for (uint32_t o = 1; o < kWave; o <<= 1) {
+    const uint32_t ua = __shfl_up(a, o, kWave), ub = __shfl_up(b, o, kWave);
+    if (tid % kWave >= o) {
+      a += ua;
+      b += ub;
+    }
+  }
+  if (tid % kWave == kWave - 1) {
+    wave_total[0][tid / kWave] = a;
+    wave_total[1][tid / kWave] = b;
+  }
+  __syncthreads();
+  for (uint32_t w = 0; w < tid / kWave; ++w) {
+    a += wave_total[0][w];
+    b += wave_total[1][w];
+  }
+  first[tid] = a - n;
+  tile_at[tid] = b - tiles;
+  if (tid == kSortThreads - 1) *p.plan.tile_count = b;
+  for (uint32_t i = 0; i < tiles; ++i)
+    p.plan.tiles[b - tiles + i] = make_uint4(tid, a - n + i * kExpertTile, min(kExpertTile, n - i * kExpertTile), 0u);
+  __syncthreads();
+  for (uint32_t i = tid; i < slots; i += kSortThreads) {
+    const uint32_t at = atomicAdd(&first[min(p.plan.ids[i], p.experts - 1)], 1u);
+    p.plan.sorted[at] = i;
+  }
+}
+
+// ---- products --------------------------------------------------------------------------------
+
+enum : int { kExpertGateUp = 0, kExpertDown = 1 };
+
+struct Products {
+  const uint16_t *w;          // the experts' matrices
+  const uint16_t *x16;
+  const float *x32;
+  uint16_t *act16;
+  float *act32, *out;
+  uint32_t rows, cols;        // output rows (gate/up: of either half), columns
+  uint32_t tokens, top;
+  float limit;
+  const uint4 *tiles;         // null: one expert, consecutive tokens
+  const uint32_t *tile_count, *sorted;
+};
+
+struct Tile {
+  uint32_t expert, first, count;
+};
+__device__ __forceinline__ bool tile_of(const Products &p, uint32_t i, Tile &t) {
+  if (p.tiles == nullptr) {
+    t = Tile{0u, i * kExpertTile, min(kExpertTile, p.tokens - i * kExpertTile)};
+    return true;
+  }
+  if (i >= *p.tile_count) return false;
+  const uint4 v = p.tiles[i];
+  t = Tile{v.x, v.y, v.z};
+  return true;
+}
+__device__ __forceinline__ uint32_t slot_of(const Products &p, uint32_t place) { return p.tiles == nullptr ? place : p.sorted[place]; }
+// Row of the input that belongs to a slot: the token for the gate/up products, the slot itself for the down product.
+template <int EPI>
+__device__ __forceinline__ uint32_t input_row(const Products &p, uint32_t slot) {
+  return EPI == kExpertGateUp ? slot / p.top : slot;
+}
+
+constexpr uint32_t kRows = 128;         // matrix rows of a workgroup (gate/up: 64 of each)
+constexpr uint32_t kStep = 64;          // columns staged at a time
+constexpr uint32_t kPitch = kStep + 8;  // LDS row pitch: 16 bytes of padding
+
+// Eight columns of a row from `c` on; columns past the end are zero.
+template <bool VEC>
+__device__ __forceinline__ uint4 piece8(const uint16_t *row, uint32_t c, uint32_t cols) {
+  if constexpr (VEC) {
+    return c < cols ? *reinterpret_cast<const uint4 *>(row + c) : make_uint4(0u, 0u, 0u, 0u);
+  } else {
+    uint32_t w[4];
+#pragma unroll
+    for (uint32_t e = 0; e < 4; ++e) {
+      const uint32_t lo = c + 2 * e < cols ? row[c + 2 * e] : 0u, hi = c + 2 * e + 1 < cols ? row[c + 2 * e + 1] : 0u;
+      w[e] = lo | (hi << 16);
+    }
+    return make_uint4(w[0], w[1], w[2], w[3]);
+  }
+}
+
+template <uint32_t DT, int EPI, bool VEC>
+__global__ __launch_bounds__(kBlock) void expert_rows_kernel(Products p) {
+  __shared__ __align__(16) uint16_t ws[kRows * kPitch];
+  __shared__ __align__(16) uint16_t xs[kExpertTile * kPitch];
+  __shared__ uint32_t slots[kExpertTile];
+  Tile tile;
+  if (!tile_of(p, blockIdx.y, tile)) return;
+  const uint32_t lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
+  constexpr uint32_t kOutRows = EPI == kExpertGateUp ? kRows / 2 : kRows;
+  const uint32_t row0 = blockIdx.x * kOutRows, cols = p.cols;
+  if (threadIdx.x < kExpertTile) slots[threadIdx.x] = slot_of(p, tile.first + min(threadIdx.x, tile.count - 1));
+  __syncthreads();
+  const uint16_t *w = p.w + static_cast<uint64_t>(tile.expert) * (EPI == kExpertGateUp ? 2u : 1u) * p.rows * cols;
+  // staging: thread -> (row of the tile, eight columns), four rows of the matrix and two of the input
+  const uint32_t sr = threadIdx.x / 8u, sc = (threadIdx.x % 8u) * 8u;
+  const uint16_t *wr[4], *xr[2];
+#pragma unroll
+  for (uint32_t i = 0; i < 4; ++i) {
+    const uint32_t r = sr + 32u * i;
+    const uint32_t row = EPI == kExpertGateUp ? (r / 64u) * p.rows + min(row0 + r % 64u, p.rows - 1) : min(row0 + r, p.rows - 1);
+    wr[i] = w + static_cast<uint64_t>(row) * cols;
+  }
+#pragma unroll
+  for (uint32_t i = 0; i < 2; ++i) xr[i] = p.x16 + static_cast<uint64_t>(input_row<EPI>(p, slots[sr + 32u * i])) * cols;
+  uint4 wq[4], xq[2];
+#pragma unroll
+  for (uint32_t i = 0; i < 4; ++i) wq[i] = piece8<VEC>(wr[i], sc, cols);
+#pragma unroll
+  for (uint32_t i = 0; i < 2; ++i) xq[i] = piece8<VEC>(xr[i], sc, cols);
+  // a wave: 32 gate and the 32 up rows of the same outputs (down: 64 rows), 32 slots
+  f32x4_t acc[4][2];
+#pragma unroll
+  for (int a = 0; a < 4; ++a)
+#pragma unroll
+    for (int b = 0; b < 2; ++b) acc[a][b] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+  const uint32_t n = lane & 15u, q = lane >> 4, half = wave & 1u;
+  const auto w_row = [&](uint32_t i) { return EPI == kExpertGateUp ? (i / 2u) * 64u + half * 32u + (i % 2u) * 16u : half * 64u + i * 16u; };
+  const uint16_t *b_at = xs + ((wave >> 1) * 32u + n) * kPitch + q * 8u;
+  for (uint32_t k = 0; k < cols; k += kStep) {
+    __syncthreads();
+#pragma unroll
+    for (uint32_t i = 0; i < 4; ++i) *reinterpret_cast<uint4 *>(ws + (sr + 32u * i) * kPitch + sc) = wq[i];
+#pragma unroll
+    for (uint32_t i = 0; i < 2; ++i) *reinterpret_cast<uint4 *>(xs + (sr + 32u * i) * kPitch + sc) = xq[i];
+    __syncthreads();
+    if (k + kStep < cols) {
+#pragma unroll
+      for (uint32_t i = 0; i < 4; ++i) wq[i] = piece8<VEC>(wr[i], k + kStep + sc, cols);
+#pragma unroll
+      for (uint32_t i = 0; i < 2; ++i) xq[i] = piece8<VEC>(xr[i], k + kStep + sc, cols);
+    }
+#pragma unroll
+    for (uint32_t s = 0; s < kStep / 32u; ++s) {
+      uint4 a[4], b[2];
+#pragma unroll
+      for (uint32_t i = 0; i < 4; ++i) a[i] = *reinterpret_cast<const uint4 *>(ws + (w_row(i) + n) * kPitch + q * 8u + s * 32u);
+#pragma unroll
+      for (uint32_t j = 0; j < 2; ++j) b[j] = *reinterpret_cast<const uint4 *>(b_at + j * 16u * kPitch + s * 32u);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) acc[i][j] = mfma_k32(a[i], b[j], acc[i][j]);
+    }
+  }
+#pragma unroll
+  for (uint32_t j = 0; j < 2; ++j) {
+    const uint32_t t = (wave >> 1) * 32u + j * 16u + n;
+    if (t >= tile.count) continue;
+    const uint64_t at = static_cast<uint64_t>(slots[t]) * p.rows;
+#pragma unroll
+    for (uint32_t i = 0; i < (EPI == kExpertGateUp ? 2u : 4u); ++i)
+#pragma unroll
+      for (uint32_t r = 0; r < 4; ++r) {
+        const uint32_t row = row0 + (EPI == kExpertGateUp ? half * 32u : half * 64u) + i * 16u + q * 4u + r;
+        if (row >= p.rows) continue;
+        if constexpr (EPI == kExpertGateUp) p.act16[at + row] = enc16<DT>(clamped_glu(acc[i][j][r], acc[i + 2][j][r], p.limit));
+        else p.out[at + row] = acc[i][j][r];
+      }
+  }
+}
+
+constexpr uint32_t kTile32 = 64, kStep32 = 16;   // output rows of a workgroup, columns staged at a time (f32 rows)
+
+template <uint32_t DT, int EPI>
+__global__ __launch_bounds__(kBlock) void expert_rows_f32_kernel(Products p) {
+  constexpr uint32_t M = EPI == kExpertGateUp ? 2 : 1;   // matrices that meet in one output
+  __shared__ float ws[M][kStep32][kTile32 + 4], xs[kStep32][kExpertTile + 4];
+  __shared__ uint32_t slots[kExpertTile];
+  Tile tile;
+  if (!tile_of(p, blockIdx.y, tile)) return;
+  const uint32_t row0 = blockIdx.x * kTile32, cols = p.cols;
+  if (threadIdx.x < kExpertTile) slots[threadIdx.x] = slot_of(p, tile.first + min(threadIdx.x, tile.count - 1));
+  __syncthreads();
+  const uint16_t *w = p.w + static_cast<uint64_t>(tile.expert) * M * p.rows * cols;
+  const uint32_t tr = threadIdx.x % 16u, tt = threadIdx.x / 16u;
+  float acc[M][4][4] = {};
+  for (uint32_t k = 0; k < cols; k += kStep32) {
+    __syncthreads();
+#pragma unroll
+    for (uint32_t i = 0; i < 4; ++i) {
+      const uint32_t r = threadIdx.x / 16u + 16u * i, c = threadIdx.x % 16u;
+      const bool in = k + c < cols;
+#pragma unroll
+      for (uint32_t m = 0; m < M; ++m)
+        ws[m][c][r] = in ? dec16<DT>(w[(static_cast<uint64_t>(m) * p.rows + min(row0 + r, p.rows - 1)) * cols + k + c]) : 0.0f;
+      xs[c][r] = in ? p.x32[static_cast<uint64_t>(input_row<EPI>(p, slots[r])) * cols + k + c] : 0.0f;
+    }
+    __syncthreads();
+#pragma unroll
+    for (uint32_t c = 0; c < kStep32; ++c)
+#pragma unroll
+      for (uint32_t m = 0; m < M; ++m)
+#pragma unroll
+        for (uint32_t i = 0; i < 4; ++i)
+#pragma unroll
+          for (uint32_t j = 0; j < 4; ++j) acc[m][i][j] = fmaf(ws[m][c][tr + 16u * i], xs[c][tt + 16u * j], acc[m][i][j]);
+  }
+#pragma unroll
+  for (uint32_t j = 0; j < 4; ++j) {
+    const uint32_t t = tt + 16u * j;
+    if (t >= tile.count) continue;
+    const uint64_t at = static_cast<uint64_t>(slots[t]) * p.rows;
+#pragma unroll
+    for (uint32_t i = 0; i < 4; ++i) {
+      const uint32_t row = row0 + tr + 16u * i;
+      if (row >= p.rows) continue;
+      if constexpr (EPI == kExpertGateUp) p.act32[at + row] = clamped_glu(acc[0][i][j], acc[M - 1][i][j], p.limit);
+      else p.out[at + row] = acc[0][i][j];
+    }
+  }
+}
+
+template <int EPI>
+hipError_t launch(const ExpertRows &e, hipStream_t stream) {
+  Products p{};
+  const bool narrow = e.x16 != nullptr;
+  p.w = EPI == kExpertGateUp ? e.w_gate_up : e.w_down;
+  p.x16 = EPI == kExpertGateUp ? e.x16 : e.act16;
+  p.x32 = EPI == kExpertGateUp ? e.x32 : e.act32;
+  p.act16 = e.act16;
+  p.act32 = e.act32;
+  p.out = e.out;
+  p.rows = EPI == kExpertGateUp ? e.ff : e.hidden;
+  p.cols = EPI == kExpertGateUp ? e.hidden : e.ff;
+  p.tokens = e.tokens;
+  p.top = e.top;
+  p.limit = e.limit;
+  uint32_t tiles = (e.tokens + kExpertTile - 1) / kExpertTile;
+  if (e.plan != nullptr) {
+    p.tiles = e.plan->tiles;
+    p.tile_count = e.plan->tile_count;
+    p.sorted = e.plan->sorted;
+    tiles = moe_max_tiles(e.tokens, e.top, e.experts);
+  }
+  const bool aligned = ((reinterpret_cast<uintptr_t>(p.w) | reinterpret_cast<uintptr_t>(p.x16)) & 15u) == 0;
+  if (tiles > 65535u) return hipErrorInvalidValue;
+  if (!narrow) {
+    hipLaunchKernelGGL((expert_rows_f32_kernel<kBF16, EPI>), dim3((p.rows + kTile32 - 1) / kTile32, tiles), dim3(kBlock), 0, stream, p);
+  } else {
+    constexpr uint32_t kOutRows = EPI == kExpertGateUp ? kRows / 2 : kRows;
+    const dim3 grid((p.rows + kOutRows - 1) / kOutRows, tiles);
+    if (p.cols % 8 == 0 && aligned) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true>), grid, dim3(kBlock), 0, stream, p);
+    else hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, false>), grid, dim3(kBlock), 0, stream, p);
+  }
+  return hipGetLastError();
+}
+
+bool rows_ok(uint32_t dtype, const ExpertRows &p) {
+  return dtype == kBF16 && p.w_gate_up != nullptr && p.w_down != nullptr && (p.x16 == nullptr) != (p.x32 == nullptr) &&
+         (p.x16 != nullptr ? p.act16 != nullptr : p.act32 != nullptr) && p.hidden != 0 && p.ff != 0 && p.tokens != 0 && p.top != 0 &&
+         p.experts != 0 && (p.plan != nullptr ? p.experts <= kMaxExperts && p.top <= kMaxTop && p.top <= p.experts : p.experts == 1 && p.top == 1);
+}
+
+}  // namespace
+
+uint64_t moe_plan_bytes(uint32_t tokens, uint32_t top, uint32_t experts) {
+  return static_cast<uint64_t>(tokens) * top * 12 + static_cast<uint64_t>(moe_max_tiles(tokens, top, experts)) * sizeof(uint4) + 64;
+}
+
+MoePlan moe_plan_at(void *base, uint32_t tokens, uint32_t top, uint32_t experts) {
+  const uint64_t slots = static_cast<uint64_t>(tokens) * top;
+  MoePlan m;
+  m.tiles = static_cast<uint4 *>(base);
+  m.ids = reinterpret_cast<uint32_t *>(m.tiles + moe_max_tiles(tokens, top, experts));
+  m.weights = reinterpret_cast<float *>(m.ids + slots);
+  m.sorted = reinterpret_cast<uint32_t *>(m.weights + slots);
+  m.tile_count = m.sorted + slots;
+  return m;
+}
+
+hipError_t launch_moe_route_rows(const MoeRouteRows &p, hipStream_t stream) {
+  if (p.logits == nullptr || p.tokens == 0 || p.experts == 0 || p.experts > kMaxExperts || p.top == 0 || p.top > p.experts || p.top > kMaxTop)
+    return hipErrorInvalidValue;
+  hipLaunchKernelGGL(moe_route_rows_kernel, dim3((p.tokens + kWavesPerBlock - 1) / kWavesPerBlock), dim3(kBlock), 0, stream, p);
+  hipError_t err = hipGetLastError();
+  if (err != hipSuccess) return err;
+  hipLaunchKernelGGL(moe_sort_kernel, dim3(1), dim3(kSortThreads), 0, stream, p);
+  return hipGetLastError();
+}
+
+hipError_t launch_expert_gate_up(uint32_t dtype, const ExpertRows &p, hipStream_t stream) {
+  return rows_ok(dtype, p) ? launch<kExpertGateUp>(p, stream) : hipErrorInvalidValue;
+}
+hipError_t launch_expert_down(uint32_t dtype, const ExpertRows &p, hipStream_t stream) {
+  return rows_ok(dtype, p) && p.out != nullptr ? launch<kExpertDown>(p, stream) : hipErrorInvalidValue;
+}
+
+}  // namespace nv

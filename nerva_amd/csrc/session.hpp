@@ -122,6 +122,14 @@ struct NervaHipHfDecodeSequenceSession {
   float *stack_state = nullptr;      // recurrent state, f32, all recurrent layers
   uint64_t stack_state_bytes = 0;
   float *y = nullptr, *py = nullptr; // output of the sublayer under way, before its norm: decode row, token rows
+  uint64_t stack_launches = 0;       // kernel launches of the step enqueued last (where the layers do not tell)
+  // layers whose sublayers read the same row: the feed-forward's normalised rows and output
+  void *pxn2 = nullptr;
+  float *pz = nullptr;
+  void *pql = nullptr;               // latent attention: normalised query latents, queries
+  float *pq = nullptr;
+  float *prouter = nullptr, *pslots = nullptr;   // experts: router logits, one output row per (token, choice)
+  void *pplan = nullptr;             // ... and the block's routing (MoePlan)
   void *pwant = nullptr;             // normalised rows whose logits are asked for, with their row numbers and logits
   uint32_t *pwant_rows = nullptr;
   float *pwant_logits = nullptr;

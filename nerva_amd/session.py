@@ -208,6 +208,7 @@ class DecodeSession:
         req = abi.NervaHipStackSessionCreateRequest()
         req.dtype, req.precision, req.hidden, req.vocab_size = 1, precision, config.hidden, config.vocab
         req.layer_count, req.max_context_tokens, req.norm_eps = len(config.layers), max_context, config.eps
+        req.arrangement, req.embedding_scale, req.logit_scale = config.arrangement, config.embedding_scale, config.logit_scale
         layers = config.c_layers()
         req.layers = layers
         return req, layers

@@ -33,10 +33,10 @@ def stack_config(width, heads, kv_heads, ff, channels, layers, chunk):
     out = []
     for i in range(layers):
         if i % 2:
-            out.append((stacks.MinGru(channels), ff))
+            out.append((stacks.MinGru(channels), stacks.XieluFeedForward(ff)))
         else:
             out.append((stacks.Attention(heads, kv_heads, HEAD, HEAD, HEAD, 1e6, HEAD ** -0.5, chunk,
-                                         i - 2 if i % 4 == 2 else None), ff))
+                                         i - 2 if i % 4 == 2 else None), stacks.XieluFeedForward(ff)))
     return stacks.StackConfig(width, VOCAB, 1e-6, out)
 
 

@@ -58,18 +58,85 @@ class MinGru:
         layer.width = self.width
 
 
-class StackConfig:
-    """hidden, vocab, eps and the layers: (mixer, feed-forward width or 0)."""
+class LatentAttention:
+    """Attention whose keys and values are projections of one normalised latent per token, with a rotated key part shared
+    by the heads, an output gate and a sliding window (0: none)."""
+    kind = abi.NERVA_HIP_MIXER_LATENT
 
-    def __init__(self, hidden, vocab, eps, layers):
+    def __init__(self, heads, key_dim, rotary_key_dim, value_dim, q_rank, kv_rank, rotary_dims, rotary_base, score_scale,
+                 window_tokens):
+        self.heads, self.key_dim, self.rotary_key_dim, self.value_dim = heads, key_dim, rotary_key_dim, value_dim
+        self.q_rank, self.kv_rank, self.window_tokens = q_rank, kv_rank, window_tokens
+        self.rotary_dims, self.rotary_base, self.score_scale = rotary_dims, rotary_base, score_scale
+
+    def tensors(self, hidden):
+        values = self.heads * self.value_dim
+        return [("dq", [self.q_rank, hidden]), ("dkv", [self.kv_rank + self.rotary_key_dim, hidden]), ("g", [values, hidden]),
+                ("dq.norm", [self.q_rank]), ("dkv.norm", [self.kv_rank]),
+                ("uq", [self.heads * (self.key_dim + self.rotary_key_dim), self.q_rank]),
+                ("uk", [self.heads * self.key_dim, self.kv_rank]), ("uv", [values, self.kv_rank]), ("o", [hidden, values])]
+
+    def fill(self, layer):
+        layer.heads, layer.key_dim, layer.value_dim, layer.rotary_key_dim = self.heads, self.key_dim, self.value_dim, self.rotary_key_dim
+        layer.q_rank, layer.kv_rank, layer.window_tokens = self.q_rank, self.kv_rank, self.window_tokens
+        layer.rotary_dims, layer.rotary_base, layer.score_scale = self.rotary_dims, self.rotary_base, self.score_scale
+
+
+class XieluFeedForward:
+    """Dense: up, xIELU, down."""
+
+    def __init__(self, ff):
+        self.ff = ff
+
+    def tensors(self, hidden):
+        return [("up", [self.ff, hidden]), ("down", [hidden, self.ff]), ("act", [2])]
+
+    def fill(self, layer):
+        layer.ff = self.ff
+
+
+class ExpertFeedForward:
+    """Routed experts with bounded gates; an expert that takes every token besides, where shared_ff != 0."""
+
+    def __init__(self, experts, top, ff, limit, shared_ff=0, shared_limit=0.0):
+        self.experts, self.top, self.ff, self.limit = experts, top, ff, limit
+        self.shared_ff, self.shared_limit = shared_ff, shared_limit
+
+    def tensors(self, hidden):
+        out = [("router", [self.experts, hidden])]
+        names = [("e%d" % e, self.ff) for e in range(self.experts)] + ([("shared", self.shared_ff)] if self.shared_ff else [])
+        for name, ff in names:
+            out += [(name + ".gate", [ff, hidden]), (name + ".up", [ff, hidden]), (name + ".down", [hidden, ff])]
+        return out
+
+    def fill(self, layer):
+        layer.experts, layer.experts_per_token, layer.expert_ff, layer.expert_limit = self.experts, self.top, self.ff, self.limit
+        layer.shared_ff, layer.shared_limit = self.shared_ff, self.shared_limit
+
+
+SANDWICH, PARALLEL = abi.NERVA_HIP_STACK_SANDWICH, abi.NERVA_HIP_STACK_PARALLEL
+
+
+class StackConfig:
+    """hidden, vocab, eps and the layers: (mixer, feed-forward or None). `arrangement`: one sublayer after the other, each
+    between two layer norms, the embedding as the head (SANDWICH); or both on the same row, each behind an RMS norm, and a
+    head of its own (PARALLEL)."""
+
+    def __init__(self, hidden, vocab, eps, layers, arrangement=SANDWICH, embedding_scale=1.0, logit_scale=1.0):
         self.hidden, self.vocab, self.eps, self.layers = hidden, vocab, eps, list(layers)
+        self.arrangement, self.embedding_scale, self.logit_scale = arrangement, embedding_scale, logit_scale
 
     def c_layers(self):
         out = (abi.NervaHipStackLayer * len(self.layers))()
         for c, (mixer, ff) in zip(out, self.layers):
-            c.mixer, c.ff, c.kv_layer = mixer.kind, ff, OWN_KEYS
+            c.mixer, c.kv_layer = mixer.kind, OWN_KEYS
             mixer.fill(c)
+            if ff is not None:
+                ff.fill(c)
         return out
+
+    def _norm(self, name):
+        return [(name, [self.hidden])] + ([(name + ".b", [self.hidden])] if self.arrangement == SANDWICH else [])
 
     def manifest(self):
         """(name, shape) of every tensor in the order of the weight arena."""
@@ -77,12 +144,13 @@ class StackConfig:
         out = [("embed", [self.vocab, h])]
         for i, (mixer, ff) in enumerate(self.layers):
             name = "l%d." % i
-            for norm in ("norm1", "norm1b") + (("norm2", "norm2b") if ff else ()):
-                out += [(name + norm, [h]), (name + norm + ".b", [h])]
+            norms = ("norm1", "norm1b", "norm2", "norm2b") if self.arrangement == SANDWICH else ("norm1", "norm2")
+            for norm in norms if ff is not None else norms[:len(norms) // 2]:
+                out += self._norm(name + norm)
             out += [(name + "mix." + t, shape) for t, shape in mixer.tensors(h)]
-            if ff:
-                out += [(name + "mlp.up", [ff, h]), (name + "mlp.down", [h, ff]), (name + "mlp.act", [2])]
-        return out + [("final.norm", [h]), ("final.norm.b", [h])]
+            if ff is not None:
+                out += [(name + "mlp." + t, shape) for t, shape in ff.tensors(h)]
+        return out + self._norm("final.norm") + ([("head", [self.vocab, h])] if self.arrangement == PARALLEL else [])
 
 
 class StackWeights:
@@ -145,13 +213,55 @@ def read_retorax(config):
             mixer = MinGru(_number(m.get("width"), what + " width"))
         else:
             raise CheckpointError("config.json: %s has type %r" % (what, kind))
-        mlp, ff = entry.get("mlp"), 0
+        mlp, ff = entry.get("mlp"), None
         if mlp is not None:
             if not isinstance(mlp, dict) or mlp.get("kind") != "dense":
                 raise CheckpointError("config.json: %s has a feed-forward of kind %r" % (what, mlp))
-            ff = _number(mlp.get("ff"), what + " ff")
+            ff = XieluFeedForward(_number(mlp.get("ff"), what + " ff"))
         layers.append((mixer, ff))
     return StackConfig(hidden, vocab, eps, layers)
 
 
-READERS = {"Retorax": read_retorax}
+def read_kavuvik(config):
+    """Kavuvik: layers of latent attention through sliding windows beside routed experts (or none), both on the same row."""
+    hidden, vocab = _number(config.get("width"), "width"), _number(config.get("vocab"), "vocab")
+    eps = _number(_part(config, "norm", "the model").get("eps"), "norm.eps", integer=False, least=0.0)
+    embedding_scale = _number(_part(config, "embedding", "the model").get("scale"), "embedding.scale", integer=False, least=-math.inf)
+    logit_scale = _number(config.get("logit_scale"), "logit_scale", integer=False, least=-math.inf)
+    entries = config.get("layers")
+    if not isinstance(entries, list) or not entries:
+        raise CheckpointError("config.json: no layers")
+    layers = []
+    for i, entry in enumerate(entries):
+        what = "layer %d" % i
+        if entry.get("type") != "latent_attention":
+            raise CheckpointError("config.json: %s has type %r" % (what, entry.get("type")))
+        m = _part(entry, "mixer", what)
+        rot = _part(m, "rot", what)
+        window = 0 if m.get("mask") is None else _number(_part(m, "mask", what).get("size"), what + " mask.size")
+        sizes = {k: _number(m.get(k), "%s %s" % (what, k)) for k in ("heads", "dim", "rot_dim", "vdim", "q_rank", "kv_rank")}
+        mixer = LatentAttention(sizes["heads"], sizes["dim"], sizes["rot_dim"], sizes["vdim"], sizes["q_rank"], sizes["kv_rank"],
+                                _number(rot.get("dims"), what + " rot.dims", least=0),
+                                _number(rot.get("base"), what + " rot.base", integer=False, least=0.0),
+                                _number(m.get("scale"), what + " scale", integer=False, least=-math.inf), window)
+        if mixer.rotary_dims % 2 != 0 or mixer.rotary_dims > mixer.rotary_key_dim:
+            raise CheckpointError("config.json: %s has sizes that do not go together" % what)
+        mlp, ff = entry.get("mlp"), None
+        if mlp is not None:
+            if not isinstance(mlp, dict) or mlp.get("kind") != "moe":
+                raise CheckpointError("config.json: %s has a feed-forward of kind %r" % (what, mlp))
+            router, expert = _part(mlp, "router", what), _part(mlp, "expert", what)
+            ff = ExpertFeedForward(_number(router.get("experts"), what + " experts"), _number(router.get("top"), what + " top"),
+                                   _number(expert.get("ff"), what + " expert ff"),
+                                   _number(expert.get("limit"), what + " expert limit", integer=False, least=0.0))
+            if mlp.get("shared") is not None:
+                shared = _part(mlp, "shared", what)
+                ff.shared_ff = _number(shared.get("ff"), what + " shared ff")
+                ff.shared_limit = _number(shared.get("limit"), what + " shared limit", integer=False, least=0.0)
+            if ff.top > ff.experts:
+                raise CheckpointError("config.json: %s takes %d of %d experts" % (what, ff.top, ff.experts))
+        layers.append((mixer, ff))
+    return StackConfig(hidden, vocab, eps, layers, PARALLEL, embedding_scale, logit_scale)
+
+
+READERS = {"Kavuvik": read_kavuvik, "Retorax": read_retorax}
