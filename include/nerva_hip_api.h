@@ -861,7 +861,7 @@ int nerva_hip_session_profile_step(NervaHipHfDecodeSequenceSession *session, uin
  * never in three-wave workgroups), "gemm_block_rotate" (1 + the K-blocks between the places where consecutive row
  * groups of that kernel start their walk; 1: a common start), "mixed_attention_wide" (2: a mixed stack's attention layers
  * through the general kernel, whatever their shape; read at every launch, so a captured step keeps what it was
- * captured with). Values a kernel
+ * captured with), "latent_attention_wide" (2: the same for layers of attention over latents). Values a kernel
  * cannot take are ignored where they are read. -1 for an unknown name. A null name restores every built-in
  * choice. */
 int nerva_hip_test_set_tuning(const char *name, int32_t value);

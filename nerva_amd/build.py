@@ -16,7 +16,7 @@ LIB = os.path.join(HERE, "libnerva_hip.so")
 
 SOURCES = ["gemv_stream.hip", "fp8_gemv.hip", "attn_decode.hip", "attn_prompt.hip", "argmax.hip", "synth_fill.hip",
            "sampler.hip", "gemm_rows.hip", "gemm_block.hip", "gemm_any.hip", "norm_join.hip", "mingru.hip", "attn_mixed.hip",
-           "attn_mixed_wide.hip", "norm_rms.hip", "attn_latent.hip", "moe_rows.hip", "op_entry.hip", "decode_session.hip", "layer_stack.hip"]
+           "attn_mixed_wide.hip", "norm_rms.hip", "attn_latent.hip", "attn_latent_wide.hip", "moe_rows.hip", "op_entry.hip", "decode_session.hip", "layer_stack.hip"]
 
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function",
          # packed fp32 VALU ops are kept off for every device function of this library
@@ -49,7 +49,7 @@ def _spilling_kernels(remarks):
 # does not know that such a register is still being written, so a spill (or any copy) of it reads garbage:
 # these kernels must compile without scratch memory, which every build checks.
 HAND_ISSUED_LOADS = ("attn_step_kernel", "moe_gate_up_lean_kernel", "moe_down_lean_kernel", "fp8_gemv_lean_kernel",
-                     "gemm_deep_kernel")
+                     "gemm_deep_kernel", "latent_rows_kernel", "latent_absorb_kernel")
 
 
 def _compile(src):

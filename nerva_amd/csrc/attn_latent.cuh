@@ -51,6 +51,8 @@ struct LatentAttnParams {
   uint16_t *out16;             // [tokens][heads * value_dim], or null
   float *out32;                // likewise f32, used when out16 is null
   uint32_t packed_tiles;       // out16: != 0 -> matrix-operand order with that many token tiles
+  void *workspace;             // the wide kernels' queries, weighted latents and split partials (latent_workspace_bytes)
+  uint32_t last_block;         // highest logical block a launch may meet (sizes the split grid of a captured step)
 };
 
 __device__ __forceinline__ uint32_t window_start(uint32_t pos, uint32_t window) {
@@ -61,5 +63,12 @@ __device__ __forceinline__ uint32_t window_start(uint32_t pos, uint32_t window) 
 hipError_t launch_latent_prepare(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream);
 // Attention of the token rows, whose own latents are in the cache. Any shape.
 hipError_t launch_latent_attention(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream);
+// Wide layers, 16-bit cache (attn_latent_wide.hip): the same for a block of token rows (launch_latent_prepare has run) or
+// for a decode step (cursor set, one token), which also writes the token's cache row.
+bool latent_attention_wide(uint32_t heads, uint32_t key_dim, uint32_t rot_dim, uint32_t value_dim, uint32_t kv_rank);
+uint64_t latent_workspace_bytes(uint32_t heads, uint32_t rot_dim, uint32_t kv_rank, uint32_t max_tokens);
+hipError_t latent_wide_setup();   // once per process, outside stream capture
+hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream);
+uint32_t latent_wide_launches(bool decode);
 
 }  // namespace nv

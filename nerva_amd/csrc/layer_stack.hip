@@ -183,7 +183,12 @@ LatentAttnParams latent_params(Session *s, const StackLayer &w, const float *pro
   a.scale = w.spec.score_scale;
   a.cache32 = wide(s) ? 1u : 0u;
   a.max_steps = s->max_ctx;
+  a.workspace = s->attn_ws;
+  a.last_block = m.logical_blocks - 1;
   return a;
+}
+bool takes_latent_wide(const Session *s, const NervaHipStackLayer &d) {
+  return !wide(s) && latent_attention_wide(d.heads, d.key_dim, d.rotary_key_dim, d.value_dim, d.kv_rank) && tuning(kTuneLatentAttentionWide) != 2;
 }
 
 // Final norm, head, sampler of the row in (row.x, s->y): logits, slot[cursor], cursor + 1.
@@ -405,8 +410,9 @@ struct Block {
       a.packed_tiles = out_tiles;
       err = launch_latent_prepare(s->dtype, a, s->stream);
       if (err == hipSuccess) err = project(kGemmF32, w.w_uq, w.q_rows(), w.spec.q_rank, s->pql, q_tiles, s->pq, 0, nullptr);
-      if (err == hipSuccess) err = launch_latent_attention(s->dtype, a, s->stream);
-      launches += 1;
+      const bool fast = takes_latent_wide(s, w.spec);
+      if (err == hipSuccess) err = fast ? launch_latent_attention_wide(s->dtype, a, s->stream) : launch_latent_attention(s->dtype, a, s->stream);
+      launches += fast ? latent_wide_launches(at_cursor) : 1u;
     } else if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION) {
       MixedAttnParams a = attention_params(s, w, s->pqkv, s->prope);
       a.position = first;
@@ -999,7 +1005,8 @@ int create_stack(const NervaHipStackSessionCreateRequest *rq, bool synthetic, ui
   }
 
   s->stack = model;
-  hipError_t err = stack_setup_state(s, &out->failure_stage, true);
+  hipError_t err = latent_wide_setup();
+  if (err == hipSuccess) err = stack_setup_state(s, &out->failure_stage, true);
   uint64_t h2d = 0, syncs = 1;
   if (err == hipSuccess) {
     char *base = s->weights->base;
@@ -1105,6 +1112,9 @@ hipError_t nv::stack_setup_state(Session *s, int32_t *failure_stage, bool with_w
     if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION && !wide(s) &&
         mixed_attention_wide(w.spec.heads, w.spec.kv_heads, w.spec.key_dim, w.spec.value_dim))
       attn_ws_bytes = std::max(attn_ws_bytes, mixed_attention_workspace_bytes(w.spec.heads, kStackBlockTokens));
+    else if (w.spec.mixer == NERVA_HIP_MIXER_LATENT && !wide(s) &&
+             latent_attention_wide(w.spec.heads, w.spec.key_dim, w.spec.rotary_key_dim, w.spec.value_dim, w.spec.kv_rank))
+      attn_ws_bytes = std::max(attn_ws_bytes, latent_workspace_bytes(w.spec.heads, w.spec.rotary_key_dim, w.spec.kv_rank, kStackBlockTokens));
   const uint64_t off_attn_ws = c.take(attn_ws_bytes);
   const uint64_t off_want = c.take(kStackWantedRows * H * es), off_want_rows = c.take(kStackWantedRows * 4ull),
                  off_want_logits = c.take(kStackWantedRows * V * 4ull);

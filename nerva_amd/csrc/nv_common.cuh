@@ -170,6 +170,7 @@ enum TuningKnob : int {
   kTuneGemmBlockWaves,       // shared-X GEMM, gate/up pairs of up to 64 token rows: 4 = never three-wave workgroups
   kTuneGemmBlockRotate,      // shared-X GEMM: 1 + the K-blocks between the starts of consecutive row groups (1: a common start)
   kTuneMixedAttentionWide,   // mixed stacks: 2 = every attention layer through the general kernel
+  kTuneLatentAttentionWide,  // mixed stacks: 2 = every layer of attention over latents through the general kernel
   kTuneKnobs
 };
 int tuning(TuningKnob knob);

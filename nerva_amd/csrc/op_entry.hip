@@ -35,7 +35,7 @@ constexpr const char *kTuningNames[kTuneKnobs] = {"attn_splits",       "batch_sp
                                                   "gemv_x_registers",  "prefill_block_tokens", "gemv_rotated_walk",
                                                   "attn_merge_spin_limit", "attn_withhold_split", "block_layout",
                                                   "prefill_attention_rows", "prefill_walk", "gemm_block_off",
-                                                  "gemm_block_waves", "gemm_block_rotate", "mixed_attention_wide"};
+                                                  "gemm_block_waves", "gemm_block_rotate", "mixed_attention_wide", "latent_attention_wide"};
 }  // namespace
 
 int tuning(TuningKnob knob) { return g_tuning[knob].load(std::memory_order_relaxed); }
