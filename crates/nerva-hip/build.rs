@@ -16,7 +16,7 @@ const SUPPORTED_ARCH: &str = "gfx950";
 
 const SOURCES: &[&str] = &[
     "gemv_stream", "fp8_gemv", "attn_decode", "attn_prompt", "argmax", "synth_fill",
-    "sampler", "gemm_rows", "gemm_block", "gemm_any", "norm_join", "mingru", "attn_mixed", "attn_mixed_wide", "norm_rms", "attn_latent", "attn_latent_wide", "moe_rows", "op_entry", "decode_session", "layer_stack",
+    "sampler", "gemm_rows", "gemm_block", "gemm_any", "norm_join", "mingru", "attn_mixed", "attn_mixed_wide", "norm_rms", "attn_latent", "attn_latent_wide", "moe_rows", "gemv_layer", "op_entry", "decode_session", "layer_stack",
 ];
 
 fn main() {

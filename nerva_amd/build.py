@@ -16,7 +16,7 @@ LIB = os.path.join(HERE, "libnerva_hip.so")
 
 SOURCES = ["gemv_stream.hip", "fp8_gemv.hip", "attn_decode.hip", "attn_prompt.hip", "argmax.hip", "synth_fill.hip",
            "sampler.hip", "gemm_rows.hip", "gemm_block.hip", "gemm_any.hip", "norm_join.hip", "mingru.hip", "attn_mixed.hip",
-           "attn_mixed_wide.hip", "norm_rms.hip", "attn_latent.hip", "attn_latent_wide.hip", "moe_rows.hip", "op_entry.hip", "decode_session.hip", "layer_stack.hip"]
+           "attn_mixed_wide.hip", "norm_rms.hip", "attn_latent.hip", "attn_latent_wide.hip", "moe_rows.hip", "gemv_layer.hip", "op_entry.hip", "decode_session.hip", "layer_stack.hip"]
 
 FLAGS = ["--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function",
          # packed fp32 VALU ops are kept off for every device function of this library

@@ -86,6 +86,7 @@ struct GemvParams {
   uint32_t cols;
   uint32_t pair_gap;  // kEpiSwiglu: elements left unused between the last gate row and the first up row
   float eps;
+  float gain;      // kProRmsNorm, optional: factor on the normalised row (0: none)
   uint32_t round_out;
   const uint32_t *cursor;  // optional step guard: skip when *cursor >= max_steps
   uint32_t max_steps;
@@ -240,7 +241,7 @@ __global__ __launch_bounds__(kBlock) void gemv_kernel(GemvParams p) {
       for (uint32_t c = threadIdx.x; c < cols; c += kBlock) ss += p.xf[c] * p.xf[c];
     }
     ss = block_sum(ss, red);
-    const float scale = 1.0f / sqrtf(ss / static_cast<float>(cols) + p.eps);
+    const float scale = (p.gain != 0.0f ? p.gain : 1.0f) / sqrtf(ss / static_cast<float>(cols) + p.eps);
     if constexpr (MODE != kScalar) {
       for (uint32_t c = threadIdx.x * 8; c < cols; c += kBlock * 8) {
         const float4 a = *reinterpret_cast<const float4 *>(p.xf + c);   // second touch: L1/L2 hit
@@ -594,7 +595,7 @@ __global__ __launch_bounds__(WG *kWave, XREG ? 4 : PRO == kProJoin && WG == 8 ? 
       }
     }
     ss = block_sum_n<WG>(ss, red);
-    const float scale = 1.0f / sqrtf(ss / static_cast<float>(cols) + p.eps);
+    const float scale = (p.gain != 0.0f ? p.gain : 1.0f) / sqrtf(ss / static_cast<float>(cols) + p.eps);
     auto emit = [&](uint32_t c, const float4 &a, const float4 &b, const uint4 &g) {
       float g0, g1, g2, g3, g4, g5, g6, g7;
       unpack2<DT>(g.x, g0, g1);

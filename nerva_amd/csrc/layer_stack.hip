@@ -9,6 +9,7 @@
 #include "attn_latent.cuh"
 #include "attn_mixed.cuh"
 #include "gemm_any.cuh"
+#include "gemv_layer.cuh"
 #include "mingru.cuh"
 #include "moe_rows.cuh"
 #include "norm_join.cuh"
@@ -61,6 +62,18 @@ bool sandwich_step(const Session *s) {
   if (wide(s) || parallel(s)) return false;
   for (const StackLayer &w : s->stack->layers)
     if (w.spec.mixer == NERVA_HIP_MIXER_LATENT) return false;
+  return true;
+}
+
+// Whether it is parallel_step_16's.
+bool parallel_step(const Session *s) {
+  if (wide(s) || !parallel(s) || s->stack->logit_scale == 0.0f) return false;
+  for (const StackLayer &w : s->stack->layers) {
+    const NervaHipStackLayer &d = w.spec;
+    if (d.mixer != NERVA_HIP_MIXER_LATENT || d.ff != 0 ||
+        !layer_gemv_takes(s->hidden, d.q_rank, w.out_cols, d.experts, d.experts_per_token, d.expert_ff, d.shared_ff))
+      return false;
+  }
   return true;
 }
 
@@ -195,13 +208,20 @@ bool takes_latent_wide(const Session *s, const NervaHipStackLayer &d) {
 hipError_t decode_head(Session *s, DecodeRow &row) {
   const StackModel &m = *s->stack;
   GemvParams p = decode_gemv(s, s->lm_head, s->vocab, s->hidden);
-  p.join = decode_seam(s, row, m.final_w, m.final_b);
+  if (parallel(s)) {
+    p.xf = row.x;
+    p.gamma = m.final_w;
+    p.eps = s->eps;
+    p.gain = m.logit_scale;
+  } else {
+    p.join = decode_seam(s, row, m.final_w, m.final_b);
+  }
   p.out_f32 = s->logits;
   sample_bind_workspace(p.sample, s->sample_ws);
   p.sample.slots = s->slots;
   p.sample.cursor_rw = s->state;
   uint32_t candidates = 0;
-  hipError_t err = launch_gemv(s->dtype, kProJoin, kEpiArgmax, p, s->stream, nullptr, &candidates);
+  hipError_t err = launch_gemv(s->dtype, parallel(s) ? kProRmsNorm : kProJoin, kEpiArgmax, p, s->stream, nullptr, &candidates);
   if (err != hipSuccess) return err;
   if (s->sampler.mode == kSamplerGreedy) return launch_sample_finish(p.sample, candidates, s->state, s->max_ctx, s->stream);
   SamplerParams sp{};
@@ -271,6 +291,91 @@ hipError_t decode_step_16(Session *s) {
       row.due = Seam{w.norm[6], w.norm[7]};
     }
   }
+  return err == hipSuccess ? decode_head(s, row) : err;
+}
+
+// Parallel layers of attention over latents and routed experts.
+hipError_t parallel_step_16(Session *s) {
+  const StackModel &m = *s->stack;
+  hipStream_t st = s->stream;
+  hipError_t err = embed_rows(s, true, 0, 1, s->x);
+  uint64_t launches = 1;
+  for (size_t l = 0; err == hipSuccess && l < m.layers.size(); ++l) {
+    const StackLayer &w = m.layers[l];
+    const NervaHipStackLayer &d = w.spec;
+    const MoePlan plan = moe_plan_at(s->pplan, 1, d.experts_per_token, d.experts);
+    LayerFront f{};
+    f.x = s->x;
+    f.mixer_norm = w.norm[0];
+    f.ff_norm = d.experts != 0 ? w.norm[1] : nullptr;
+    f.eps = s->eps;
+    f.hidden = s->hidden;
+    f.w_in = w.w_in;
+    f.in_rows = w.gate_col + w.out_cols;
+    f.in = s->qkv;
+    f.router = w.router;
+    f.experts = d.experts;
+    f.logits = s->prouter;
+    f.shared_in = w.shared_in;
+    f.shared_ff = d.shared_ff;
+    f.shared_limit = d.shared_limit;
+    f.shared_act = s->ff16;
+    f.h16 = static_cast<uint16_t *>(s->pxn2);
+    f.cursor = s->state;
+    f.max_steps = s->max_ctx;
+    err = launch_layer_front(s->dtype, f, st);
+    LayerMiddle g{};
+    g.latent = s->qkv + w.q_col;
+    g.latent_norm = w.q_norm;
+    g.eps = s->eps;
+    g.w_uq = w.w_uq;
+    g.q_rank = d.q_rank;
+    g.q_rows = w.q_rows();
+    g.q = s->pq;
+    g.h16 = f.h16;
+    g.logits = s->prouter;
+    g.hidden = s->hidden;
+    g.experts = d.experts;
+    g.top = d.experts_per_token;
+    g.e_in = w.e_in;
+    g.ff = d.expert_ff;
+    g.limit = d.expert_limit;
+    g.act = static_cast<uint16_t *>(s->pff);
+    g.ids = plan.ids;
+    g.weights = plan.weights;
+    g.cursor = s->state;
+    g.max_steps = s->max_ctx;
+    if (err == hipSuccess) err = launch_layer_middle(s->dtype, g, st);
+    LatentAttnParams a = latent_params(s, w, s->qkv, s->pq, s->prope);
+    a.cursor = s->state;
+    a.tokens = 1;
+    a.out16 = s->attn16;
+    const bool fast = takes_latent_wide(s, d);
+    if (!fast) a.q_latent16 = static_cast<uint16_t *>(s->pql);   // (the middle launch has its own)
+    if (err == hipSuccess && !fast) err = launch_latent_prepare(s->dtype, a, st);
+    if (err == hipSuccess) err = fast ? launch_latent_attention_wide(s->dtype, a, st) : launch_latent_attention(s->dtype, a, st);
+    LayerBack b{};
+    b.x = s->x;
+    b.hidden = s->hidden;
+    b.w_o = w.w_out;
+    b.mixed = s->attn16;
+    b.mix_cols = w.out_cols;
+    b.e_out = w.e_out;
+    b.act = g.act;
+    b.ids = plan.ids;
+    b.weights = plan.weights;
+    b.ff = d.expert_ff;
+    b.top = d.experts != 0 ? d.experts_per_token : 0u;
+    b.shared_out = w.shared_out;
+    b.shared_act = s->ff16;
+    b.shared_ff = d.shared_ff;
+    b.cursor = s->state;
+    b.max_steps = s->max_ctx;
+    if (err == hipSuccess) err = launch_layer_back(s->dtype, b, st);
+    launches += 3 + (fast ? latent_wide_launches(true) : 2u);
+  }
+  s->stack_launches = launches + (s->sampler.mode == kSamplerGreedy ? 2 : 3);
+  DecodeRow row{s->x, nullptr, Seam{}};
   return err == hipSuccess ? decode_head(s, row) : err;
 }
 
@@ -611,6 +716,7 @@ hipError_t sample_logits(Session *s) {
 
 hipError_t nv::stack_enqueue_step(Session *s) {
   if (sandwich_step(s)) return decode_step_16(s);
+  if (parallel_step(s)) return parallel_step_16(s);
   Block b{s, 1, 0, true, Seam{}, 0};
   hipError_t err = b.layers(nullptr, 0);
   if (err == hipSuccess) err = b.logits_of(nullptr, 1, s->logits);
@@ -663,6 +769,11 @@ hipError_t nv::stack_prompt(Session *s, uint32_t begin, uint32_t end, const uint
         err = hipMemcpyAsync(s->x, s->px + last * H, H * sizeof(float), hipMemcpyDeviceToDevice, s->stream);
         if (err == hipSuccess) err = hipMemcpyAsync(s->y, s->py + last * H, H * sizeof(float), hipMemcpyDeviceToDevice, s->stream);
         DecodeRow row{s->x, s->r, b.due};
+        if (err == hipSuccess) err = decode_head(s, row);
+      } else if (err == hipSuccess && parallel_step(s)) {
+        err = b.settle();
+        if (err == hipSuccess) err = hipMemcpyAsync(s->x, s->px + last * H, H * sizeof(float), hipMemcpyDeviceToDevice, s->stream);
+        DecodeRow row{s->x, nullptr, Seam{}};
         if (err == hipSuccess) err = decode_head(s, row);
       } else if (err == hipSuccess) {
         s->host_state[kStackWantedRows] = static_cast<uint32_t>(last);
