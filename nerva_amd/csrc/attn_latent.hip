@@ -1,6 +1,8 @@
 // Attention over normalised latents, for any shape (see attn_latent.cuh).
 #include "attn_latent.cuh"
 
+#include <algorithm>
+
 #include "activations.cuh"
 #include "attn_mixed.cuh"
 #include "gemm_rows.cuh"
@@ -38,7 +40,7 @@ __global__ __launch_bounds__(kBlock) void latent_prepare_kernel(LatentAttnParams
   for (uint32_t i = threadIdx.x; i < p.q_rank; i += kBlock) {
     const float v = src[p.q_col + i] * qs * dec16<DT>(p.q_norm[i]);
     if (p.q_latent32 != nullptr) p.q_latent32[static_cast<uint64_t>(t) * p.q_rank + i] = v;
-    else p.q_latent16[p.q_latent_tiles != 0 ? gemm_x_packed_index(p.q_latent_tiles, t, i) : static_cast<uint64_t>(t) * p.q_rank + i] = enc16<DT>(v);
+    else p.q_latent16[p.q_latent_tiles != 0 ? gemm_x_block_index(p.q_latent_tiles, t, i, p.q_rank) : static_cast<uint64_t>(t) * p.q_rank + i] = enc16<DT>(v);
   }
   const uint32_t width = p.kv_rank + p.rot_dim, row = pos % kKvBlockTokens;
   const uint64_t block = static_cast<uint64_t>(p.table[pos / kKvBlockTokens]) * kKvBlockTokens * width;
@@ -141,7 +143,7 @@ __global__ __launch_bounds__(kBlock) void latent_attention_kernel(LatentAttnPara
     for (uint32_t d = 0; d < R; ++d) o = fmaf(dec16<DT>(uv[d]), q_s[d], o);
     o *= sigmoid(src[p.gate_col + e]);
     if (p.out16 == nullptr) p.out32[t * out_width + e] = o;
-    else if (p.packed_tiles != 0) p.out16[gemm_x_packed_index(p.packed_tiles, t, e)] = enc16<DT>(o);
+    else if (p.packed_tiles != 0) p.out16[gemm_x_block_index(p.packed_tiles, t, e, p.heads * p.value_dim)] = enc16<DT>(o);
     else p.out16[t * out_width + e] = enc16<DT>(o);
   }
 }
@@ -157,7 +159,7 @@ bool shape_ok(const LatentAttnParams &p) {
 
 hipError_t launch_latent_prepare(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream) {
   if (!shape_ok(p) || dtype != kBF16 || (p.q_latent16 == nullptr) == (p.q_latent32 == nullptr) ||
-      (p.q_latent_tiles != 0 && (p.q_latent16 == nullptr || p.q_latent_tiles * 16u < p.tokens || p.q_rank % 32 != 0)))
+      (p.q_latent_tiles != 0 && (p.q_latent16 == nullptr || p.q_latent_tiles * 16u < std::min(p.tokens, kGemmDeepMaxTokens) || p.q_rank % 32 != 0)))
     return hipErrorInvalidValue;
   if (p.cache32) hipLaunchKernelGGL((latent_prepare_kernel<kBF16, true>), dim3(p.tokens), dim3(kBlock), 0, stream, p);
   else hipLaunchKernelGGL((latent_prepare_kernel<kBF16, false>), dim3(p.tokens), dim3(kBlock), 0, stream, p);
@@ -167,7 +169,7 @@ hipError_t launch_latent_prepare(uint32_t dtype, const LatentAttnParams &p, hipS
 hipError_t launch_latent_attention(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream) {
   if (!shape_ok(p) || dtype != kBF16 || p.q == nullptr || p.w_uk == nullptr || p.w_uv == nullptr || (p.out16 == nullptr) == (p.out32 == nullptr))
     return hipErrorInvalidValue;
-  if (p.packed_tiles != 0 && (p.out16 == nullptr || p.packed_tiles * 16u < p.tokens || p.heads * p.value_dim % 32 != 0))
+  if (p.packed_tiles != 0 && (p.out16 == nullptr || p.packed_tiles * 16u < std::min(p.tokens, kGemmDeepMaxTokens) || p.heads * p.value_dim % 32 != 0))
     return hipErrorInvalidValue;
   const size_t lds = static_cast<size_t>(p.kv_rank + p.rot_dim) * sizeof(float);
   const dim3 grid(p.tokens, p.heads);

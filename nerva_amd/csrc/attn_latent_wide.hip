@@ -33,7 +33,7 @@ using namespace attn;
 constexpr uint32_t kUnitKeys = 2 * kKvBlockTokens;   // keys a step of the rows kernel takes
 constexpr uint32_t kPairRows = 32;
 constexpr size_t kPairExchange = 4096 + 512;
-constexpr uint32_t kMostSplits = 128, kBlockSplits = 8, kWorkgroups = 256;
+constexpr uint32_t kMostSplits = 128, kBlockSplits = 8, kWorkgroups = 512;   // (two a CU)
 constexpr float kLazy = 8.0f;
 
 struct Work {
@@ -381,7 +381,7 @@ __global__ __launch_bounds__(kBlock) void latent_merge_kernel(LatentAttnParams p
 
 __device__ __forceinline__ void gated_store(const LatentAttnParams &p, uint32_t t, uint32_t e, const f32x4_t &o) {
   const float *g = p.proj + static_cast<uint64_t>(t) * p.proj_stride + p.gate_col + e;
-  uint16_t *out = p.out16 + (p.packed_tiles != 0 ? gemm_x_packed_index(p.packed_tiles, t, e) : static_cast<uint64_t>(t) * p.heads * p.value_dim + e);
+  uint16_t *out = p.out16 + (p.packed_tiles != 0 ? gemm_x_block_index(p.packed_tiles, t, e, p.heads * p.value_dim) : static_cast<uint64_t>(t) * p.heads * p.value_dim + e);
   // (four columns stay together in operand order)
   *reinterpret_cast<uint2 *>(out) = make_uint2(pack16(o[0] * sigmoid(g[0]), o[1] * sigmoid(g[1])), pack16(o[2] * sigmoid(g[2]), o[3] * sigmoid(g[3])));
 }
@@ -566,7 +566,7 @@ hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &
   if (dtype != kBF16 || !latent_attention_wide(p.heads, p.key_dim, p.rot_dim, p.value_dim, p.kv_rank) || p.cache32 != 0 || p.out16 == nullptr ||
       p.workspace == nullptr || p.proj == nullptr || p.q == nullptr || p.w_uk == nullptr || p.w_uv == nullptr || p.cache == nullptr ||
       p.table == nullptr || p.kv_norm == nullptr || p.tokens == 0 || p.rot_dims % 2 != 0 || p.rot_dims > p.rot_dim ||
-      (p.rot_dims != 0 && p.rope_cs == nullptr) || (p.packed_tiles != 0 && (p.packed_tiles * 16u < p.tokens || p.heads * p.value_dim % 32 != 0)))
+      (p.rot_dims != 0 && p.rope_cs == nullptr) || (p.packed_tiles != 0 && (p.packed_tiles * 16u < std::min(p.tokens, kGemmDeepMaxTokens) || p.heads * p.value_dim % 32 != 0)))
     return hipErrorInvalidValue;
   if (!aligned(p.workspace, 256) || !aligned(p.cache, 16) || !aligned(p.w_uk, 16) || !aligned(p.w_uv, 16) || !aligned(p.q, 16) || !aligned(p.out16, 16))
     return hipErrorInvalidValue;

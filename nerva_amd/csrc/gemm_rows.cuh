@@ -33,6 +33,11 @@ constexpr uint32_t kGemmDeepMaxTokens = 512;   // ... where gemm_deep_slices tak
 __host__ __device__ __forceinline__ uint64_t gemm_x_packed_index(uint32_t tiles, uint32_t t, uint32_t k) {
   return (static_cast<uint64_t>(k / 32u) * tiles + t / 16u) * 512u + (((k % 32u) / 8u) * 16u + t % 16u) * 8u + k % 8u;
 }
+// The same for rows past kGemmDeepMaxTokens: pieces of that many token rows, one after the other, each in operand order.
+__host__ __device__ __forceinline__ uint64_t gemm_x_block_index(uint32_t tiles, uint32_t t, uint32_t k, uint32_t cols) {
+  constexpr uint32_t kPiece = 512;
+  return static_cast<uint64_t>(t / kPiece) * kPiece * cols + gemm_x_packed_index(tiles, t % kPiece, k);
+}
 // Token tiles the GEMM works with for a block of `tokens` rows (its X buffer in operand order has as many).
 __host__ __device__ __forceinline__ uint32_t gemm_packed_tiles(uint32_t tokens) {
   return tokens > 256u ? 32u : tokens > 128u ? 16u : tokens > 64u ? 8u : tokens > 32u ? 4u : 2u;

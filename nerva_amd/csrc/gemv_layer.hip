@@ -66,69 +66,78 @@ struct Unit {
 
 constexpr int kBatch = 4;   // chunks of a request batch: 4 KiB of each row
 
-// Walks this wave's units. unit_at(i) -> Unit for i < units (i is wave-uniform).
+// A wave's walk over its units first, first + stride, .. < units; unit_at(i) -> Unit (i is wave-uniform). The first two
+// batches of weights are requested by start(), which does not need the staged inputs.
 template <uint32_t DT, typename At>
-__device__ __forceinline__ void walk_pairs(const uint16_t *xs, uint32_t units, uint32_t first, uint32_t stride, At unit_at) {
-  const uint32_t lane = threadIdx.x & (kWave - 1);
+struct PairWalk {
+  At unit_at;
+  uint32_t units, stride, lane;
   uint4 b0[2][kBatch], b1[2][kBatch];
-  uint32_t iu = first, ic = 0;      // next batch to request: unit, first column
-  Unit in{};
-  if (iu < units) in = unit_at(iu);
-  uint32_t cu = first, cc = 0;      // next batch to multiply
-  Unit cur = in;
-  float acc0 = 0.0f, acc1 = 0.0f;
-#define NV_LAYER_ISSUE(DST)                                                                          \
-  if (iu < units) {                                                                                 \
-    _Pragma("unroll") for (int u = 0; u < kBatch; ++u) {                                            \
-      const uint32_t c = ic + u * kChunk + lane * 8u;                                               \
-      const bool on = c < in.cols;                                                                  \
-      DST[0][u] = on ? load_stream(in.w0 + c) : make_uint4(0u, 0u, 0u, 0u);                         \
-      DST[1][u] = on ? load_stream(in.w1 + c) : make_uint4(0u, 0u, 0u, 0u);                         \
-    }                                                                                               \
-    ic += kBatch * kChunk;                                                                          \
-    if (ic >= in.cols) {                                                                            \
-      ic = 0;                                                                                       \
-      iu += stride;                                                                                 \
-      if (iu < units) in = unit_at(iu);                                                             \
-    }                                                                                               \
+  uint32_t iu, ic;      // next batch to request: unit, first column
+  Unit in;
+  uint32_t cu, cc;      // next batch to multiply
+  Unit cur;
+  float acc0, acc1;
+
+  __device__ __forceinline__ PairWalk(At at, uint32_t n, uint32_t first, uint32_t step)
+      : unit_at(at), units(n), stride(step), lane(threadIdx.x & (kWave - 1)), iu(first), ic(0), in{}, cu(first), cc(0), cur{}, acc0(0.0f), acc1(0.0f) {}
+  __device__ __forceinline__ void issue(uint4 (&to)[2][kBatch]) {
+    if (iu >= units) return;
+#pragma unroll
+    for (int u = 0; u < kBatch; ++u) {
+      const uint32_t c = ic + u * kChunk + lane * 8u;
+      const bool on = c < in.cols;
+      to[0][u] = on ? load_stream(in.w0 + c) : make_uint4(0u, 0u, 0u, 0u);
+      to[1][u] = on ? load_stream(in.w1 + c) : make_uint4(0u, 0u, 0u, 0u);
+    }
+    ic += kBatch * kChunk;
+    if (ic >= in.cols) {
+      ic = 0;
+      iu += stride;
+      if (iu < units) in = unit_at(iu);
+    }
   }
-#define NV_LAYER_CONSUME(SRC)                                                                        \
-  _Pragma("unroll") for (int u = 0; u < kBatch; ++u) {                                              \
-    if (cc + u * kChunk < cur.cols) {                                                               \
-      const uint4 x = *reinterpret_cast<const uint4 *>(xs + cur.at + cc + u * kChunk + lane * 8u);       \
-      acc0 = dot8<DT, true>(SRC[0][u], x, acc0);                                                    \
-      acc1 = dot8<DT, true>(SRC[1][u], x, acc1);                                                    \
-    }                                                                                               \
-  }                                                                                                 \
-  cc += kBatch * kChunk;                                                                            \
-  if (cc >= cur.cols) {                                                                             \
-    acc0 = wave_sum(acc0);                                                                          \
-    acc1 = wave_sum(acc1);                                                                          \
-    if (lane == 0) {                                                                                \
-      if (cur.act != nullptr) {                                                                     \
-        *cur.act = enc16<DT>(clamped_glu(acc0, acc1, cur.limit));                                   \
-      } else {                                                                                      \
-        *cur.out0 = acc0;                                                                           \
-        if (cur.out1 != nullptr) *cur.out1 = acc1;                                                  \
-      }                                                                                             \
-    }                                                                                               \
-    acc0 = acc1 = 0.0f;                                                                             \
-    cc = 0;                                                                                         \
-    cu += stride;                                                                                   \
-    if (cu < units) cur = unit_at(cu);                                                              \
+  __device__ __forceinline__ void consume(const uint4 (&from)[2][kBatch], const uint16_t *xs) {
+#pragma unroll
+    for (int u = 0; u < kBatch; ++u) {
+      if (cc + u * kChunk < cur.cols) {
+        const uint4 x = *reinterpret_cast<const uint4 *>(xs + cur.at + cc + u * kChunk + lane * 8u);
+        acc0 = dot8<DT, true>(from[0][u], x, acc0);
+        acc1 = dot8<DT, true>(from[1][u], x, acc1);
+      }
+    }
+    cc += kBatch * kChunk;
+    if (cc < cur.cols) return;
+    acc0 = wave_sum(acc0);
+    acc1 = wave_sum(acc1);
+    if (lane == 0) {
+      if (cur.act != nullptr) {
+        *cur.act = enc16<DT>(clamped_glu(acc0, acc1, cur.limit));
+      } else {
+        *cur.out0 = acc0;
+        if (cur.out1 != nullptr) *cur.out1 = acc1;
+      }
+    }
+    acc0 = acc1 = 0.0f;
+    cc = 0;
+    cu += stride;
+    if (cu < units) cur = unit_at(cu);
   }
-  NV_LAYER_ISSUE(b0)
-  NV_LAYER_ISSUE(b1)
-  while (cu < units) {
-    NV_LAYER_CONSUME(b0)
-    NV_LAYER_ISSUE(b0)
-    if (cu >= units) break;
-    NV_LAYER_CONSUME(b1)
-    NV_LAYER_ISSUE(b1)
+  __device__ __forceinline__ void start() {
+    if (iu < units) in = cur = unit_at(iu);
+    issue(b0);
+    issue(b1);
   }
-#undef NV_LAYER_ISSUE
-#undef NV_LAYER_CONSUME
-}
+  __device__ __forceinline__ void run(const uint16_t *xs) {
+    while (cu < units) {
+      consume(b0, xs);
+      issue(b0);
+      if (cu >= units) break;
+      consume(b1, xs);
+      issue(b1);
+    }
+  }
+};
 
 __device__ __forceinline__ Unit two_rows(const uint16_t *w, uint32_t cols, uint32_t rows, uint32_t i, uint32_t at, float *out) {
   const uint32_t r0 = 2u * i, r1 = min(r0 + 1u, rows - 1u);
@@ -143,21 +152,24 @@ template <uint32_t DT>
 __global__ __launch_bounds__(kThreads, 4) void layer_front_kernel(LayerFront p) {
   extern __shared__ __align__(16) uint16_t xs[];   // the mixer's row, the feed-forward's
   __shared__ float red[kWaves];
-  if (*p.cursor >= p.max_steps) return;
+  const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
+  const uint32_t n_in = (p.in_rows + 1) / 2, n_router = (p.experts + 1) / 2, units = n_in + n_router + p.shared_ff;
+  const auto unit_at = [&](uint32_t i) {
+    if (i < n_router) return two_rows(p.router, p.hidden, p.experts, i, padded(p.hidden), p.logits);
+    i -= n_router;
+    if (i < n_in) return two_rows(p.w_in, p.hidden, p.in_rows, i, 0u, p.in);
+    return gate_and_up(p.shared_in, p.hidden, p.shared_ff, i - n_in, padded(p.hidden), p.shared_act, p.shared_limit);
+  };
+  // (consecutive units go to different workgroups)
+  PairWalk<DT, decltype(unit_at)> walk(unit_at, units, wave * gridDim.x + blockIdx.x, gridDim.x * kWaves);
+  walk.start();
+  if (*p.cursor >= p.max_steps) return;   // (after the requests, which do not depend on it)
   uint16_t *xs2 = xs + padded(p.hidden);
   rms_stage<DT>(p.x, p.hidden, p.eps, p.mixer_norm, xs, p.ff_norm, xs2, red);
   __syncthreads();
   if (p.ff_norm != nullptr && blockIdx.x == 0)
     for (uint32_t c = threadIdx.x * 8u; c < p.hidden; c += kThreads * 8u) *reinterpret_cast<uint4 *>(p.h16 + c) = *reinterpret_cast<const uint4 *>(xs2 + c);
-  const uint32_t wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
-  const uint32_t n_in = (p.in_rows + 1) / 2, n_router = (p.experts + 1) / 2, units = n_in + n_router + p.shared_ff;
-  // (consecutive units go to different workgroups)
-  walk_pairs<DT>(xs, units, wave * gridDim.x + blockIdx.x, gridDim.x * kWaves, [&](uint32_t i) {
-    if (i < n_router) return two_rows(p.router, p.hidden, p.experts, i, padded(p.hidden), p.logits);
-    i -= n_router;
-    if (i < n_in) return two_rows(p.w_in, p.hidden, p.in_rows, i, 0u, p.in);
-    return gate_and_up(p.shared_in, p.hidden, p.shared_ff, i - n_in, padded(p.hidden), p.shared_act, p.shared_limit);
-  });
+  walk.run(xs);
 }
 
 template <uint32_t DT>
@@ -171,17 +183,16 @@ __global__ __launch_bounds__(kThreads, 4) void layer_middle_kernel(LayerMiddle p
   uint16_t *xs2 = xs + padded(p.q_rank);
   const uint32_t tid = threadIdx.x;
   for (uint32_t e = tid; e < p.experts; e += kThreads) score[e] = 1.0f / (1.0f + expf(-p.logits[e]));
-  if (p.experts != 0) {
-    for (uint32_t c = tid * 8u; c < p.hidden; c += kThreads * 8u) *reinterpret_cast<uint4 *>(xs2 + c) = *reinterpret_cast<const uint4 *>(p.h16 + c);
-    clear_tail(xs2, p.hidden);
-    if (tid < kMaxTop) id_s[tid] = 0u;   // (scores that are no numbers choose nothing: some expert that exists)
-    if (tid < kMaxTop) s_s[tid] = 0.0f;
+  if (tid < kMaxTop) {   // (scores that are no numbers choose nothing: some expert that exists)
+    id_s[tid] = 0u;
+    s_s[tid] = 0.0f;
   }
-  rms_stage<DT>(p.latent, p.q_rank, p.eps, p.latent_norm, xs, nullptr, nullptr, red);   // (its barriers publish the scores)
+  __syncthreads();
   // an expert's place is the number of experts ahead of it
   for (uint32_t e = tid; e < p.experts; e += kThreads) {
     const float s = score[e];
     uint32_t ahead = 0;
+#pragma unroll 8
     for (uint32_t j = 0; j < p.experts; ++j) ahead += score[j] > s || (score[j] == s && j < e) ? 1u : 0u;
     if (ahead < p.top) {
       id_s[ahead] = e;
@@ -189,20 +200,29 @@ __global__ __launch_bounds__(kThreads, 4) void layer_middle_kernel(LayerMiddle p
     }
   }
   __syncthreads();
-  if (p.experts != 0 && blockIdx.x == 0 && tid < p.top) {
-    float sum = 0.0f;
-    for (uint32_t k = 0; k < p.top; ++k) sum += s_s[k];
-    p.ids[tid] = id_s[tid];
-    p.weights[tid] = s_s[tid] / (sum + 1e-20f);
-  }
   const uint32_t wave = __builtin_amdgcn_readfirstlane(tid / kWave);
-  const uint32_t n_q = (p.q_rows + 1) / 2, units = n_q + (p.experts != 0 ? p.top * p.ff : 0u);
-  walk_pairs<DT>(xs, units, wave * gridDim.x + blockIdx.x, gridDim.x * kWaves, [&](uint32_t i) {
-    if (i < n_q) return two_rows(p.w_uq, p.q_rank, p.q_rows, i, 0u, p.q);
-    i -= n_q;
+  const uint32_t n_experts = p.experts != 0 ? p.top * p.ff : 0u, units = n_experts + (p.q_rows + 1) / 2;
+  const auto unit_at = [&](uint32_t i) {
+    if (i >= n_experts) return two_rows(p.w_uq, p.q_rank, p.q_rows, i - n_experts, 0u, p.q);
     const uint32_t k = i / p.ff, e = __builtin_amdgcn_readfirstlane(id_s[k]);
-    return gate_and_up(p.e_in + static_cast<uint64_t>(e) * 2u * p.ff * p.hidden, p.hidden, p.ff, i % p.ff, padded(p.q_rank), p.act + k * p.ff, p.limit);
-  });
+    return gate_and_up(p.e_in + static_cast<uint64_t>(e) * 2u * p.ff * p.hidden, p.hidden, p.ff, i - k * p.ff, padded(p.q_rank), p.act + k * p.ff,
+                       p.limit);
+  };
+  PairWalk<DT, decltype(unit_at)> walk(unit_at, units, wave * gridDim.x + blockIdx.x, gridDim.x * kWaves);
+  walk.start();
+  if (p.experts != 0) {
+    for (uint32_t c = tid * 8u; c < p.hidden; c += kThreads * 8u) *reinterpret_cast<uint4 *>(xs2 + c) = *reinterpret_cast<const uint4 *>(p.h16 + c);
+    clear_tail(xs2, p.hidden);
+    if (blockIdx.x == 0 && tid < p.top) {
+      float sum = 0.0f;
+      for (uint32_t k = 0; k < p.top; ++k) sum += s_s[k];
+      p.ids[tid] = id_s[tid];
+      p.weights[tid] = s_s[tid] / (sum + 1e-20f);
+    }
+  }
+  rms_stage<DT>(p.latent, p.q_rank, p.eps, p.latent_norm, xs, nullptr, nullptr, red);
+  __syncthreads();
+  walk.run(xs);
 }
 
 // ---- back ------------------------------------------------------------------------------------
@@ -220,27 +240,18 @@ template <uint32_t DT>
 __global__ __launch_bounds__(kThreads, 4) void layer_back_kernel(LayerBack p) {
   extern __shared__ __align__(16) uint16_t xs[];   // the runs' inputs, each padded to whole chunks
   __shared__ Run runs[kMaxRuns];
-  __shared__ uint32_t total_chunks;
   if (*p.cursor >= p.max_steps) return;
   const uint32_t tid = threadIdx.x, lane = tid & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(tid / kWave);
   const uint32_t n_runs = 1u + p.top + (p.shared_ff != 0 ? 1u : 0u);
-  const auto stage = [&](const uint16_t *src, uint32_t cols, uint32_t at) {
-    for (uint32_t c = tid * 8u; c < cols; c += kThreads * 8u) *reinterpret_cast<uint4 *>(xs + at + c) = *reinterpret_cast<const uint4 *>(src + c);
-    clear_tail(xs + at, cols);
-  };
   const uint32_t expert_at = padded(p.mix_cols), shared_at = expert_at + p.top * padded(p.ff);
-  stage(p.mixed, p.mix_cols, 0);
-  for (uint32_t k = 0; k < p.top; ++k) stage(p.act + k * p.ff, p.ff, expert_at + k * padded(p.ff));
-  if (p.shared_ff != 0) stage(p.shared_act, p.shared_ff, shared_at);
   if (tid < n_runs) {
     if (tid == 0) runs[tid] = Run{p.w_o, p.mix_cols, p.mix_cols, 0u, 1.0f};
     else if (tid <= p.top)
       runs[tid] = Run{p.e_out + static_cast<uint64_t>(p.ids[tid - 1]) * p.hidden * p.ff, p.ff, p.ff, expert_at + (tid - 1) * padded(p.ff), p.weights[tid - 1]};
     else runs[tid] = Run{p.shared_out, p.shared_ff, p.shared_ff, shared_at, 1.0f};
   }
-  if (tid == 0) total_chunks = (shared_at + padded(p.shared_ff)) / kChunk;
   __syncthreads();
-  const uint32_t chunks = __builtin_amdgcn_readfirstlane(total_chunks);
+  const uint32_t chunks = (shared_at + padded(p.shared_ff)) / kChunk;
   // The row's chunks lie one after the other as their inputs do. Cursors over them (wave-uniform): run, column in it.
   struct Cursor {
     const uint16_t *base;
@@ -306,6 +317,14 @@ __global__ __launch_bounds__(kThreads, 4) void layer_back_kernel(LayerBack p) {
   }
   NV_BACK_ISSUE(b0)
   NV_BACK_ISSUE(b1)
+  const auto stage = [&](const uint16_t *src, uint32_t cols, uint32_t at) {
+    for (uint32_t c = tid * 8u; c < cols; c += kThreads * 8u) *reinterpret_cast<uint4 *>(xs + at + c) = *reinterpret_cast<const uint4 *>(src + c);
+    clear_tail(xs + at, cols);
+  };
+  stage(p.mixed, p.mix_cols, 0);
+  for (uint32_t k = 0; k < p.top; ++k) stage(p.act + k * p.ff, p.ff, expert_at + k * padded(p.ff));
+  if (p.shared_ff != 0) stage(p.shared_act, p.shared_ff, shared_at);
+  __syncthreads();
   while (crow < p.hidden) {
     NV_BACK_CONSUME(b0)
     NV_BACK_ISSUE(b0)

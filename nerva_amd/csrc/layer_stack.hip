@@ -303,7 +303,7 @@ hipError_t parallel_step_16(Session *s) {
   for (size_t l = 0; err == hipSuccess && l < m.layers.size(); ++l) {
     const StackLayer &w = m.layers[l];
     const NervaHipStackLayer &d = w.spec;
-    const MoePlan plan = moe_plan_at(s->pplan, 1, d.experts_per_token, d.experts);
+    const MoePlan plan = moe_plan_at(s->pplan, 1, d.experts_per_token, d.experts, true);
     LayerFront f{};
     f.x = s->x;
     f.mixer_norm = w.norm[0];
@@ -384,6 +384,7 @@ hipError_t parallel_step_16(Session *s) {
 // Token tiles of the matrix-operand order a projection's input takes, 0 where its shape goes through gemm_any.
 uint32_t operand_tiles(const Session *s, int epilogue, uint32_t rows, uint32_t cols, uint32_t tokens) {
   if (wide(s) || cols % 32 != 0) return 0;
+  tokens = std::min(tokens, kGemmDeepMaxTokens);   // (larger blocks go in pieces)
   const bool taken = tokens <= kGemmMaxTokens       ? gemm_rows_supported(rows, cols, tokens)
                      : tokens <= kGemmWideMaxTokens ? gemm_wide_slices(epilogue, rows, cols, tokens, s->pgemm_ws_bytes) != 0
                                                     : gemm_deep_slices(epilogue, rows, cols, tokens, s->pgemm_ws_bytes) != 0;
@@ -426,6 +427,20 @@ struct Block {
                      uint32_t out_tiles, const uint16_t *act) {
     launches += 1;
     const bool narrow = epilogue == kGemmXielu && !wide(s);
+    if (tiles != 0 && tokens > kGemmDeepMaxTokens) {
+      // pieces of kGemmDeepMaxTokens rows; the last one has the others' layout, so enough rows for that are multiplied
+      hipError_t err = hipSuccess;
+      const uint32_t all = tokens;
+      for (uint32_t at = 0; err == hipSuccess && at < all; at += kGemmDeepMaxTokens) {
+        tokens = std::min(kGemmDeepMaxTokens, std::max(all - at, kGemmWideMaxTokens + 1));
+        const uint64_t done = static_cast<uint64_t>(at) * rows;
+        err = project(epilogue, w, rows, cols, static_cast<const uint16_t *>(x) + static_cast<uint64_t>(at) * cols, tiles,
+                      narrow ? static_cast<void *>(static_cast<uint16_t *>(out) + done) : static_cast<void *>(static_cast<float *>(out) + done),
+                      out_tiles, act);
+      }
+      tokens = all;
+      return err;
+    }
     if (tiles != 0) {
       GemmRowsParams g{};
       g.w = w;
@@ -568,7 +583,7 @@ struct Block {
     r.tokens = tokens;
     r.experts = d.experts;
     r.top = d.experts_per_token;
-    r.plan = moe_plan_at(s->pplan, tokens, r.top, r.experts);
+    r.plan = moe_plan_at(s->pplan, tokens, r.top, r.experts, wide(s));
     ExpertRows e{};
     if (wide(s)) {
       e.x32 = static_cast<const float *>(h);
@@ -740,8 +755,9 @@ hipError_t nv::stack_prompt(Session *s, uint32_t begin, uint32_t end, const uint
   hipError_t err = hipSuccess;
   uint32_t next_wanted = 0;
   const uint64_t H = s->hidden;
-  for (uint32_t first = begin; err == hipSuccess && first < end; first += kStackBlockTokens) {
-    Block b{s, std::min(kStackBlockTokens, end - first), first, false, Seam{}, 0};
+  const uint32_t most = s->stack->block_tokens;
+  for (uint32_t first = begin; err == hipSuccess && first < end; first += most) {
+    Block b{s, std::min(most, end - first), first, false, Seam{}, 0};
     err = b.layers(residuals != nullptr ? residuals + static_cast<uint64_t>(first - begin) * H : nullptr,
                    static_cast<uint64_t>(end - begin) * H);
     while (err == hipSuccess && next_wanted < wanted_count && wanted[next_wanted] < first + b.tokens - begin) {
@@ -974,17 +990,22 @@ int create_stack(const NervaHipStackSessionCreateRequest *rq, bool synthetic, ui
     if (d.experts != 0) {
       m.max_experts = std::max(m.max_experts, d.experts);
       m.max_top = std::max(m.max_top, d.experts_per_token);
-      m.plan_bytes = std::max(m.plan_bytes, moe_plan_bytes(kStackBlockTokens, d.experts_per_token, d.experts));
     }
   }
   s->intermediate = m.max_ff;
+  bool experts = !sandwich;
+  for (const StackLayer &w : m.layers) experts = experts && w.spec.mixer == NERVA_HIP_MIXER_LATENT && w.spec.ff == 0;
+  if (experts) m.block_tokens = kExpertBlockTokens;
+  for (const StackLayer &w : m.layers)
+    if (w.spec.experts != 0)
+      m.plan_bytes = std::max(m.plan_bytes, moe_plan_bytes(m.block_tokens, w.spec.experts_per_token, w.spec.experts));
   for (uint32_t l = 0; l < L; ++l) {
     StackLayer &w = m.layers[l];
     if (!w.own_cache()) continue;
     // A block of token rows writes all its keys before its first query looks back: the oldest key that query may see
-    // and the newest key written lie less than view + kStackBlockTokens positions apart, one block more for the edges.
+    // and the newest key written lie less than view + block_tokens positions apart, one block more for the edges.
     const uint32_t view = widest_view(m.layers, l);
-    const uint64_t reach = (static_cast<uint64_t>(view) + kStackBlockTokens + kKvBlockTokens - 1) / kKvBlockTokens + 1;
+    const uint64_t reach = (static_cast<uint64_t>(view) + m.block_tokens + kKvBlockTokens - 1) / kKvBlockTokens + 1;
     w.ring_blocks = view == 0 || reach > m.logical_blocks ? m.logical_blocks : static_cast<uint32_t>(reach);
     const auto area = [&](uint32_t dim) {
       const uint64_t at = m.cache_bytes;
@@ -1188,7 +1209,7 @@ int create_stack(const NervaHipStackSessionCreateRequest *rq, bool synthetic, ui
   }
   out->failure_stage = 0;
   fill_create_result(s, out);
-  out->prefill_chunk_tokens = kStackBlockTokens;
+  out->prefill_chunk_tokens = m.block_tokens;
   out->h2d_bytes = h2d;
   out->sync_calls = syncs;
   out->status = 0;
@@ -1200,7 +1221,7 @@ int create_stack(const NervaHipStackSessionCreateRequest *rq, bool synthetic, ui
 
 hipError_t nv::stack_setup_state(Session *s, int32_t *failure_stage, bool with_weights) {
   const StackModel &m = *s->stack;
-  const uint64_t H = s->hidden, V = s->vocab, T = kStackBlockTokens, es = wide(s) ? 4 : 2;
+  const uint64_t H = s->hidden, V = s->vocab, T = m.block_tokens, es = wide(s) ? 4 : 2;
   s->block_count = m.logical_blocks;
   s->kv_bytes = m.cache_bytes;
   s->stack_state_bytes = m.state_floats * sizeof(float);
@@ -1222,10 +1243,10 @@ hipError_t nv::stack_setup_state(Session *s, int32_t *failure_stage, bool with_w
   for (const StackLayer &w : m.layers)
     if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION && !wide(s) &&
         mixed_attention_wide(w.spec.heads, w.spec.kv_heads, w.spec.key_dim, w.spec.value_dim))
-      attn_ws_bytes = std::max(attn_ws_bytes, mixed_attention_workspace_bytes(w.spec.heads, kStackBlockTokens));
+      attn_ws_bytes = std::max(attn_ws_bytes, mixed_attention_workspace_bytes(w.spec.heads, m.block_tokens));
     else if (w.spec.mixer == NERVA_HIP_MIXER_LATENT && !wide(s) &&
              latent_attention_wide(w.spec.heads, w.spec.key_dim, w.spec.rotary_key_dim, w.spec.value_dim, w.spec.kv_rank))
-      attn_ws_bytes = std::max(attn_ws_bytes, latent_workspace_bytes(w.spec.heads, w.spec.rotary_key_dim, w.spec.kv_rank, kStackBlockTokens));
+      attn_ws_bytes = std::max(attn_ws_bytes, latent_workspace_bytes(w.spec.heads, w.spec.rotary_key_dim, w.spec.kv_rank, m.block_tokens));
   const uint64_t off_attn_ws = c.take(attn_ws_bytes);
   const uint64_t off_want = c.take(kStackWantedRows * H * es), off_want_rows = c.take(kStackWantedRows * 4ull),
                  off_want_logits = c.take(kStackWantedRows * V * 4ull);

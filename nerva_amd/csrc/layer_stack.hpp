@@ -14,6 +14,10 @@
 
 namespace nv {
 
+// Token rows a block holds at most. Layers of latents and experts take larger ones: an expert sees a few of a block's
+// tokens, and its weights are read once a block whatever it sees.
+constexpr uint32_t kStackBlockTokens = kGemmDeepMaxTokens, kExpertBlockTokens = 2048;
+
 // Tensors of one layer in device memory. Row-concatenated: w_in is [q; k; v; gate] ([q; gate] where the keys are
 // another layer's), [z; candidate; gate] or [query latent; latent and rotated key part; gate].
 struct StackLayer {
@@ -42,6 +46,7 @@ struct StackLayer {
 struct StackModel {
   std::vector<StackLayer> layers;
   uint32_t precision = NERVA_HIP_PRECISION_16;
+  uint32_t block_tokens = kStackBlockTokens;
   uint32_t arrangement = NERVA_HIP_STACK_SANDWICH;
   float embedding_scale = 1.0f, logit_scale = 1.0f;
   const uint16_t *final_w = nullptr, *final_b = nullptr;
@@ -55,7 +60,6 @@ struct StackModel {
   uint32_t table_entries = 0, logical_blocks = 0;
 };
 
-constexpr uint32_t kStackBlockTokens = kGemmDeepMaxTokens;   // token rows a block holds at most
 constexpr uint32_t kStackWantedRows = 32;                    // rows whose logits are computed at a time
 
 hipError_t stack_setup_state(Session *s, int32_t *failure_stage, bool with_weights);

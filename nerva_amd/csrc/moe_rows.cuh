@@ -13,7 +13,7 @@
 
 namespace nv {
 
-constexpr uint32_t kExpertTile = 64;        // slots of a tile
+constexpr uint32_t kExpertTile = 64;        // slots of a tile; twice as many where an expert has enough of them
 constexpr uint32_t kMaxExperts = 1024, kMaxTop = 64;
 
 // Device memory of a block's routing: tokens * top slots, every array sized by moe_plan_bytes.
@@ -23,13 +23,18 @@ struct MoePlan {
   uint32_t *sorted;     // [tokens * top] slots in the order of their experts
   uint4 *tiles;         // (expert, first place in `sorted`, slots, 0)
   uint32_t *tile_count;
+  uint32_t tile;        // slots of a tile
 };
-__host__ inline uint32_t moe_max_tiles(uint32_t tokens, uint32_t top, uint32_t experts) {
+__host__ inline uint32_t expert_tile(uint32_t slots, uint32_t experts) {
+  return slots >= 80u * experts ? 2u * kExpertTile : kExpertTile;
+}
+__host__ inline uint32_t moe_max_tiles(uint32_t tokens, uint32_t top, uint32_t experts, uint32_t tile) {
   const uint32_t slots = tokens * top;
-  return slots / kExpertTile + (experts < slots ? experts : slots);
+  return slots / tile + (experts < slots ? experts : slots);
 }
 uint64_t moe_plan_bytes(uint32_t tokens, uint32_t top, uint32_t experts);
-MoePlan moe_plan_at(void *base, uint32_t tokens, uint32_t top, uint32_t experts);
+// small_tiles: kExpertTile whatever the block holds (f32 rows)
+MoePlan moe_plan_at(void *base, uint32_t tokens, uint32_t top, uint32_t experts, bool small_tiles);
 
 struct MoeRouteRows {
   const float *logits;   // [tokens][experts]

@@ -70,7 +70,7 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(MoeRouteRows p) 
   __syncthreads();
   // exclusive sums over the experts (one each), of slots and of tiles
   static_assert(kMaxExperts == kSortThreads, "one expert a thread");
-  const uint32_t n = count[tid], tiles = (n + kExpertTile - 1) / kExpertTile;
+  const uint32_t size = p.plan.tile, n = count[tid], tiles = (n + size - 1) / size;
   uint32_t a = n, b = tiles;
 #pragma unroll
   for (uint32_t o = 1; o < kWave; o <<= 1) {
@@ -93,7 +93,7 @@ __global__ __launch_bounds__(kSortThreads) void moe_sort_kernel(MoeRouteRows p) 
   tile_at[tid] = b - tiles;
   if (tid == kSortThreads - 1) *p.plan.tile_count = b;
   for (uint32_t i = 0; i < tiles; ++i)
-    p.plan.tiles[b - tiles + i] = make_uint4(tid, a - n + i * kExpertTile, min(kExpertTile, n - i * kExpertTile), 0u);
+    p.plan.tiles[b - tiles + i] = make_uint4(tid, a - n + i * size, min(size, n - i * size), 0u);
   __syncthreads();
   for (uint32_t i = tid; i < slots; i += kSortThreads) {
     const uint32_t at = atomicAdd(&first[min(p.plan.ids[i], p.experts - 1)], 1u);
@@ -121,9 +121,10 @@ struct Products {
 struct Tile {
   uint32_t expert, first, count;
 };
+template <uint32_t TN>
 __device__ __forceinline__ bool tile_of(const Products &p, uint32_t i, Tile &t) {
   if (p.tiles == nullptr) {
-    t = Tile{0u, i * kExpertTile, min(kExpertTile, p.tokens - i * kExpertTile)};
+    t = Tile{0u, i * TN, min(TN, p.tokens - i * TN)};
     return true;
   }
   if (i >= *p.tile_count) return false;
@@ -158,22 +159,24 @@ __device__ __forceinline__ uint4 piece8(const uint16_t *row, uint32_t c, uint32_
   }
 }
 
-template <uint32_t DT, int EPI, bool VEC>
+// TN: slots of a tile.
+template <uint32_t DT, int EPI, bool VEC, uint32_t TN>
 __global__ __launch_bounds__(kBlock) void expert_rows_kernel(Products p) {
   __shared__ __align__(16) uint16_t ws[kRows * kPitch];
-  __shared__ __align__(16) uint16_t xs[kExpertTile * kPitch];
-  __shared__ uint32_t slots[kExpertTile];
+  __shared__ __align__(16) uint16_t xs[TN * kPitch];
+  __shared__ uint32_t slots[TN];
   Tile tile;
-  if (!tile_of(p, blockIdx.y, tile)) return;
+  if (!tile_of<TN>(p, blockIdx.y, tile)) return;
   const uint32_t lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave;
   constexpr uint32_t kOutRows = EPI == kExpertGateUp ? kRows / 2 : kRows;
   const uint32_t row0 = blockIdx.x * kOutRows, cols = p.cols;
-  if (threadIdx.x < kExpertTile) slots[threadIdx.x] = slot_of(p, tile.first + min(threadIdx.x, tile.count - 1));
+  if (threadIdx.x < TN) slots[threadIdx.x] = slot_of(p, tile.first + min(threadIdx.x, tile.count - 1));
   __syncthreads();
   const uint16_t *w = p.w + static_cast<uint64_t>(tile.expert) * (EPI == kExpertGateUp ? 2u : 1u) * p.rows * cols;
-  // staging: thread -> (row of the tile, eight columns), four rows of the matrix and two of the input
+  // staging: thread -> (row of the tile, eight columns), four rows of the matrix, TN / 32 of the input
   const uint32_t sr = threadIdx.x / 8u, sc = (threadIdx.x % 8u) * 8u;
-  const uint16_t *wr[4], *xr[2];
+  constexpr uint32_t XR = TN / 32, JT = TN / 32;   // input rows a thread stages, slot tiles a wave holds
+  const uint16_t *wr[4], *xr[XR];
 #pragma unroll
   for (uint32_t i = 0; i < 4; ++i) {
     const uint32_t r = sr + 32u * i;
@@ -181,50 +184,50 @@ __global__ __launch_bounds__(kBlock) void expert_rows_kernel(Products p) {
     wr[i] = w + static_cast<uint64_t>(row) * cols;
   }
 #pragma unroll
-  for (uint32_t i = 0; i < 2; ++i) xr[i] = p.x16 + static_cast<uint64_t>(input_row<EPI>(p, slots[sr + 32u * i])) * cols;
-  uint4 wq[4], xq[2];
+  for (uint32_t i = 0; i < XR; ++i) xr[i] = p.x16 + static_cast<uint64_t>(input_row<EPI>(p, slots[sr + 32u * i])) * cols;
+  uint4 wq[4], xq[XR];
 #pragma unroll
   for (uint32_t i = 0; i < 4; ++i) wq[i] = piece8<VEC>(wr[i], sc, cols);
 #pragma unroll
-  for (uint32_t i = 0; i < 2; ++i) xq[i] = piece8<VEC>(xr[i], sc, cols);
-  // a wave: 32 gate and the 32 up rows of the same outputs (down: 64 rows), 32 slots
-  f32x4_t acc[4][2];
+  for (uint32_t i = 0; i < XR; ++i) xq[i] = piece8<VEC>(xr[i], sc, cols);
+  // a wave: 32 gate and the 32 up rows of the same outputs (down: 64 rows), half of the slots
+  f32x4_t acc[4][JT];
 #pragma unroll
   for (int a = 0; a < 4; ++a)
 #pragma unroll
-    for (int b = 0; b < 2; ++b) acc[a][b] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+    for (uint32_t b = 0; b < JT; ++b) acc[a][b] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
   const uint32_t n = lane & 15u, q = lane >> 4, half = wave & 1u;
   const auto w_row = [&](uint32_t i) { return EPI == kExpertGateUp ? (i / 2u) * 64u + half * 32u + (i % 2u) * 16u : half * 64u + i * 16u; };
-  const uint16_t *b_at = xs + ((wave >> 1) * 32u + n) * kPitch + q * 8u;
+  const uint16_t *b_at = xs + ((wave >> 1) * (TN / 2) + n) * kPitch + q * 8u;
   for (uint32_t k = 0; k < cols; k += kStep) {
     __syncthreads();
 #pragma unroll
     for (uint32_t i = 0; i < 4; ++i) *reinterpret_cast<uint4 *>(ws + (sr + 32u * i) * kPitch + sc) = wq[i];
 #pragma unroll
-    for (uint32_t i = 0; i < 2; ++i) *reinterpret_cast<uint4 *>(xs + (sr + 32u * i) * kPitch + sc) = xq[i];
+    for (uint32_t i = 0; i < XR; ++i) *reinterpret_cast<uint4 *>(xs + (sr + 32u * i) * kPitch + sc) = xq[i];
     __syncthreads();
     if (k + kStep < cols) {
 #pragma unroll
       for (uint32_t i = 0; i < 4; ++i) wq[i] = piece8<VEC>(wr[i], k + kStep + sc, cols);
 #pragma unroll
-      for (uint32_t i = 0; i < 2; ++i) xq[i] = piece8<VEC>(xr[i], k + kStep + sc, cols);
+      for (uint32_t i = 0; i < XR; ++i) xq[i] = piece8<VEC>(xr[i], k + kStep + sc, cols);
     }
 #pragma unroll
     for (uint32_t s = 0; s < kStep / 32u; ++s) {
-      uint4 a[4], b[2];
+      uint4 a[4], b[JT];
 #pragma unroll
       for (uint32_t i = 0; i < 4; ++i) a[i] = *reinterpret_cast<const uint4 *>(ws + (w_row(i) + n) * kPitch + q * 8u + s * 32u);
 #pragma unroll
-      for (uint32_t j = 0; j < 2; ++j) b[j] = *reinterpret_cast<const uint4 *>(b_at + j * 16u * kPitch + s * 32u);
+      for (uint32_t j = 0; j < JT; ++j) b[j] = *reinterpret_cast<const uint4 *>(b_at + j * 16u * kPitch + s * 32u);
 #pragma unroll
       for (int i = 0; i < 4; ++i)
 #pragma unroll
-        for (int j = 0; j < 2; ++j) acc[i][j] = mfma_k32(a[i], b[j], acc[i][j]);
+        for (uint32_t j = 0; j < JT; ++j) acc[i][j] = mfma_k32(a[i], b[j], acc[i][j]);
     }
   }
 #pragma unroll
-  for (uint32_t j = 0; j < 2; ++j) {
-    const uint32_t t = (wave >> 1) * 32u + j * 16u + n;
+  for (uint32_t j = 0; j < JT; ++j) {
+    const uint32_t t = (wave >> 1) * (TN / 2) + j * 16u + n;
     if (t >= tile.count) continue;
     const uint64_t at = static_cast<uint64_t>(slots[t]) * p.rows;
 #pragma unroll
@@ -247,7 +250,7 @@ __global__ __launch_bounds__(kBlock) void expert_rows_f32_kernel(Products p) {
   __shared__ float ws[M][kStep32][kTile32 + 4], xs[kStep32][kExpertTile + 4];
   __shared__ uint32_t slots[kExpertTile];
   Tile tile;
-  if (!tile_of(p, blockIdx.y, tile)) return;
+  if (!tile_of<kExpertTile>(p, blockIdx.y, tile)) return;
   const uint32_t row0 = blockIdx.x * kTile32, cols = p.cols;
   if (threadIdx.x < kExpertTile) slots[threadIdx.x] = slot_of(p, tile.first + min(threadIdx.x, tile.count - 1));
   __syncthreads();
@@ -305,12 +308,15 @@ hipError_t launch(const ExpertRows &e, hipStream_t stream) {
   p.tokens = e.tokens;
   p.top = e.top;
   p.limit = e.limit;
-  uint32_t tiles = (e.tokens + kExpertTile - 1) / kExpertTile;
+  // (f32 rows: the sort has made small tiles)
+  const uint32_t size = e.plan != nullptr ? e.plan->tile : narrow ? expert_tile(e.tokens, 1) : kExpertTile;
+  if (!narrow && size != kExpertTile) return hipErrorInvalidValue;
+  uint32_t tiles = (e.tokens + size - 1) / size;
   if (e.plan != nullptr) {
     p.tiles = e.plan->tiles;
     p.tile_count = e.plan->tile_count;
     p.sorted = e.plan->sorted;
-    tiles = moe_max_tiles(e.tokens, e.top, e.experts);
+    tiles = moe_max_tiles(e.tokens, e.top, e.experts, size);
   }
   const bool aligned = ((reinterpret_cast<uintptr_t>(p.w) | reinterpret_cast<uintptr_t>(p.x16)) & 15u) == 0;
   if (tiles > 65535u) return hipErrorInvalidValue;
@@ -319,8 +325,11 @@ hipError_t launch(const ExpertRows &e, hipStream_t stream) {
   } else {
     constexpr uint32_t kOutRows = EPI == kExpertGateUp ? kRows / 2 : kRows;
     const dim3 grid((p.rows + kOutRows - 1) / kOutRows, tiles);
-    if (p.cols % 8 == 0 && aligned) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true>), grid, dim3(kBlock), 0, stream, p);
-    else hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, false>), grid, dim3(kBlock), 0, stream, p);
+    const bool large = size != kExpertTile;
+    if (p.cols % 8 == 0 && aligned && large) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true, 2 * kExpertTile>), grid, dim3(kBlock), 0, stream, p);
+    else if (p.cols % 8 == 0 && aligned) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true, kExpertTile>), grid, dim3(kBlock), 0, stream, p);
+    else if (large) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, false, 2 * kExpertTile>), grid, dim3(kBlock), 0, stream, p);
+    else hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, false, kExpertTile>), grid, dim3(kBlock), 0, stream, p);
   }
   return hipGetLastError();
 }
@@ -334,17 +343,18 @@ bool rows_ok(uint32_t dtype, const ExpertRows &p) {
 }  // namespace
 
 uint64_t moe_plan_bytes(uint32_t tokens, uint32_t top, uint32_t experts) {
-  return static_cast<uint64_t>(tokens) * top * 12 + static_cast<uint64_t>(moe_max_tiles(tokens, top, experts)) * sizeof(uint4) + 64;
+  return static_cast<uint64_t>(tokens) * top * 12 + static_cast<uint64_t>(moe_max_tiles(tokens, top, experts, kExpertTile)) * sizeof(uint4) + 64;
 }
 
-MoePlan moe_plan_at(void *base, uint32_t tokens, uint32_t top, uint32_t experts) {
+MoePlan moe_plan_at(void *base, uint32_t tokens, uint32_t top, uint32_t experts, bool small_tiles) {
   const uint64_t slots = static_cast<uint64_t>(tokens) * top;
   MoePlan m;
   m.tiles = static_cast<uint4 *>(base);
-  m.ids = reinterpret_cast<uint32_t *>(m.tiles + moe_max_tiles(tokens, top, experts));
+  m.ids = reinterpret_cast<uint32_t *>(m.tiles + moe_max_tiles(tokens, top, experts, kExpertTile));
   m.weights = reinterpret_cast<float *>(m.ids + slots);
   m.sorted = reinterpret_cast<uint32_t *>(m.weights + slots);
   m.tile_count = m.sorted + slots;
+  m.tile = small_tiles ? kExpertTile : expert_tile(tokens * top, experts);
   return m;
 }
 

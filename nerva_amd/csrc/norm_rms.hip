@@ -1,6 +1,8 @@
 // RMS norm of token rows with the residual sum in front (see norm_rms.cuh).
 #include "norm_rms.cuh"
 
+#include <algorithm>
+
 #include "gemm_rows.cuh"
 
 namespace nv {
@@ -97,7 +99,7 @@ __global__ __launch_bounds__(WG *kWave) void rms_rows_kernel(RmsRows p) {
         store_piece<V>(out.out32 + at, h);
       } else {
         // (four columns stay together in operand order)
-        uint16_t *to = out.out16 + (out.packed_tiles != 0 ? gemm_x_packed_index(out.packed_tiles, row, c) : at);
+        uint16_t *to = out.out16 + (out.packed_tiles != 0 ? gemm_x_block_index(out.packed_tiles, row, c, cols) : at);
         if constexpr (V == 4)
           *reinterpret_cast<uint2 *>(to) = make_uint2(enc16<DT>(h.v[0]) | (static_cast<uint32_t>(enc16<DT>(h.v[1])) << 16),
                                                       enc16<DT>(h.v[2]) | (static_cast<uint32_t>(enc16<DT>(h.v[3])) << 16));
@@ -135,7 +137,7 @@ hipError_t launch_rms_rows(uint32_t dtype, const RmsRows &p, hipStream_t stream)
   if (p.slot_rows != nullptr && (p.slot_weights == nullptr || p.slots == 0)) return hipErrorInvalidValue;
   for (const RmsOut &o : p.out) {
     if (o.gamma != nullptr && (o.out16 == nullptr) == (o.out32 == nullptr)) return hipErrorInvalidValue;
-    if (o.packed_tiles != 0 && (o.packed_tiles * 16u < p.tokens || p.cols % 32 != 0)) return hipErrorInvalidValue;
+    if (o.packed_tiles != 0 && (o.packed_tiles * 16u < std::min(p.tokens, kGemmDeepMaxTokens) || p.cols % 32 != 0)) return hipErrorInvalidValue;
   }
   if (dtype == kBF16) return launch_dt<kBF16>(p, stream);
   return hipErrorInvalidValue;
