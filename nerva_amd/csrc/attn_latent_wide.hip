@@ -4,9 +4,10 @@
 //   absorb  q' = [W_uk^T q_unrotated, rotate(q_rotated)] * scale * log2(e), 16-bit, kv_rank + rot_dim elements a row. W_uk is
 //           read as it lies (rows = contraction) and turned by the transposing LDS reads. A decode step's launch also
 //           writes the token's cache row.
-//   rows    scores, softmax and weighted latents: two waves share 32 rows and walk the keys 32 at a time. Each takes the
-//           scores of 16 rows, their q' in registers for the whole launch, and half the latent columns of the 32 rows'
-//           sums; the weights cross through LDS. The waves of a workgroup share the keys: two cache blocks go from the
+//   rows    scores, softmax and weighted latents: two waves share 32 rows and walk the keys 32 at a time. Each takes
+//           half the elements of the rows' score products, their q' in registers for the whole launch - so that a key
+//           operand read once serves both row tiles - the softmax of 16 rows, and half the latent columns of the 32
+//           rows' sums; partial scores and weights cross through LDS. The waves of a workgroup share the keys: two cache blocks go from the
 //           cache to LDS as they lie (matrix-operand order, global_load_lds, 1 KiB a request), the next two while these
 //           are worked on. The scores read them as operands; for the sums the same bytes are read transposed
 //           (ds_read_b64_tr_b16), keys along the contraction - so a cache row is fetched once for both. Scores come out
@@ -32,7 +33,9 @@ using namespace attn;
 
 constexpr uint32_t kUnitKeys = 2 * kKvBlockTokens;   // keys a step of the rows kernel takes
 constexpr uint32_t kPairRows = 32;
-constexpr size_t kPairExchange = 4096 + 512;
+// [row tile][2 KiB]: the partial scores of the wave that has the row tile ([key tile][lane]), and - once it has read them -
+// the tile's weights as the second product wants them ([hi, lo][lane])
+constexpr size_t kPairExchange = 4096;
 constexpr uint32_t kMostSplits = 128, kBlockSplits = 8, kWorkgroups = 512;   // (two a CU)
 constexpr float kLazy = 8.0f;
 
@@ -153,14 +156,15 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
   constexpr uint32_t DT = kBF16;
   constexpr int D = R + RD, KS = D / 32, DTL = R / 32;        // K-steps of the scores, tiles of 16 latent columns a wave
   constexpr int kTileBytes = 16 * D * 2, kBuf = 2 * kTileBytes, kPieces = kBuf / 1024, kWaves = 2 * PAIRS;
-  static_assert(KS > 2 && DTL % 2 == 0 && D % 32 == 0, "whole groups");
+  constexpr int KH = KS / 2;                                  // ... of a wave
+  static_assert(KS % 2 == 0 && KH > 2 && DTL % 2 == 0 && D % 32 == 0, "whole groups");
   extern __shared__ __align__(16) unsigned char smem[];
   const uint32_t pos0 = p.cursor != nullptr ? *p.cursor : p.position;
   if (p.cursor != nullptr && pos0 >= p.max_steps) return;
   const uint32_t rows = p.tokens * p.heads;
   const uint32_t split = blockIdx.x % splits, row0 = blockIdx.x / splits * (PAIRS * kPairRows);
   const uint32_t lane = threadIdx.x & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
-  const uint32_t pair = wave / 2u, part = wave % 2u;          // part: the wave's row tile in the scores, its columns in the sums
+  const uint32_t pair = wave / 2u, part = wave % 2u;          // part: the wave's elements in the score products, row tile in the softmax, columns in the sums
   const uint32_t n = lane & 15u, q4 = lane >> 4;
   const uint32_t first_token = row0 / p.heads, last_token = (min(row0 + PAIRS * kPairRows, rows) - 1) / p.heads;
   const Units units = units_of(p, pos0, first_token, last_token, splits);
@@ -192,11 +196,12 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
     }
   };
   request(u0, 0);
-  uint4 q[KS];
-  {
-    const uint16_t *src = ws.q16 + static_cast<uint64_t>(min(row, rows - 1)) * D + q4 * 8u;
+  uint4 q[2][KH];   // of both row tiles
 #pragma unroll
-    for (int j = 0; j < KS; ++j) q[j] = *reinterpret_cast<const uint4 *>(src + j * 32);
+  for (int r = 0; r < 2; ++r) {
+    const uint16_t *src = ws.q16 + static_cast<uint64_t>(min(row0 + pair * kPairRows + r * 16u + n, rows - 1)) * D + part * (KH * 32u) + q4 * 8u;
+#pragma unroll
+    for (int j = 0; j < KH; ++j) q[r][j] = *reinterpret_cast<const uint4 *>(src + j * 32);
   }
   float m = -INFINITY, l = 0.0f;
   f32x4_t acc[2][DTL];
@@ -205,45 +210,53 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
 #pragma unroll
     for (int i = 0; i < DTL; ++i) acc[r][i] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
   const uint32_t lds0 = lds_address(smem);
-  const uint32_t k_lane = lds0 + lane * 16u;
-  const uint32_t v_lane = lds0 + ((n % 4u / 2u) * 16u + 4u * q4 + n / 4u) * 16u + (n % 2u) * 8u + part * (DTL * 512u);
-  // exchange of a pair: weights as the second product wants them, [row tile][hi, lo][lane], then factors [row tile][lane]
-  const uint32_t w_at = lds0 + 2 * kBuf + pair * static_cast<uint32_t>(kPairExchange) + lane * 16u;
-  const uint32_t f_at = lds0 + 2 * kBuf + pair * static_cast<uint32_t>(kPairExchange) + 4096u + lane * 4u;
   const uint32_t first_pos = pos0 + first_token, last_lo = window_start(pos0 + last_token, p.window);
 
   // LDS is read and written by hand, operands a group ahead of the products that use them (the compiler would wait for the
   // requests in flight to LDS as well); the awaited registers are in/out operands of the wait.
 #define NV_LR_K(DST, KT, J) asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(DST) : "v"(ka), "n"((KT) * kTileBytes + (J) * 1024) : "memory")
 #define NV_LR_V(DST, KT, T) asm volatile("ds_read_b64_tr_b16 %0, %1 offset:%2" : "=v"(DST) : "v"(va), "n"((KT) * kTileBytes + (T) * 512) : "memory")
-#define NV_LR_WAIT2(N_, B_) asm volatile("s_waitcnt lgkmcnt(" #N_ ")" : "+v"(B_[0]), "+v"(B_[1]) :: "memory")
-#define NV_LR_WAIT(N_, B_) asm volatile("s_waitcnt lgkmcnt(" #N_ ")" : "+v"(B_[0]), "+v"(B_[1]), "+v"(B_[2]), "+v"(B_[3]) :: "memory")
+  // (waits until at most min(LEFT_, MOST_) younger reads are outstanding)
+#define NV_LR_AWAIT(LEFT_, MOST_, ...) asm volatile("s_waitcnt lgkmcnt(%c[n])" : __VA_ARGS__ : [n] "n"((LEFT_) < (MOST_) ? (LEFT_) : (MOST_)) : "memory")
   for (uint32_t u = u0; u < u1; ++u) {
     const uint32_t b = (u - u0) & 1u;
     asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");   // this unit is there, the last one is done with
     if (u + 1 < u1) request(u + 1, b ^ 1u);
-    const uint32_t ka = k_lane + b * kBuf, va = v_lane + b * kBuf;
-    f32x4_t s[2];
+    // addresses, made anew for every unit: kept in registers across the loop they would not fit
+    uint32_t id = lane;
+    asm volatile("" : "+v"(id));
+    const uint32_t ka = lds0 + b * kBuf + part * (KH * 1024u) + id * 16u;
+    f32x4_t part_s[2][2];   // [row tile][key tile]
 #pragma unroll
-    for (int t = 0; t < 2; ++t) s[t] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+    for (int r = 0; r < 2; ++r)
+#pragma unroll
+      for (int t = 0; t < 2; ++t) part_s[r][t] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
     {
-      u32x4_t kq[3][2];   // a K-step of two key tiles
+      u32x4_t kq[5];   // K-step i / 2 of key tile i % 2, four reads ahead
+      constexpr int kReads = 2 * KH;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) NV_LR_K(kq[i >> 1][i & 1], i & 1, i >> 1);
+      for (int i = 0; i < 4; ++i) NV_LR_K(kq[i], i & 1, i >> 1);
 #pragma unroll
-      for (int j = 0; j < KS; ++j) {
-        if (j + 2 < KS) {
+      for (int i = 0; i < kReads; ++i) {
+        if (i + 4 < kReads) NV_LR_K(kq[(i + 4) % 5], i & 1, (i + 4) >> 1);
+        NV_LR_AWAIT(kReads - 1 - i, 4, "+v"(kq[i % 5]));
 #pragma unroll
-          for (int t = 0; t < 2; ++t) NV_LR_K(kq[(j + 2) % 3][t], t, j + 2);
-          NV_LR_WAIT2(4, kq[j % 3]);
-        } else if (j + 1 < KS) {
-          NV_LR_WAIT2(2, kq[j % 3]);
-        } else {
-          NV_LR_WAIT2(0, kq[j % 3]);
-        }
-#pragma unroll
-        for (int t = 0; t < 2; ++t) s[t] = mfma_k32<DT>(__builtin_bit_cast(uint4, kq[j % 3][t]), q[j], s[t]);
+        for (int r = 0; r < 2; ++r) part_s[r][i & 1] = mfma_k32<DT>(__builtin_bit_cast(uint4, kq[i % 5]), q[r][i >> 1], part_s[r][i & 1]);
       }
+    }
+    // the other wave's row tile goes to it, this one's missing half comes back
+    f32x4_t s[2];
+    {
+      const f32x4_t give0 = part != 0 ? part_s[0][0] : part_s[1][0], give1 = part != 0 ? part_s[0][1] : part_s[1][1];
+      // (the products' results are read behind the compiler's back: their latency is waited out here)
+      const uint32_t s_at = lds0 + 2 * kBuf + pair * static_cast<uint32_t>(kPairExchange) + id * 16u;
+      asm volatile("s_nop 15\n\ts_nop 15\n\tds_write_b128 %0, %1\n\tds_write_b128 %0, %2 offset:1024\n\ts_waitcnt lgkmcnt(0)\n\ts_barrier" ::
+                   "v"(s_at + (part ^ 1u) * 2048u), "v"(give0), "v"(give1) : "memory");
+      f32x4_t got0, got1;
+      asm volatile("ds_read_b128 %0, %2\n\tds_read_b128 %1, %2 offset:1024\n\ts_waitcnt lgkmcnt(0)" : "=&v"(got0), "=&v"(got1) :
+                   "v"(s_at + part * 2048u) : "memory");
+      s[0] = (part != 0 ? part_s[1][0] : part_s[0][0]) + got0;
+      s[1] = (part != 0 ? part_s[1][1] : part_s[0][1]) + got1;
     }
     const uint32_t key0 = (units.block0 + 2u * u) * kKvBlockTokens;
     if (key0 < last_lo || key0 + kUnitKeys - 1u > first_pos) {
@@ -265,6 +278,10 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
       m = top;
       l *= keep;
     }
+    // (the factors [row tile][lane] lie where this unit's rotated key elements were: everyone has multiplied them)
+    asm volatile("" : "+v"(id));
+    const uint32_t w_at = lds0 + 2 * kBuf + pair * static_cast<uint32_t>(kPairExchange) + id * 16u;
+    const uint32_t f_at = lds0 + b * kBuf + R / 32 * 1024u + pair * 512u + id * 4u;
     const float ref = m > -INFINITY ? m : 0.0f;   // (a row may not have seen a key yet)
     {
       u32x4_t hi, low;
@@ -283,14 +300,16 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
     }
     asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory");
     u32x4_t w[4];   // [row tile][hi, lo]
+    asm volatile("" : "+v"(id));
+    const uint32_t va = lds0 + b * kBuf + part * (DTL * 512u) + ((id % 4u / 2u) * 16u + id / 16u * 4u + id % 16u / 4u) * 16u + (id % 2u) * 8u;
     float factor[2];
-    u32x2_t vq[2][4];   // a group: two tiles of columns, two key tiles each
+    u32x2_t vq[4][2];   // a tile of columns, two key tiles; three tiles ahead
     asm volatile("ds_read_b32 %0, %2\n\tds_read_b32 %1, %2 offset:256" : "=&v"(factor[0]), "=&v"(factor[1]) : "v"(f_at) : "memory");
 #pragma unroll
     for (int i = 0; i < 4; ++i) asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(w[i]) : "v"(w_at), "n"(i * 1024) : "memory");
 #pragma unroll
-    for (int i = 0; i < 4; ++i) NV_LR_V(vq[0][i], i & 1, i >> 1);
-    asm volatile("s_waitcnt lgkmcnt(4)" : "+v"(factor[0]), "+v"(factor[1]), "+v"(w[0]), "+v"(w[1]), "+v"(w[2]), "+v"(w[3]) :: "memory");
+    for (int i = 0; i < 6; ++i) NV_LR_V(vq[i >> 1][i & 1], i & 1, i >> 1);
+    asm volatile("s_waitcnt lgkmcnt(6)" : "+v"(factor[0]), "+v"(factor[1]), "+v"(w[0]), "+v"(w[1]), "+v"(w[2]), "+v"(w[3]) :: "memory");
     if (__any(factor[0] != 1.0f || factor[1] != 1.0f)) {
 #pragma unroll
       for (int r = 0; r < 2; ++r)
@@ -298,29 +317,22 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
         for (int i = 0; i < DTL; ++i) acc[r][i] *= factor[r];
     }
 #pragma unroll
-    for (int g = 0; g < DTL / 2; ++g) {
-      if (g + 1 < DTL / 2) {
+    for (int c = 0; c < DTL; ++c) {
+      if (c + 3 < DTL) {
 #pragma unroll
-        for (int i = 0; i < 4; ++i) NV_LR_V(vq[(g + 1) & 1][i], i & 1, 2 * (g + 1) + (i >> 1));
-        NV_LR_WAIT(4, vq[g & 1]);
-      } else {
-        NV_LR_WAIT(0, vq[g & 1]);
+        for (int t = 0; t < 2; ++t) NV_LR_V(vq[(c + 3) % 4][t], t, c + 3);
       }
+      NV_LR_AWAIT(2 * (DTL - 1 - c), 6, "+v"(vq[c % 4][0]), "+v"(vq[c % 4][1]));
+      const uint4 a = make_uint4(vq[c % 4][0].x, vq[c % 4][0].y, vq[c % 4][1].x, vq[c % 4][1].y);
 #pragma unroll
-      for (int c = 0; c < 2; ++c) {
-        const u32x2_t a0 = vq[g & 1][2 * c], a1 = vq[g & 1][2 * c + 1];
-        const uint4 a = make_uint4(a0.x, a0.y, a1.x, a1.y);
+      for (int k = 0; k < 2; ++k)
 #pragma unroll
-        for (int k = 0; k < 2; ++k)
-#pragma unroll
-          for (int r = 0; r < 2; ++r) acc[r][2 * g + c] = mfma_k32<DT>(a, __builtin_bit_cast(uint4, w[2 * r + k]), acc[r][2 * g + c]);
-      }
+        for (int r = 0; r < 2; ++r) acc[r][c] = mfma_k32<DT>(a, __builtin_bit_cast(uint4, w[2 * r + k]), acc[r][c]);
     }
   }
 #undef NV_LR_K
 #undef NV_LR_V
-#undef NV_LR_WAIT2
-#undef NV_LR_WAIT
+#undef NV_LR_AWAIT
   // the rows' denominators cross to the wave with their other columns
   float total = l;
   total += __shfl_xor(total, 16, kWave);
