@@ -49,7 +49,7 @@ def _spilling_kernels(remarks):
 # does not know that such a register is still being written, so a spill (or any copy) of it reads garbage:
 # these kernels must compile without scratch memory, which every build checks.
 HAND_ISSUED_LOADS = ("attn_step_kernel", "moe_gate_up_lean_kernel", "moe_down_lean_kernel", "fp8_gemv_lean_kernel",
-                     "gemm_deep_kernel", "latent_rows_kernel", "latent_absorb_kernel")
+                     "gemm_deep_kernel", "latent_rows_kernel", "latent_absorb_kernel", "expert_deep_kernel")
 
 
 def _compile(src):

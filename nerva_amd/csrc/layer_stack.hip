@@ -1138,6 +1138,7 @@ int create_stack(const NervaHipStackSessionCreateRequest *rq, bool synthetic, ui
 
   s->stack = model;
   hipError_t err = latent_wide_setup();
+  if (err == hipSuccess) err = expert_rows_setup();
   if (err == hipSuccess) err = stack_setup_state(s, &out->failure_stage, true);
   uint64_t h2d = 0, syncs = 1;
   if (err == hipSuccess) {

@@ -5,7 +5,8 @@
 // taken in tiles, each a product of the expert's matrix with the gathered rows. The down products leave one row per
 // slot; whoever adds them (norm_rms.cuh) weighs them. One expert that takes every token (a shared one) goes through the
 // same kernels without lists: slot = token.
-//   16-bit rows: matrix cores (v_mfma_f32_16x16x32), both operands through LDS, the next K-step's pieces in registers;
+//   16-bit rows: matrix cores (v_mfma_f32_16x16x32), both operands through LDS: small tiles and odd sizes with the next
+//                K-step's pieces in registers, large tiles of whole steps with requests straight to LDS, two steps ahead;
 //   f32 rows:    vector ALU, every product and sum in f32.
 #pragma once
 
@@ -55,6 +56,7 @@ struct ExpertRows {
   float limit;
   const MoePlan *plan;         // host struct; null: one expert, slot = token (top = experts = 1)
 };
+hipError_t expert_rows_setup();   // once per process, outside stream capture
 hipError_t launch_expert_gate_up(uint32_t dtype, const ExpertRows &p, hipStream_t stream);
 hipError_t launch_expert_down(uint32_t dtype, const ExpertRows &p, hipStream_t stream);
 

@@ -2,6 +2,7 @@
 #include "moe_rows.cuh"
 
 #include <algorithm>
+#include <mutex>
 
 #include "activations.cuh"
 
@@ -242,6 +243,120 @@ __global__ __launch_bounds__(kBlock) void expert_rows_kernel(Products p) {
   }
 }
 
+// Large tiles, whole 64-column steps: 256 matrix rows (gate/up: 128 of each) x 128 slots on eight waves, a wave 64 x 64.
+// Matrix rows and gathered input rows go from global memory to LDS directly (global_load_lds, 1 KiB a request: eight rows
+// of 128 bytes, whose 16-byte pieces are XORed with the row number on the way in - operand reads are then free of bank
+// conflicts), three buffers, two steps ahead; one barrier a step. Operand reads are issued by hand with counted waits (the
+// compiler would wait for the requests in flight as well).
+constexpr uint32_t kDeepRows = 256, kDeepSlots = 2 * kExpertTile, kDeepStep = 64;
+constexpr int kDeepW = kDeepRows * kDeepStep * 2, kDeepX = kDeepSlots * kDeepStep * 2, kDeepBuf = kDeepW + kDeepX;
+typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
+
+template <uint32_t DT, int EPI>
+__global__ __launch_bounds__(8 * kWave, 2) void expert_deep_kernel(Products p, uint32_t row_tiles) {
+  extern __shared__ __align__(16) unsigned char smem[];
+  constexpr uint32_t kOutRows = EPI == kExpertGateUp ? kDeepRows / 2 : kDeepRows;
+  // an XCD takes a run of consecutive (slot tile, row tile) pairs, row tiles fastest: it meets an expert's rows, and a
+  // tile's slots, again while its L2 holds them
+  const uint32_t all = row_tiles * (p.tiles != nullptr ? *p.tile_count : (p.tokens + kDeepSlots - 1) / kDeepSlots), run = (all + 7u) / 8u;
+  const uint32_t at = (blockIdx.x % 8u) * run + blockIdx.x / 8u;
+  if (blockIdx.x / 8u >= run || at >= all) return;
+  Tile tile;
+  if (!tile_of<kDeepSlots>(p, at / row_tiles, tile)) return;
+  const uint32_t row0 = at % row_tiles * kOutRows, cols = p.cols;
+  const uint32_t lane = threadIdx.x & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
+  const uint32_t n = lane & 15u, q = lane >> 4, th = wave & 1u, rq = wave >> 1;
+  const uint16_t *w = p.w + static_cast<uint64_t>(tile.expert) * (EPI == kExpertGateUp ? 2u : 1u) * p.rows * cols;
+  // requests of this wave: 32 rows of the matrix, 16 of the input, eight a request; lane (row, piece)
+  const uint32_t lr = lane >> 3, lc = ((lane & 7u) ^ lr) * 8u;
+  const uint16_t *wsrc[4], *xsrc[2];
+#pragma unroll
+  for (uint32_t i = 0; i < 4; ++i) {
+    const uint32_t r = wave * 32u + i * 8u + lr;
+    const uint32_t row = EPI == kExpertGateUp ? (r / 128u) * p.rows + min(row0 + r % 128u, p.rows - 1) : min(row0 + r, p.rows - 1);
+    wsrc[i] = w + static_cast<uint64_t>(row) * cols + lc;
+  }
+#pragma unroll
+  for (uint32_t i = 0; i < 2; ++i)
+    xsrc[i] = p.x16 + static_cast<uint64_t>(input_row<EPI>(p, slot_of(p, tile.first + min(wave * 16u + i * 8u + lr, tile.count - 1)))) * cols + lc;
+#define NV_ED_LDS(P) ((__attribute__((address_space(3))) void *)(P))
+  const auto request = [&](uint32_t step, uint32_t buffer) {
+    unsigned char *to = smem + buffer * kDeepBuf;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      __builtin_amdgcn_global_load_lds(reinterpret_cast<const uint32_t *>(wsrc[i] + step * kDeepStep), NV_ED_LDS(to + (wave * 4 + i) * 1024), 16, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+      __builtin_amdgcn_global_load_lds(reinterpret_cast<const uint32_t *>(xsrc[i] + step * kDeepStep), NV_ED_LDS(to + kDeepW + (wave * 2 + i) * 1024), 16, 0, 0);
+  };
+  const uint32_t lds0 = static_cast<uint32_t>(reinterpret_cast<uintptr_t>(NV_ED_LDS(smem)));
+#undef NV_ED_LDS
+  // operand addresses of the step's two K-steps: row tile i of the wave at + (gate/up: tiles 0, 1 gate, 2, 3 up) ...
+  uint32_t a_at[2], b_at[2];
+#pragma unroll
+  for (uint32_t e = 0; e < 2; ++e) {
+    const uint32_t piece = ((e * 4u + q) ^ (n & 7u)) << 4;
+    a_at[e] = lds0 + (rq * (EPI == kExpertGateUp ? 32u : 64u) + n) * 128u + piece;
+    b_at[e] = lds0 + kDeepW + (th * 64u + n) * 128u + piece;
+  }
+  constexpr auto a_tile = [](int i) { return EPI == kExpertGateUp ? (i / 2) * 128 * 128 + (i % 2) * 2048 : i * 2048; };
+  f32x4_t acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+  const uint32_t steps = cols / kDeepStep;   // at least two
+  request(0, 0);
+  request(1, 1);
+  uint32_t buffer = 0;
+  for (uint32_t k = 0; k < steps; ++k) {
+    // this step's requests are through (the next step's six may be in flight), nobody reads the last step's any more
+    if (k + 1 < steps) asm volatile("s_waitcnt vmcnt(6) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    else asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)\n\ts_barrier" ::: "memory");
+    if (k + 2 < steps) request(k + 2, buffer == 0 ? 2u : buffer - 1u);
+    const uint32_t off = buffer * kDeepBuf;
+    u32x4_t a[2][4], b[2][4];
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(a[e][i]) : "v"(a_at[e] + off), "n"(a_tile(i)) : "memory");
+#pragma unroll
+      for (int j = 0; j < 4; ++j) asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(b[e][j]) : "v"(b_at[e] + off), "n"(j * 2048) : "memory");
+    }
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+      asm volatile("s_waitcnt lgkmcnt(%c[left])" : "+v"(a[e][0]), "+v"(a[e][1]), "+v"(a[e][2]), "+v"(a[e][3]), "+v"(b[e][0]), "+v"(b[e][1]),
+                   "+v"(b[e][2]), "+v"(b[e][3]) : [left] "n"(8 - 8 * e) : "memory");
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = mfma_k32(__builtin_bit_cast(uint4, a[e][i]), __builtin_bit_cast(uint4, b[e][j]), acc[i][j]);
+    }
+    buffer = buffer == 2 ? 0u : buffer + 1u;
+  }
+#pragma unroll
+  for (uint32_t j = 0; j < 4; ++j) {
+    const uint32_t t = th * 64u + j * 16u + n;
+    if (t >= tile.count) continue;
+    const uint64_t to = static_cast<uint64_t>(slot_of(p, tile.first + t)) * p.rows;
+#pragma unroll
+    for (uint32_t i = 0; i < (EPI == kExpertGateUp ? 2u : 4u); ++i) {
+      const uint32_t row = row0 + rq * (EPI == kExpertGateUp ? 32u : 64u) + i * 16u + q * 4u;
+      if (row >= p.rows) continue;   // (rows are whole groups of four)
+      if constexpr (EPI == kExpertGateUp) {
+        uint32_t o[2];
+#pragma unroll
+        for (int r = 0; r < 2; ++r)
+          o[r] = enc16<DT>(clamped_glu(acc[i][j][2 * r], acc[i + 2][j][2 * r], p.limit)) |
+                 (static_cast<uint32_t>(enc16<DT>(clamped_glu(acc[i][j][2 * r + 1], acc[i + 2][j][2 * r + 1], p.limit))) << 16);
+        *reinterpret_cast<uint2 *>(p.act16 + to + row) = make_uint2(o[0], o[1]);
+      } else {
+        *reinterpret_cast<float4 *>(p.out + to + row) = make_float4(acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]);
+      }
+    }
+  }
+}
+
 constexpr uint32_t kTile32 = 64, kStep32 = 16;   // output rows of a workgroup, columns staged at a time (f32 rows)
 
 template <uint32_t DT, int EPI>
@@ -326,7 +441,14 @@ hipError_t launch(const ExpertRows &e, hipStream_t stream) {
     constexpr uint32_t kOutRows = EPI == kExpertGateUp ? kRows / 2 : kRows;
     const dim3 grid((p.rows + kOutRows - 1) / kOutRows, tiles);
     const bool large = size != kExpertTile;
-    if (p.cols % 8 == 0 && aligned && large) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true, 2 * kExpertTile>), grid, dim3(kBlock), 0, stream, p);
+    if (large && aligned && p.cols % kDeepStep == 0 && p.cols >= 2 * kDeepStep && p.rows % 4 == 0 && (reinterpret_cast<uintptr_t>(p.out) & 15u) == 0 &&
+        (reinterpret_cast<uintptr_t>(p.act16) & 7u) == 0) {
+      constexpr uint32_t kDeepOut = EPI == kExpertGateUp ? kDeepRows / 2 : kDeepRows;
+      const uint32_t row_tiles = (p.rows + kDeepOut - 1) / kDeepOut;
+      const uint64_t most = (static_cast<uint64_t>(row_tiles) * tiles + 7u) / 8u * 8u;
+      if (most > 0x7fffffffu) return hipErrorInvalidValue;
+      hipLaunchKernelGGL((expert_deep_kernel<kBF16, EPI>), dim3(static_cast<uint32_t>(most)), dim3(8 * kWave), 3 * kDeepBuf, stream, p, row_tiles);
+    } else if (p.cols % 8 == 0 && aligned && large) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true, 2 * kExpertTile>), grid, dim3(kBlock), 0, stream, p);
     else if (p.cols % 8 == 0 && aligned) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, true, kExpertTile>), grid, dim3(kBlock), 0, stream, p);
     else if (large) hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, false, 2 * kExpertTile>), grid, dim3(kBlock), 0, stream, p);
     else hipLaunchKernelGGL((expert_rows_kernel<kBF16, EPI, false, kExpertTile>), grid, dim3(kBlock), 0, stream, p);
@@ -356,6 +478,19 @@ MoePlan moe_plan_at(void *base, uint32_t tokens, uint32_t top, uint32_t experts,
   m.tile_count = m.sorted + slots;
   m.tile = small_tiles ? kExpertTile : expert_tile(tokens * top, experts);
   return m;
+}
+
+hipError_t expert_rows_setup() {
+  static std::once_flag once;
+  static hipError_t raised = hipSuccess;
+  std::call_once(once, [] {
+    raised = hipFuncSetAttribute(reinterpret_cast<const void *>(&expert_deep_kernel<kBF16, kExpertGateUp>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                 3 * kDeepBuf);
+    if (raised == hipSuccess)
+      raised = hipFuncSetAttribute(reinterpret_cast<const void *>(&expert_deep_kernel<kBF16, kExpertDown>), hipFuncAttributeMaxDynamicSharedMemorySize,
+                                   3 * kDeepBuf);
+  });
+  return raised;
 }
 
 hipError_t launch_moe_route_rows(const MoeRouteRows &p, hipStream_t stream) {

@@ -274,6 +274,14 @@ def test_wide_layers_take_the_streaming_kernels():
     s.destroy()
 
 
+@pytest.mark.parametrize("sizes", [[700], [400, 90, 80, 2, 1, 127]], ids=str)
+def test_experts_with_many_tokens(sizes):
+    """Blocks in which an expert has enough tokens for the large tiles: whole steps, rows past the last tile, uneven experts."""
+    cfg = M.parallel_config([M.latent(experts=2, top=1, ff=192, limit=1.1, shared=128), M.latent(experts=3, top=2, ff=136, shared=320, shared_limit=0.9),
+                             M.latent(experts=1, top=1, ff=64, shared=0)], width=128)
+    check(cfg, weights(cfg, 24, 0), tokens_of(cfg, 700, seed=9), sizes, 0)
+
+
 def test_greedy_generation_through_the_session_loop():
     """start / advance / run: every token is the plain statement's choice, or within rounding of it."""
     cfg = M.parallel_config(EVERYTHING)
