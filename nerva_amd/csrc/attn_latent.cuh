@@ -68,7 +68,7 @@ hipError_t launch_latent_attention(uint32_t dtype, const LatentAttnParams &p, hi
 bool latent_attention_wide(uint32_t heads, uint32_t key_dim, uint32_t rot_dim, uint32_t value_dim, uint32_t kv_rank);
 uint64_t latent_workspace_bytes(uint32_t heads, uint32_t rot_dim, uint32_t kv_rank, uint32_t max_tokens);
 hipError_t latent_wide_setup();   // once per process, outside stream capture
-hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream);
-uint32_t latent_wide_launches(bool decode);
+// (launches: counted up)
+hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream, uint64_t *launches);
 
 }  // namespace nv

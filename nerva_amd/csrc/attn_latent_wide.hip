@@ -36,7 +36,7 @@ constexpr uint32_t kPairRows = 32;
 // [row tile][2 KiB]: the partial scores of the wave that has the row tile ([key tile][lane]), and - once it has read them -
 // the tile's weights as the second product wants them ([hi, lo][lane])
 constexpr size_t kPairExchange = 4096;
-constexpr uint32_t kMostSplits = 128, kBlockSplits = 8, kWorkgroups = 512;   // (two a CU)
+constexpr uint32_t kMostSplits = 256, kBlockSplits = 8, kWorkgroups = 512;   // (two a CU)
 constexpr float kLazy = 8.0f;
 
 struct Work {
@@ -398,37 +398,117 @@ __device__ __forceinline__ void gated_store(const LatentAttnParams &p, uint32_t 
   *reinterpret_cast<uint2 *>(out) = make_uint2(pack16(o[0] * sigmoid(g[0]), o[1] * sigmoid(g[1])), pack16(o[2] * sigmoid(g[2]), o[3] * sigmoid(g[3])));
 }
 
-// Blocks of token rows. A workgroup: one head, up to 64 value columns, 64 tokens (16 a wave).
+// Blocks of token rows. A workgroup: one head, up to 128 value columns, 128 tokens (32 a wave).
+constexpr uint32_t kValueColumns = 128, kValueTokens = 128;
 __global__ __launch_bounds__(kBlock) void latent_value_kernel(LatentAttnParams p, const uint16_t *o16) {
-  constexpr uint32_t DT = kBF16;
-  const uint32_t R = p.kv_rank, h = blockIdx.y, c0 = blockIdx.x * 64u;
+  constexpr uint32_t DT = kBF16, CT = kValueColumns / 16;
+  const uint32_t R = p.kv_rank, h = blockIdx.y, c0 = blockIdx.x * kValueColumns;
   const uint32_t lane = threadIdx.x & (kWave - 1), wave = threadIdx.x / kWave, n = lane & 15u, q4 = lane >> 4;
-  const uint32_t t = blockIdx.z * 64u + wave * 16u + n;
-  const uint16_t *x = o16 + (static_cast<uint64_t>(min(t, p.tokens - 1)) * p.heads + h) * R + q4 * 8u;
-  const uint16_t *w[4];
+  const uint32_t t0 = blockIdx.z * kValueTokens + wave * 32u + n;
+  const uint16_t *x[2], *w[CT];
 #pragma unroll
-  for (uint32_t i = 0; i < 4; ++i)
+  for (uint32_t j = 0; j < 2; ++j) x[j] = o16 + (static_cast<uint64_t>(min(t0 + j * 16u, p.tokens - 1)) * p.heads + h) * R + q4 * 8u;
+#pragma unroll
+  for (uint32_t i = 0; i < CT; ++i)
     w[i] = p.w_uv + (static_cast<uint64_t>(h) * p.value_dim + min(c0 + i * 16u + n, p.value_dim - 1)) * R + q4 * 8u;
-  f32x4_t acc[4];
+  f32x4_t acc[CT][2];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) acc[i] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll 4
+  for (uint32_t i = 0; i < CT; ++i)
+#pragma unroll
+    for (int j = 0; j < 2; ++j) acc[i][j] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+  uint4 a[CT], b[2];
+#pragma unroll
+  for (uint32_t i = 0; i < CT; ++i) a[i] = *reinterpret_cast<const uint4 *>(w[i]);
+#pragma unroll
+  for (int j = 0; j < 2; ++j) b[j] = *reinterpret_cast<const uint4 *>(x[j]);
   for (uint32_t r = 0; r < R; r += 32) {
-    const uint4 b = *reinterpret_cast<const uint4 *>(x + r);
+    const uint32_t next = r + 32 < R ? r + 32 : r;   // (the last step asks for its own again)
+    uint4 an[CT], bn[2];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) acc[i] = mfma_k32<DT>(*reinterpret_cast<const uint4 *>(w[i] + r), b, acc[i]);
+    for (int j = 0; j < 2; ++j) bn[j] = *reinterpret_cast<const uint4 *>(x[j] + next);
+#pragma unroll
+    for (uint32_t i = 0; i < CT; ++i) an[i] = *reinterpret_cast<const uint4 *>(w[i] + next);
+#pragma unroll
+    for (uint32_t i = 0; i < CT; ++i)
+#pragma unroll
+      for (int j = 0; j < 2; ++j) acc[i][j] = mfma_k32<DT>(a[i], b[j], acc[i][j]);
+#pragma unroll
+    for (uint32_t i = 0; i < CT; ++i) a[i] = an[i];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) b[j] = bn[j];
   }
-  if (t >= p.tokens) return;
 #pragma unroll
-  for (uint32_t i = 0; i < 4; ++i) {
-    const uint32_t c = c0 + i * 16u + 4u * q4;
-    if (c < p.value_dim) gated_store(p, t, h * p.value_dim + c, acc[i]);
+  for (uint32_t j = 0; j < 2; ++j) {
+    const uint32_t t = t0 + j * 16u;
+    if (t >= p.tokens) continue;
+#pragma unroll
+    for (uint32_t i = 0; i < CT; ++i) {
+      const uint32_t c = c0 + i * 16u + 4u * q4;
+      if (c < p.value_dim) gated_store(p, t, h * p.value_dim + c, acc[i][j]);
+    }
   }
 }
 
-// Decode step: merges the splits of one head, then a wave a value column at a time.
+// Factors of a head's splits (those that have left sums) into f_s; the lane's share of the splits' maxima and denominators
+// as they were asked for. Returns 1 / denominator.
+__device__ __forceinline__ float step_factors(float ms, float ls, uint32_t splits, float *f_s, float *red) {
+  const uint32_t tid = threadIdx.x;
+  float top = wave_max(ms);
+  if (tid % kWave == 0) red[tid / kWave] = top;
+  __syncthreads();
+  top = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
+  const float f = ms > -INFINITY ? attn_exp2(ms - top) : 0.0f;
+  if (tid < splits) f_s[tid] = f;
+  return 1.0f / block_sum(ls * f, red);   // (its barriers publish f_s)
+}
+__device__ __forceinline__ uint32_t used_splits(const LatentAttnParams &p, uint32_t pos, uint32_t splits) {
+  const Units u = units_of(p, pos, 0, 0, splits);
+  return (u.count + u.per - 1) / u.per;
+}
+
+// Decode step with many splits: one workgroup per head and 64 latent columns - sixteen lanes a row, sixteen rows at a time;
+// the merged row takes the place of the first split's.
+constexpr uint32_t kMergeColumns = 64, kStepMergeSplits = 32;
+__global__ __launch_bounds__(kBlock) void latent_merge_step_kernel(LatentAttnParams p, uint32_t splits) {
+  __shared__ float f_s[kMostSplits], red[kWavesPerBlock];
+  __shared__ float4 sum_s[kBlock];
+  const uint32_t pos = *p.cursor;
+  if (pos >= p.max_steps) return;
+  const uint32_t R = p.kv_rank, h = blockIdx.y, tid = threadIdx.x, group = tid / 16u, c = blockIdx.x * kMergeColumns + tid % 16u * 4u;
+  const Work ws = work_at(p.workspace, p.heads, R, R + p.rot_dim, splits);
+  const uint64_t base = static_cast<uint64_t>(h) * splits;
+  const uint32_t used = used_splits(p, pos, splits);
+  constexpr uint32_t kEach = kMostSplits / 16u;
+  float4 v[kEach];
+#pragma unroll
+  for (uint32_t i = 0; i < kEach; ++i) v[i] = *reinterpret_cast<const float4 *>(ws.sum + (base + min(group + i * 16u, used - 1)) * R + c);
+  const float inv = step_factors(tid < splits ? ws.m[base + tid] : -INFINITY, tid < splits ? ws.l[base + tid] : 0.0f, splits, f_s, red);
+  float4 o = make_float4(0.0f, 0.0f, 0.0f, 0.0f);
+#pragma unroll
+  for (uint32_t i = 0; i < kEach; ++i) {
+    const float f = group + i * 16u < used ? f_s[group + i * 16u] : 0.0f;
+    o.x = fmaf(v[i].x, f, o.x);
+    o.y = fmaf(v[i].y, f, o.y);
+    o.z = fmaf(v[i].z, f, o.z);
+    o.w = fmaf(v[i].w, f, o.w);
+  }
+  sum_s[tid] = o;
+  __syncthreads();   // (everyone has read its splits, the first one among them)
+  if (group != 0) return;
+#pragma unroll
+  for (uint32_t i = 1; i < 16u; ++i) {
+    const float4 a = sum_s[i * 16u + tid];
+    o.x += a.x;
+    o.y += a.y;
+    o.z += a.z;
+    o.w += a.w;
+  }
+  *reinterpret_cast<float4 *>(ws.sum + base * R + c) = make_float4(o.x * inv, o.y * inv, o.z * inv, o.w * inv);
+}
+
+// Decode step: merges the splits of one head where that has not been done, then a wave a value column at a time.
 constexpr uint32_t kStepColumns = 16;   // value columns of a workgroup
-__global__ __launch_bounds__(kBlock) void latent_value_step_kernel(LatentAttnParams p, uint32_t splits) {
+__global__ __launch_bounds__(kBlock) void latent_value_step_kernel(LatentAttnParams p, uint32_t splits, bool merged) {
   constexpr uint32_t DT = kBF16;
   __shared__ __align__(16) float o_s[kLatentMaxRank];
   __shared__ float f_s[kMostSplits], red[kWavesPerBlock];
@@ -444,26 +524,22 @@ __global__ __launch_bounds__(kBlock) void latent_value_step_kernel(LatentAttnPar
     const uint32_t c = min(blockIdx.x * kStepColumns + wave + i * kWavesPerBlock, p.value_dim - 1);
     w[i] = *reinterpret_cast<const uint4 *>(p.w_uv + (static_cast<uint64_t>(h) * p.value_dim + c) * R + (lane * 8u < R ? lane * 8u : 0u));
   }
-  const float ms = tid < splits ? ws.m[base + tid] : -INFINITY, ls = tid < splits ? ws.l[base + tid] : 0.0f;
-  float top = wave_max(ms);
-  if (lane == 0) red[wave] = top;
-  __syncthreads();
-  top = fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3]));
-  const float f = ms > -INFINITY ? attn_exp2(ms - top) : 0.0f;
-  if (tid < splits) f_s[tid] = f;
-  const float inv = 1.0f / block_sum(ls * f, red);   // (its barriers publish f_s)
-  const uint32_t active = units_of(p, pos, 0, 0, splits).count, per = units_of(p, pos, 0, 0, splits).per;
-  const uint32_t used = (active + per - 1) / per;    // the splits that have left sums
-  for (uint32_t c = tid * 2u; c < R; c += kBlock * 2u) {
-    float2 o = make_float2(0.0f, 0.0f);
+  if (merged) {
+    for (uint32_t c = tid * 2u; c < R; c += kBlock * 2u) *reinterpret_cast<float2 *>(o_s + c) = *reinterpret_cast<const float2 *>(ws.sum + base * R + c);
+  } else {
+    const float inv = step_factors(tid < splits ? ws.m[base + tid] : -INFINITY, tid < splits ? ws.l[base + tid] : 0.0f, splits, f_s, red);
+    const uint32_t used = used_splits(p, pos, splits);
+    for (uint32_t c = tid * 2u; c < R; c += kBlock * 2u) {
+      float2 o = make_float2(0.0f, 0.0f);
 #pragma unroll 16
-    for (uint32_t i = 0; i < used; ++i) {
-      const float2 v = *reinterpret_cast<const float2 *>(ws.sum + (base + i) * R + c);
-      o.x = fmaf(v.x, f_s[i], o.x);
-      o.y = fmaf(v.y, f_s[i], o.y);
+      for (uint32_t i = 0; i < used; ++i) {
+        const float2 v = *reinterpret_cast<const float2 *>(ws.sum + (base + i) * R + c);
+        o.x = fmaf(v.x, f_s[i], o.x);
+        o.y = fmaf(v.y, f_s[i], o.y);
+      }
+      o_s[c] = o.x * inv;
+      o_s[c + 1] = o.y * inv;
     }
-    o_s[c] = o.x * inv;
-    o_s[c + 1] = o.y * inv;
   }
   __syncthreads();
 #pragma unroll
@@ -508,7 +584,7 @@ hipError_t launch_rows(const LatentAttnParams &p, uint32_t splits, hipStream_t s
 }
 
 template <int R, int RD>
-hipError_t launch_shape(const LatentAttnParams &p, hipStream_t stream) {
+hipError_t launch_shape(const LatentAttnParams &p, hipStream_t stream, uint64_t *launches) {
   const bool step = p.cursor != nullptr;
   const uint32_t rows = p.tokens * p.heads, splits = step ? step_splits(p) : block_splits(rows);
   const Work ws = work_at(p.workspace, rows, R, R + RD, splits);
@@ -520,15 +596,25 @@ hipError_t launch_shape(const LatentAttnParams &p, hipStream_t stream) {
   err = rows > kPairRows ? launch_rows<R, RD, 2>(p, splits, stream) : launch_rows<R, RD, 1>(p, splits, stream);
   if (err != hipSuccess) return err;
   if (step) {
-    hipLaunchKernelGGL(latent_value_step_kernel, dim3((p.value_dim + kStepColumns - 1) / kStepColumns, p.heads), dim3(kBlock), 0, stream, p, splits);
+    const bool merged = splits > kStepMergeSplits;
+    *launches += merged ? 4 : 3;
+    if (merged) {
+      hipLaunchKernelGGL(latent_merge_step_kernel, dim3(R / kMergeColumns, p.heads), dim3(kBlock), 0, stream, p, splits);
+      err = hipGetLastError();
+      if (err != hipSuccess) return err;
+    }
+    hipLaunchKernelGGL(latent_value_step_kernel, dim3((p.value_dim + kStepColumns - 1) / kStepColumns, p.heads), dim3(kBlock), 0, stream, p, splits,
+                       merged);
     return hipGetLastError();
   }
+  *launches += splits > 1 ? 4 : 3;
   if (splits > 1) {
     hipLaunchKernelGGL(latent_merge_kernel, dim3(rows), dim3(kBlock), 0, stream, p, splits);
     err = hipGetLastError();
     if (err != hipSuccess) return err;
   }
-  hipLaunchKernelGGL(latent_value_kernel, dim3((p.value_dim + 63) / 64, p.heads, token_tiles), dim3(kBlock), 0, stream, p,
+  hipLaunchKernelGGL(latent_value_kernel, dim3((p.value_dim + kValueColumns - 1) / kValueColumns, p.heads, (p.tokens + kValueTokens - 1) / kValueTokens),
+                     dim3(kBlock), 0, stream, p,
                      static_cast<const uint16_t *>(ws.o16));
   return hipGetLastError();
 }
@@ -571,9 +657,7 @@ hipError_t latent_wide_setup() {
   return raised;
 }
 
-uint32_t latent_wide_launches(bool decode) { return decode ? 3u : 4u; }
-
-hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream) {
+hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &p, hipStream_t stream, uint64_t *launches) {
   const auto aligned = [](const void *q, uintptr_t n) { return (reinterpret_cast<uintptr_t>(q) & (n - 1)) == 0; };
   if (dtype != kBF16 || !latent_attention_wide(p.heads, p.key_dim, p.rot_dim, p.value_dim, p.kv_rank) || p.cache32 != 0 || p.out16 == nullptr ||
       p.workspace == nullptr || p.proj == nullptr || p.q == nullptr || p.w_uk == nullptr || p.w_uv == nullptr || p.cache == nullptr ||
@@ -583,9 +667,9 @@ hipError_t launch_latent_attention_wide(uint32_t dtype, const LatentAttnParams &
   if (!aligned(p.workspace, 256) || !aligned(p.cache, 16) || !aligned(p.w_uk, 16) || !aligned(p.w_uv, 16) || !aligned(p.q, 16) || !aligned(p.out16, 16))
     return hipErrorInvalidValue;
   if (p.cursor != nullptr ? p.tokens != 1 : (p.position + p.tokens - 1) / kKvBlockTokens > p.last_block) return hipErrorInvalidValue;
-  if (p.kv_rank == 512) return launch_shape<512, 64>(p, stream);
-  if (p.kv_rank == 256) return launch_shape<256, 64>(p, stream);
-  return launch_shape<128, 64>(p, stream);
+  if (p.kv_rank == 512) return launch_shape<512, 64>(p, stream, launches);
+  if (p.kv_rank == 256) return launch_shape<256, 64>(p, stream, launches);
+  return launch_shape<128, 64>(p, stream, launches);
 }
 
 }  // namespace nv

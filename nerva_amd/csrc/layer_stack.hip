@@ -353,7 +353,7 @@ hipError_t parallel_step_16(Session *s) {
     const bool fast = takes_latent_wide(s, d);
     if (!fast) a.q_latent16 = static_cast<uint16_t *>(s->pql);   // (the middle launch has its own)
     if (err == hipSuccess && !fast) err = launch_latent_prepare(s->dtype, a, st);
-    if (err == hipSuccess) err = fast ? launch_latent_attention_wide(s->dtype, a, st) : launch_latent_attention(s->dtype, a, st);
+    if (err == hipSuccess) err = fast ? launch_latent_attention_wide(s->dtype, a, st, &launches) : launch_latent_attention(s->dtype, a, st);
     LayerBack b{};
     b.x = s->x;
     b.hidden = s->hidden;
@@ -372,7 +372,7 @@ hipError_t parallel_step_16(Session *s) {
     b.cursor = s->state;
     b.max_steps = s->max_ctx;
     if (err == hipSuccess) err = launch_layer_back(s->dtype, b, st);
-    launches += 3 + (fast ? latent_wide_launches(true) : 2u);
+    launches += 3 + (fast ? 0 : 2);
   }
   s->stack_launches = launches + (s->sampler.mode == kSamplerGreedy ? 2 : 3);
   DecodeRow row{s->x, nullptr, Seam{}};
@@ -531,8 +531,8 @@ struct Block {
       err = launch_latent_prepare(s->dtype, a, s->stream);
       if (err == hipSuccess) err = project(kGemmF32, w.w_uq, w.q_rows(), w.spec.q_rank, s->pql, q_tiles, s->pq, 0, nullptr);
       const bool fast = takes_latent_wide(s, w.spec);
-      if (err == hipSuccess) err = fast ? launch_latent_attention_wide(s->dtype, a, s->stream) : launch_latent_attention(s->dtype, a, s->stream);
-      launches += fast ? latent_wide_launches(at_cursor) : 1u;
+      if (err == hipSuccess) err = fast ? launch_latent_attention_wide(s->dtype, a, s->stream, &launches) : launch_latent_attention(s->dtype, a, s->stream);
+      launches += fast ? 0 : 1;
     } else if (w.spec.mixer == NERVA_HIP_MIXER_ATTENTION) {
       MixedAttnParams a = attention_params(s, w, s->pqkv, s->prope);
       a.position = first;
