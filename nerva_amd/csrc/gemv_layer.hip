@@ -227,96 +227,78 @@ __global__ __launch_bounds__(kThreads, 4) void layer_middle_kernel(LayerMiddle p
 
 // ---- back ------------------------------------------------------------------------------------
 
-// A run of a row's columns: weights at base + row * stride, `cols` of them meet the staged inputs from `at` on.
-struct Run {
-  const uint16_t *base;
-  uint32_t stride, cols, at;
+// A row's columns are the pieces' columns one after the other, each piece padded to whole chunks, as their inputs lie in
+// LDS. A chunk: where it starts in row 0, bytes from row to row, lanes that have columns, what its products are worth.
+struct Chunk {
+  uint64_t base;
+  uint16_t stride, lanes;
   float factor;
 };
-constexpr uint32_t kMaxRuns = kMaxTop + 2;
+static_assert(sizeof(Chunk) == 16, "one LDS read");
+constexpr uint32_t kMaxChunks = kMaxLds / (2 * kChunk);
 constexpr int kBackBatch = 8;   // chunks of a request batch
 
 template <uint32_t DT>
 __global__ __launch_bounds__(kThreads, 4) void layer_back_kernel(LayerBack p) {
-  extern __shared__ __align__(16) uint16_t xs[];   // the runs' inputs, each padded to whole chunks
-  __shared__ Run runs[kMaxRuns];
+  extern __shared__ __align__(16) uint16_t xs[];   // the pieces' inputs
+  __shared__ __align__(16) Chunk table[kMaxChunks + kBackBatch];
   if (*p.cursor >= p.max_steps) return;
   const uint32_t tid = threadIdx.x, lane = tid & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(tid / kWave);
-  const uint32_t n_runs = 1u + p.top + (p.shared_ff != 0 ? 1u : 0u);
   const uint32_t expert_at = padded(p.mix_cols), shared_at = expert_at + p.top * padded(p.ff);
-  if (tid < n_runs) {
-    if (tid == 0) runs[tid] = Run{p.w_o, p.mix_cols, p.mix_cols, 0u, 1.0f};
-    else if (tid <= p.top)
-      runs[tid] = Run{p.e_out + static_cast<uint64_t>(p.ids[tid - 1]) * p.hidden * p.ff, p.ff, p.ff, expert_at + (tid - 1) * padded(p.ff), p.weights[tid - 1]};
-    else runs[tid] = Run{p.shared_out, p.shared_ff, p.shared_ff, shared_at, 1.0f};
+  const uint32_t chunks = (shared_at + padded(p.shared_ff)) / kChunk, batches = (chunks + kBackBatch - 1) / kBackBatch;
+  if (tid < batches * kBackBatch) {
+    const uint32_t at = tid * kChunk;
+    const uint16_t *base = p.w_o;
+    uint32_t cols = p.mix_cols, c = at;
+    float factor = 1.0f;
+    if (at >= shared_at) {
+      base = p.shared_out;
+      cols = p.shared_ff;
+      c = at - shared_at;
+    } else if (at >= expert_at) {
+      const uint32_t k = (at - expert_at) / padded(p.ff);
+      base = p.e_out + static_cast<uint64_t>(p.ids[k]) * p.hidden * p.ff;
+      cols = p.ff;
+      c = at - expert_at - k * padded(p.ff);
+      factor = p.weights[k];
+    }
+    const uint32_t lanes = tid < chunks ? min((cols - c) / 8u, static_cast<uint32_t>(kWave)) : 0u;   // (the last batch's chunks past the end)
+    table[tid] = Chunk{reinterpret_cast<uint64_t>(base) + 2u * (lanes != 0 ? c : 0u), static_cast<uint16_t>(2u * cols), static_cast<uint16_t>(lanes), factor};
   }
   __syncthreads();
-  const uint32_t chunks = (shared_at + padded(p.shared_ff)) / kChunk;
-  // The row's chunks lie one after the other as their inputs do. Cursors over them (wave-uniform): run, column in it.
-  struct Cursor {
-    const uint16_t *base;
-    uint32_t run, c, cols;
-    float factor;
-  };
-  const auto open = [&](Cursor &k, uint32_t run, uint32_t row) {
-    const Run &r = runs[run];
-    const uint64_t base = reinterpret_cast<uint64_t>(r.base) + static_cast<uint64_t>(row) * r.stride * 2u;
-    // (the builtin returns a signed word: narrowed again before it is widened to an address)
-    const uint32_t low = __builtin_amdgcn_readfirstlane(static_cast<uint32_t>(base)), high = __builtin_amdgcn_readfirstlane(static_cast<uint32_t>(base >> 32));
-    k.base = reinterpret_cast<const uint16_t *>(static_cast<uint64_t>(low) | static_cast<uint64_t>(high) << 32);
-    k.run = run;
-    k.c = 0;
-    k.cols = __builtin_amdgcn_readfirstlane(r.cols);
-    k.factor = r.factor;
-  };
-  const uint32_t stride = gridDim.x * kWaves, batches = (chunks + kBackBatch - 1) / kBackBatch;
+  const uint32_t stride = gridDim.x * kWaves;
   uint4 b0[kBackBatch], b1[kBackBatch];
   uint32_t irow = wave * gridDim.x + blockIdx.x, ib = 0, crow = irow, cb = 0;
-  Cursor in{}, cur{};
-  if (irow < p.hidden) {
-    open(in, 0, irow);
-    open(cur, 0, irow);
-  }
-  float acc = 0.0f, total = 0.0f;
-  const auto next = [&](Cursor &k, uint32_t row) {   // one chunk further
-    k.c += kChunk;
-    if (k.c >= k.cols && k.run + 1 < n_runs) open(k, k.run + 1, row);
+  float total = 0.0f;
+  const auto issue = [&](uint4 (&to)[kBackBatch]) {
+    if (irow >= p.hidden) return;
+#pragma unroll
+    for (int u = 0; u < kBackBatch; ++u) {
+      const Chunk k = table[ib * kBackBatch + u];
+      to[u] = make_uint4(0u, 0u, 0u, 0u);
+      if (lane < k.lanes) to[u] = load_stream(reinterpret_cast<const char *>(k.base) + static_cast<uint64_t>(irow) * k.stride + lane * 16u);
+    }
+    if (++ib == batches) {
+      ib = 0;
+      irow += stride;
+    }
   };
-#define NV_BACK_ISSUE(DST)                                                                           \
-  if (irow < p.hidden) {                                                                            \
-    _Pragma("unroll") for (int u = 0; u < kBackBatch; ++u) {                                        \
-      const uint32_t c = in.c + lane * 8u;                                                          \
-      DST[u] = ib * kBackBatch + u < chunks && c < in.cols ? load_stream(in.base + c) : make_uint4(0u, 0u, 0u, 0u); \
-      if (ib * kBackBatch + u + 1 < chunks) next(in, irow);                                         \
-    }                                                                                               \
-    if (++ib == batches) {                                                                          \
-      ib = 0;                                                                                       \
-      irow += stride;                                                                               \
-      if (irow < p.hidden) open(in, 0, irow);                                                       \
-    }                                                                                               \
-  }
-#define NV_BACK_CONSUME(SRC)                                                                         \
-  _Pragma("unroll") for (int u = 0; u < kBackBatch; ++u) {                                          \
-    if (cb * kBackBatch + u < chunks) {                                                             \
-      const uint4 x = *reinterpret_cast<const uint4 *>(xs + (cb * kBackBatch + u) * kChunk + lane * 8u); \
-      acc = dot8<DT, true>(SRC[u], x, acc);                                                         \
-      if (cur.c + kChunk >= cur.cols) {                                                             \
-        total = fmaf(cur.factor, acc, total);                                                       \
-        acc = 0.0f;                                                                                 \
-      }                                                                                             \
-      if (cb * kBackBatch + u + 1 < chunks) next(cur, crow);                                        \
-    }                                                                                               \
-  }                                                                                                 \
-  if (++cb == batches) {                                                                            \
-    total = wave_sum(total);                                                                        \
-    if (lane == 0) p.x[crow] += total;                                                              \
-    total = 0.0f;                                                                                   \
-    cb = 0;                                                                                         \
-    crow += stride;                                                                                 \
-    if (crow < p.hidden) open(cur, 0, crow);                                                        \
-  }
-  NV_BACK_ISSUE(b0)
-  NV_BACK_ISSUE(b1)
+  const auto consume = [&](const uint4 (&from)[kBackBatch]) {
+#pragma unroll
+    for (int u = 0; u < kBackBatch; ++u) {
+      const uint32_t i = cb * kBackBatch + u;
+      if (i < chunks) total = fmaf(table[i].factor, dot8<DT, true>(from[u], *reinterpret_cast<const uint4 *>(xs + i * kChunk + lane * 8u), 0.0f), total);
+    }
+    if (++cb < batches) return;
+    total = wave_sum(total);
+    if (lane == 0) p.x[crow] += total;
+    total = 0.0f;
+    cb = 0;
+    crow += stride;
+  };
+  issue(b0);
+  issue(b1);
+  // the inputs, under the first requests
   const auto stage = [&](const uint16_t *src, uint32_t cols, uint32_t at) {
     for (uint32_t c = tid * 8u; c < cols; c += kThreads * 8u) *reinterpret_cast<uint4 *>(xs + at + c) = *reinterpret_cast<const uint4 *>(src + c);
     clear_tail(xs + at, cols);
@@ -326,14 +308,12 @@ __global__ __launch_bounds__(kThreads, 4) void layer_back_kernel(LayerBack p) {
   if (p.shared_ff != 0) stage(p.shared_act, p.shared_ff, shared_at);
   __syncthreads();
   while (crow < p.hidden) {
-    NV_BACK_CONSUME(b0)
-    NV_BACK_ISSUE(b0)
+    consume(b0);
+    issue(b0);
     if (crow >= p.hidden) break;
-    NV_BACK_CONSUME(b1)
-    NV_BACK_ISSUE(b1)
+    consume(b1);
+    issue(b1);
   }
-#undef NV_BACK_ISSUE
-#undef NV_BACK_CONSUME
 }
 
 uint32_t workgroups(uint32_t units) { return std::max(1u, std::min(kMaxWorkgroups, (units + kWaves - 1) / kWaves)); }
