@@ -159,16 +159,23 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
   constexpr int KH = KS / 2;                                  // ... of a wave
   static_assert(KS % 2 == 0 && KH > 2 && DTL % 2 == 0 && D % 32 == 0, "whole groups");
   extern __shared__ __align__(16) unsigned char smem[];
-  const uint32_t pos0 = p.cursor != nullptr ? *p.cursor : p.position;
-  if (p.cursor != nullptr && pos0 >= p.max_steps) return;
   const uint32_t rows = p.tokens * p.heads;
   const uint32_t split = blockIdx.x % splits, row0 = blockIdx.x / splits * (PAIRS * kPairRows);
   const uint32_t lane = threadIdx.x & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(threadIdx.x / kWave);
   const uint32_t pair = wave / 2u, part = wave % 2u;          // part: the wave's elements in the score products, row tile in the softmax, columns in the sums
   const uint32_t n = lane & 15u, q4 = lane >> 4;
+  const Work ws = work_at(p.workspace, rows, R, D, splits);
+  uint4 q[2][KH];   // of both row tiles; requested ahead of everything that depends on the position
+#pragma unroll
+  for (int r = 0; r < 2; ++r) {
+    const uint16_t *src = ws.q16 + static_cast<uint64_t>(min(row0 + pair * kPairRows + r * 16u + n, rows - 1)) * D + part * (KH * 32u) + q4 * 8u;
+#pragma unroll
+    for (int j = 0; j < KH; ++j) q[r][j] = *reinterpret_cast<const uint4 *>(src + j * 32);
+  }
+  const uint32_t pos0 = p.cursor != nullptr ? *p.cursor : p.position;
+  if (p.cursor != nullptr && pos0 >= p.max_steps) return;
   const uint32_t first_token = row0 / p.heads, last_token = (min(row0 + PAIRS * kPairRows, rows) - 1) / p.heads;
   const Units units = units_of(p, pos0, first_token, last_token, splits);
-  const Work ws = work_at(p.workspace, rows, R, D, splits);
   const uint32_t u0 = split * units.per, u1 = min(u0 + units.per, units.count);
   const uint32_t row = row0 + pair * kPairRows + part * 16u + n, pos = pos0 + min(row, rows - 1) / p.heads, lo = window_start(pos, p.window);
   if (u0 >= u1) {   // a split without keys
@@ -196,13 +203,6 @@ __global__ __launch_bounds__(2 * PAIRS * kWave, 2) void latent_rows_kernel(Laten
     }
   };
   request(u0, 0);
-  uint4 q[2][KH];   // of both row tiles
-#pragma unroll
-  for (int r = 0; r < 2; ++r) {
-    const uint16_t *src = ws.q16 + static_cast<uint64_t>(min(row0 + pair * kPairRows + r * 16u + n, rows - 1)) * D + part * (KH * 32u) + q4 * 8u;
-#pragma unroll
-    for (int j = 0; j < KH; ++j) q[r][j] = *reinterpret_cast<const uint4 *>(src + j * 32);
-  }
   float m = -INFINITY, l = 0.0f;
   f32x4_t acc[2][DTL];
 #pragma unroll
