@@ -210,7 +210,7 @@ def main():
     ap.add_argument("--copy-probe-mib", type=int, default=0,
                     help="also launch one plain copy kernel of this size (memory-counter calibration runs)")
     ap.add_argument("--stack", nargs="?", const="all", default=None, metavar="SIZE",
-                    help="instead of the workload: a mixed layer stack beside the uniform decoder, at one size of "
+                    help="instead of the workload: mixed layer stacks beside the uniform decoder, at one size of "
                          "nerva_amd/stackbench.py or at all of them")
     args = ap.parse_args()
     if args.gpus != 1:

@@ -7,15 +7,15 @@
 //   rows    scores, softmax and weighted latents: two waves share 32 rows and walk the keys 32 at a time. Each takes
 //           half the elements of the rows' score products, their q' in registers for the whole launch - so that a key
 //           operand read once serves both row tiles - the softmax of 16 rows, and half the latent columns of the 32
-//           rows' sums; partial scores and weights cross through LDS. The waves of a workgroup share the keys: two cache blocks go from the
-//           cache to LDS as they lie (matrix-operand order, global_load_lds, 1 KiB a request), the next two while these
-//           are worked on. The scores read them as operands; for the sums the same bytes are read transposed
-//           (ds_read_b64_tr_b16), keys along the contraction - so a cache row is fetched once for both. Scores come out
-//           with a lane's keys in the order the second product wants its weights in; weights enter as hi + lo 16-bit
-//           halves. A running maximum is moved only when a score passes it by more than 8 (log2), so the sums are
-//           rarely rescaled.
-//   merge   splits of the key range into one row (blocks of token rows with few rows), or
-//   value   o = sigmoid(gate) * W_uv (weighted latents); a decode step's launch merges the splits itself.
+//           rows' sums; partial scores and weights cross through LDS. The waves of a workgroup share the keys: two
+//           cache blocks go from the cache to LDS as they lie (matrix-operand order, global_load_lds, 1 KiB a request),
+//           the next two while these are worked on. The scores read them as operands; for the sums the same bytes are
+//           read transposed (ds_read_b64_tr_b16), keys along the contraction - so a cache row is fetched once for both.
+//           Scores come out with a lane's keys in the order the second product wants its weights in; weights enter as
+//           hi + lo 16-bit halves. A running maximum is moved only when a score passes it by more than 8 (log2), so the
+//           sums are rarely rescaled.
+//   merge   splits of the key range into one row, where there are any (decode steps: where there are many)
+//   value   o = sigmoid(gate) * W_uv (weighted latents); a decode step's launch merges few splits itself.
 #include <algorithm>
 #include <mutex>
 
@@ -468,7 +468,7 @@ __device__ __forceinline__ uint32_t used_splits(const LatentAttnParams &p, uint3
 
 // Decode step with many splits: one workgroup per head and 64 latent columns - sixteen lanes a row, sixteen rows at a time;
 // the merged row takes the place of the first split's.
-constexpr uint32_t kMergeColumns = 64, kStepMergeSplits = 32;
+constexpr uint32_t kMergeColumns = 64, kStepMergeSplits = 48;
 __global__ __launch_bounds__(kBlock) void latent_merge_step_kernel(LatentAttnParams p, uint32_t splits) {
   __shared__ float f_s[kMostSplits], red[kWavesPerBlock];
   __shared__ float4 sum_s[kBlock];

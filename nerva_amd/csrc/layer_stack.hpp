@@ -2,9 +2,12 @@
 // The session object, its lifecycle, sampler, slots and graphs are decode_session.hip's; here are the weights' layout,
 // the cache and state of such a stack, and its two ways through the layers:
 //   a decode step (16-bit precision): per sublayer a weight-streaming GEMV whose prologue is the seam between the
-//     sublayers and whose epilogue is the activation or the recurrence (gemv_stream.cuh), attention in between;
-//   blocks of token rows (prompts, portions, and every step of a 32-bit session): the seam, projections, attention or
-//     scan, projection - row kernels, the projections on the streaming multi-row kernels where a shape has one.
+//     sublayers and whose epilogue is the activation or the recurrence (gemv_stream.cuh), attention in between; in
+//     parallel layers of attention over latents and experts what does not wait for each other shares a launch
+//     (gemv_layer.cuh);
+//   blocks of token rows (prompts, portions, every step of a 32-bit session, and steps of layers the above does not
+//     take): norms, projections, attention or scan, projection, experts - row kernels, the projections on the streaming
+//     multi-row kernels where a shape has one.
 #pragma once
 
 #include <memory>
